@@ -8,7 +8,7 @@ KvBufferCache.java:826-841,851-865); there is no pool with a limit and nothing i
 between requests.  Here a pool of fixed size serves all requests:
 
 * A *group* is a set of cache slots (one per caching layer call) with the same needs: all
-  keys, or a window of the last w.  Each group has pages of its own; one page id names the
+  keys, a window of the last w, or the chunk of c positions that the next one lies in.  Each group has pages of its own; one page id names the
   same page in every slot of the group.
 * A request's *block table* for a group lists the page of each run of ``page_size``
   positions; the entry is -1 once a window has passed that run and the page went back
@@ -36,12 +36,14 @@ class OutOfPages(CacheError):
 @dataclass(frozen=True)
 class KVGroupSpec:
     """Cache slots that share pages.  ``window`` None keeps every key; with a window, the pages that hold
-    a request's first ``keep_first`` positions are never given back while it lives."""
+    a request's first ``keep_first`` positions are never given back while it lives.  With ``chunk`` (in place of a
+    window) a position sees keys of its own chunk of so many positions only, counted from the sequence's start."""
     slots: Tuple[int, ...]
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     keep_first: int = 0
+    chunk: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -162,7 +164,9 @@ class CacheManager:
     # ---- pages -------------------------------------------------------------------
     def _first_live_page(self, group: int, first_query_pos: int) -> int:
         """Index of the first page a query at ``first_query_pos`` or later can still see."""
-        w = self.groups[group].window
+        w, c = self.groups[group].window, self.groups[group].chunk
+        if c is not None:
+            return (first_query_pos // c * c) // self.page_size
         if w is None:
             return 0
         lo = max(0, first_query_pos - w + 1)

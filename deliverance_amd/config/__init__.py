@@ -5,7 +5,9 @@ from .virudra import VirudraConfig
 from .pedatar import PedatarConfig
 from .pafolorn import PafolornConfig
 from .salivik import SalivikConfig
+from .luvatar import LuvatarConfig
 from .engine_config import EngineConfig
 
 __all__ = ["AttentionSpec", "ConfigError", "DenseFeedForwardSpec", "LayerCall", "LayerSpec",
-           "ModelConfig", "NormSpec", "PositionSpec", "Gpt2Config", "VirudraConfig", "PedatarConfig", "PafolornConfig", "SalivikConfig", "EngineConfig"]
+           "ModelConfig", "NormSpec", "PositionSpec", "Gpt2Config", "VirudraConfig", "PedatarConfig", "PafolornConfig", "SalivikConfig", "LuvatarConfig",
+           "EngineConfig"]

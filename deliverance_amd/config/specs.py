@@ -106,6 +106,12 @@ class AttentionSpec:
     # the heads' results are multiplied, element by element, with this function of one more projection of the
     # mixer's input before the output projection: None or "sigmoid" (parameter ``gate_weight`` [heads * value size, width])
     out_gate: Optional[str] = None
+    # positions are cut into chunks of so many, counted from a sequence's start, and a row sees the earlier keys of its
+    # own chunk only (instead of a window)
+    chunk: Optional[int] = None
+    # no keys and values of its own: the run order gives this layer another layer's cache slot to read (``write`` off);
+    # there is no key or value matrix, no key gain, and heads, sizes and rotation are the other layer's
+    shared_kv: bool = False
 
     @property
     def value_dim(self) -> int:
@@ -126,16 +132,23 @@ class RampedSpeedsSpec:
 
 
 @dataclass(frozen=True)
+class LinearSpeedsSpec:
+    """Every pair turns ``factor`` times slower: positions count as if they lay ``factor`` times closer together."""
+    factor: float
+
+
+@dataclass(frozen=True)
 class RotarySpec:
     """Pairs of the first ``dims`` entries of a query or key vector are turned by the angle position * speed_i,
     speed_i = base^(-2i / dims), i = 0 .. dims / 2 - 1; entries behind ``dims`` pass.  ``interleaved``: pair i is
     (2i, 2i + 1), else (i, i + dims / 2).  (u, v) becomes (u cos a - v sin a, v cos a + u sin a).  ``scaling``
-    changes the speeds and the length of the turned pairs (``RampedSpeedsSpec``)."""
+    changes the speeds and the length of the turned pairs (``RampedSpeedsSpec``) or divides the speeds
+    (``LinearSpeedsSpec``)."""
     kind: str            # "rotary"
     dims: int
     base: float
     interleaved: bool = True
-    scaling: Optional[RampedSpeedsSpec] = None
+    scaling: Optional[object] = None         # RampedSpeedsSpec | LinearSpeedsSpec
 
 
 @dataclass(frozen=True)
@@ -179,6 +192,25 @@ class RetentionSpec:
     decay: Tuple[float, ...]
     norm_eps: float
     rotary: Optional[RotarySpec] = None
+    gate: str = "silu"
+
+
+@dataclass(frozen=True)
+class GatedLinearSpec:
+    """Linear attention with a decay per head and key channel that the input sets, and neither softmax nor
+    denominator.  Per head a matrix S (``head_dim`` x ``v_head_dim``, 32-bit) is carried from token to token:
+    S <- diag(a) S + k v^T, o = S^T q, with a = logistic(z)^(1 / ``tau``), z = W_a2 (W_a1 h) + b (``decay_rank`` numbers
+    in between; -1: as many as the two matrices share).  q is multiplied by head_dim^-1/2.  Each head's o is divided by
+    its root mean square (``norm_eps``) and multiplied by a gain of ``v_head_dim`` entries that the heads share, the
+    heads are multiplied by ``gate`` ("silu") of one more projection and projected back to the width."""
+    kind: str            # "gated_linear"
+    width: int
+    n_heads: int
+    head_dim: int
+    v_head_dim: int
+    tau: float
+    norm_eps: float
+    decay_rank: int = -1
     gate: str = "silu"
 
 

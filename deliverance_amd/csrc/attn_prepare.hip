@@ -9,6 +9,7 @@
 //                    (speeds in double precision; sine and cosine of the double angle, used in 32-bit)
 //
 // `v_from_k`: the rows hold no values; a key as it was projected (normalised, not turned) is also the value (Dv = D).
+// Hkv = 0: the rows hold queries only (a layer that reads another layer's keys and values).
 // `pass_cols`: so many columns behind q | k | v of the rows (a gate's, say) go over into the queries' rows behind the
 // queries, converted.  `mag` multiplies sine and cosine (the length that a turned pair gains; 1 as a rule).
 //
@@ -33,7 +34,7 @@ attn_prepare_kernel(const float* __restrict__ raw, int ld, int Hq, int Hkv, int 
   const float* row = raw + (size_t)n * ld;
   const int half = dims / 2;
   const bool normed = gq != nullptr;
-  const int q_groups = whole ? 1 : Hq, k_groups = whole ? 1 : Hkv;
+  const int q_groups = whole ? 1 : Hq, k_groups = whole ? (Hkv > 0 ? 1 : 0) : Hkv;
   const int q_len = whole ? Hq * D : D, k_len = whole ? Hkv * D : D;
   if (dims > 0) {
     const double p = (double)positions[n];
@@ -105,11 +106,12 @@ extern "C" int da_attn_prepare(const float* raw, int ld, int Hq, int Hkv, int D,
                                const double* speeds, int dims, int interleaved, void* q_out, int out_dtype, int q_ld,
                                void* cache, const int* slot_map, int page, int N, int v_from_k, int pass_cols, float mag,
                                void* stream) {
-  DA_REQUIRE(N >= 0 && Hq > 0 && Hkv > 0 && D > 0 && Dv > 0 && page > 0 && pass_cols >= 0, "attn_prepare: bad sizes");
+  DA_REQUIRE(N >= 0 && Hq > 0 && Hkv >= 0 && D > 0 && Dv > 0 && page > 0 && pass_cols >= 0, "attn_prepare: bad sizes");
+  DA_REQUIRE(Hkv > 0 || cache == nullptr, "attn_prepare: rows without keys have nothing to keep");
   DA_REQUIRE(!v_from_k || Dv == D, "attn_prepare: values that are the keys have the keys' size %d, not %d", D, Dv);
   DA_REQUIRE(ld >= (Hq + Hkv) * D + (v_from_k ? 0 : Hkv * Dv) + pass_cols && q_ld >= Hq * D + pass_cols,
              "attn_prepare: row lengths too small");
-  DA_REQUIRE((gq == nullptr) == (gk == nullptr), "attn_prepare: a norm needs both gains");
+  DA_REQUIRE(Hkv == 0 || (gq == nullptr) == (gk == nullptr), "attn_prepare: a norm needs both gains");
   DA_REQUIRE(gq == nullptr || eps > 0.f, "attn_prepare: the norm needs a positive eps");
   DA_REQUIRE(dims >= 0 && dims <= D && dims % 2 == 0 && dims / 2 <= PREP_MAX_HALF, "attn_prepare: %d turned entries of %d", dims, D);
   DA_REQUIRE(dims == 0 || (positions != nullptr && speeds != nullptr), "attn_prepare: a turn needs positions and speeds");

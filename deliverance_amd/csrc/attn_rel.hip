@@ -6,6 +6,7 @@
 //   s_j = cap((q . k_j) * scale * temp(p)) + bias[h][min(p - j, n_dist - 1)]
 //   temp(p) = 1 + t_coef * ln(floor((p + 1) / t_every) + 1)          (1 when t_every is 0)
 //   cap(s) = softcap * tanh(s / softcap)                              (s itself when softcap is 0)
+// With `chunk` c (in place of a window) the keys are j in [floor(p / c) c, p].
 // With a window w the keys are j in [p - w + 1, p] and, with keep_first, also j < keep_first: the first keys of a
 // sequence stay visible at their true positions.
 //   w = softmax(s),  o = sum_j w_j v_j                                 (all in 32-bit)
@@ -28,7 +29,7 @@ __global__ void __launch_bounds__(DA_WAVE)
 attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cache,
                     const int* __restrict__ block_table, int max_blocks,
                     const int* __restrict__ seq_of_token, const int* __restrict__ positions,
-                    int Hq, int Hkv, int D, int Dv, int page, float scale, int window,
+                    int Hq, int Hkv, int D, int Dv, int page, float scale, int window, int chunk,
                     const float* __restrict__ bias, int n_dist, float t_coef, int t_every, float softcap, int keep_first,
                     const float* __restrict__ sink, const T* __restrict__ gate, int gate_ld,
                     T* __restrict__ out, int out_ld) {
@@ -49,7 +50,7 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
   for (int d = lane; d < D; d += DA_WAVE) qs[d] = to_f32(q[(size_t)n * q_ld + h * D + d]);
   __syncthreads();
 
-  const int lo = (window > 0 && p - window + 1 > 0) ? p - window + 1 : 0;
+  const int lo = chunk > 0 ? p / chunk * chunk : ((window > 0 && p - window + 1 > 0) ? p - window + 1 : 0);
   float m = -INFINITY, l = 0.f;
   float acc[REL_MAX_D / DA_WAVE];
 #pragma unroll
@@ -121,14 +122,15 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
 
 extern "C" int da_attn_rel_ref(const void* q, int q_ld, const void* cache, int dtype, const int* block_table,
                                int max_blocks, const int* seq_of_token, const int* positions, int N, int Hq, int Hkv,
-                               int D, int Dv, int page, float scale, int window, const float* bias, int n_dist,
+                               int D, int Dv, int page, float scale, int window, int chunk, const float* bias, int n_dist,
                                float t_coef, int t_every, float softcap, int keep_first, const float* sink,
                                const void* gate, int gate_ld, void* out, int out_ld, void* stream) {
   DA_REQUIRE(N >= 0 && Hq > 0 && Hkv > 0 && D > 0 && Dv > 0 && page > 0, "attn_rel_ref: bad sizes");
   DA_REQUIRE(Hq % Hkv == 0, "attn_rel_ref: %d query heads are not a multiple of %d key heads", Hq, Hkv);
   DA_REQUIRE(D <= REL_MAX_D && Dv <= REL_MAX_D, "attn_rel_ref: head sizes %d, %d exceed %d", D, Dv, REL_MAX_D);
   DA_REQUIRE(q_ld >= Hq * D && out_ld >= Hq * Dv, "attn_rel_ref: row lengths too small");
-  DA_REQUIRE(window >= 0 && max_blocks > 0, "attn_rel_ref: bad window or block table");
+  DA_REQUIRE(window >= 0 && chunk >= 0 && max_blocks > 0, "attn_rel_ref: bad window, chunk or block table");
+  DA_REQUIRE(window == 0 || chunk == 0, "attn_rel_ref: a window or chunks, not both");
   DA_REQUIRE(!bias || n_dist > 0, "attn_rel_ref: a bias table without entries");
   DA_REQUIRE(t_every >= 0, "attn_rel_ref: bad temperature period %d", t_every);
   DA_REQUIRE(softcap >= 0.f && keep_first >= 0, "attn_rel_ref: bad score cap or kept first keys");
@@ -137,12 +139,12 @@ extern "C" int da_attn_rel_ref(const void* q, int q_ld, const void* cache, int d
   if (dtype == DA_BF16)
     hipLaunchKernelGGL(attn_rel_ref_kernel<bf16_t>, dim3(N * Hq), dim3(DA_WAVE), 0, (hipStream_t)stream,
                        (const bf16_t*)q, q_ld, (const bf16_t*)cache, block_table, max_blocks, seq_of_token, positions,
-                       Hq, Hkv, D, Dv, page, scale, window, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
+                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
                        (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld);
   else
     hipLaunchKernelGGL(attn_rel_ref_kernel<float>, dim3(N * Hq), dim3(DA_WAVE), 0, (hipStream_t)stream,
                        (const float*)q, q_ld, (const float*)cache, block_table, max_blocks, seq_of_token, positions,
-                       Hq, Hkv, D, Dv, page, scale, window, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
+                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
                        (const float*)gate, gate_ld, (float*)out, out_ld);
   DA_CHECK_LAUNCH("attn_rel_ref");
   return 0;

@@ -2,7 +2,8 @@
 // different sizes, a cap on the scores, and a window that keeps a sequence's first keys.  Prompt portions and
 // decode rows alike; scores never leave the chip.
 //
-// For the row at position p, key j is seen when j <= p and (no window, or p - j < window, or j < keep_first);
+// For the row at position p, key j is seen when j <= p and (no window, or p - j < window, or j < keep_first); with
+// `chunk` in place of a window, when j <= p and floor(j / chunk) = floor(p / chunk);
 //   s_j = cap((q . k_j) * scale),  cap(s) = softcap * tanh(s / softcap)   (s itself when softcap is 0)
 //   o   = sum_j softmax(s)_j v_j                                           (scores, weights and sums in 32-bit)
 // `sink` (optional, [Hq], 32-bit): the softmax's denominator also holds exp(sink[h]), a term without a key or a
@@ -50,7 +51,7 @@ __global__ void __launch_bounds__(AW_WAVES * DA_WAVE)
 attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ cache,
                    const int* __restrict__ block_table, int max_blocks, const int* __restrict__ q_start,
                    const int* __restrict__ seq_lens, int seq0, int Hq, int Hkv, int D, int Dv, int page, float scale,
-                   int window, int keep_first, float softcap, const float* __restrict__ sink,
+                   int window, int chunk, int keep_first, float softcap, const float* __restrict__ sink,
                    const bf16_t* __restrict__ gate, int gate_ld, bf16_t* __restrict__ out, int out_ld, int RB) {
   constexpr int PER = DT * 16 + 2;
   __shared__ float mg[3 * PER * DA_WAVE];              // (KP - 1) * RB <= 3 partial results
@@ -71,11 +72,17 @@ attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restr
   const bf16_t* kbase = cache + (long long)hk * page * D;
   const bf16_t* vbase = cache + (long long)Hkv * page * D + (long long)hk * Dv * page;
   const int kfw = window > 0 ? keep_first : 0;
+  // the first position that a row at position p sees (apart from kept first keys)
+  auto low_of = [&](int p) -> int {
+    if (chunk > 0) return p / chunk * chunk;
+    return window > 0 && p - window + 1 > 0 ? p - window + 1 : 0;
+  };
 
   // this lane's query row (a column of Q^T) and its position; a row that does not exist sees nothing
   const int qi = wrow + col;
   const bool q_ok = qi < T && past + qi >= 0;
   const int pq = q_ok ? past + qi : -1;
+  const int p_low = q_ok ? low_of(pq) : 0;
   aw_bf16x8_t qf[D16];
 #pragma unroll
   for (int kd = 0; kd < D16; ++kd) {
@@ -89,7 +96,7 @@ attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restr
   const int w_first = past + wrow;
   const int w_last = past + ((wrow + 31 < T - 1) ? wrow + 31 : T - 1);
   const bool wave_on = wrow < T && w_last >= 0 && w_first >= 0;
-  const int w_lo = (window > 0 && w_first - window + 1 > 0) ? w_first - window + 1 : 0;
+  const int w_lo = wave_on ? low_of(w_first) : 0;
   const int t_lo = w_lo / AW_BK, t_hi = wave_on ? w_last / AW_BK : -1;
   const int kept_tiles = (kfw + AW_BK - 1) / AW_BK;
   const int n_kept = kept_tiles < t_lo ? kept_tiles : t_lo;       // tiles below the window's first that hold kept keys
@@ -169,7 +176,7 @@ attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restr
       } else {
         v = sc[r] * (scale * AW_LOG2E);
       }
-      const bool seen = key <= pq && (window <= 0 || pq - key < window || key < keep_first);
+      const bool seen = key <= pq && (key >= p_low || key < kfw);
       v = seen ? v : -INFINITY;
       sc[r] = v;
       tmax = fmaxf(tmax, v);
@@ -292,7 +299,7 @@ extern "C" int da_attn_window_takes(int D, int Dv, int page) {
 // last of them at position seq_lens[s] - 1.  form: 0, or the row blocks a workgroup (1, 2, 4).
 extern "C" int da_attn_window(const void* q, int q_ld, const void* cache, const int* block_table, int max_blocks,
                               const int* q_start, const int* seq_lens, int seq0, int n_seqs, int max_query_len, int Hq,
-                              int Hkv, int D, int Dv, int page, float scale, int window, int keep_first, float softcap,
+                              int Hkv, int D, int Dv, int page, float scale, int window, int chunk, int keep_first, float softcap,
                               const float* sink, const void* gate, int gate_ld, void* out, int out_ld, int form,
                               void* stream) {
   DA_REQUIRE(n_seqs >= 0 && Hq > 0 && Hkv > 0 && max_query_len >= 0, "attn_window: bad sizes");
@@ -301,7 +308,8 @@ extern "C" int da_attn_window(const void* q, int q_ld, const void* cache, const 
   DA_REQUIRE(da_attn_window_takes(D, Dv, page), "attn_window: head sizes %d and %d with pages of %d are not taken", D, Dv, page);
   DA_REQUIRE(q_ld >= Hq * D && q_ld % 8 == 0 && out_ld >= Hq * Dv, "attn_window: row lengths");
   DA_REQUIRE(((uintptr_t)q % 16 == 0) && ((uintptr_t)cache % 16 == 0), "attn_window: operands must be 16-byte aligned");
-  DA_REQUIRE(window >= 0 && keep_first >= 0 && softcap >= 0.f && max_blocks > 0, "attn_window: bad window, kept keys, cap or block table");
+  DA_REQUIRE(window >= 0 && chunk >= 0 && keep_first >= 0 && softcap >= 0.f && max_blocks > 0, "attn_window: bad window, chunk, kept keys, cap or block table");
+  DA_REQUIRE(window == 0 || chunk == 0, "attn_window: a window or chunks, not both");
   DA_REQUIRE(scale > 0.f, "attn_window: the score scale must be positive, found %g", (double)scale);
   DA_REQUIRE(!gate || gate_ld >= Hq * Dv, "attn_window: the gate's rows are too short");
   DA_REQUIRE((long)n_seqs * Hq < (1L << 31) && max_query_len <= 65535 * 32, "attn_window: too many sequences, heads or rows for one launch");
@@ -318,7 +326,7 @@ extern "C" int da_attn_window(const void* q, int q_ld, const void* cache, const 
 #define AW_GO(N, M)                                                                                                  \
   hipLaunchKernelGGL((attn_window_kernel<N, M>), grid, block, 0, (hipStream_t)stream, (const bf16_t*)q, q_ld,        \
                      (const bf16_t*)cache, block_table, max_blocks, q_start, seq_lens, seq0, Hq, Hkv, D, Dv, page,   \
-                     scale, window, keep_first, softcap, sink, (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld, RB)
+                     scale, window, chunk, keep_first, softcap, sink, (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld, RB)
 #define AW_VALUES(N)                 \
   do {                               \
     if (Dv <= 32) AW_GO(N, 1);       \

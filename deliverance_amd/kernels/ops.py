@@ -99,9 +99,9 @@ _ARGTYPES = {
     "da_attn_prefill_rel": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _VP, _I, _I, _VP],
     "da_rmsnorm": [_VP, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
     "da_rmsnorm_add": [_VP, _VP, _I, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
-    "da_attn_rel_ref": [_VP, _I, _VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _F, _I, _VP, _VP, _I,
+    "da_attn_rel_ref": [_VP, _I, _VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _I, _I, _VP, _I, _F, _I, _F, _I, _VP, _VP, _I,
                         _VP, _I, _VP],
-    "da_attn_window": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _F, _VP, _VP, _I, _VP, _I, _I,
+    "da_attn_window": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _VP, _VP, _I, _VP, _I, _I,
                        _VP],
     "da_attn_window_takes": [_I, _I, _I],
     "da_attn_prepare": [_VP, _I, _I, _I, _I, _I, _VP, _I, _VP, _I, _F, _I, _VP, _VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _I, _I, _F,
@@ -115,6 +115,7 @@ _ARGTYPES = {
     "da_concat_rows": [_VP, _VP, _I, _I, _I, _I, _I, _VP],
     "da_retention": [_VP, _I, _I, _I, _I, _I, _VP, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP,
                      ctypes.c_long, _VP],
+    "da_gla_walk": [_VP, _I, _I, _I, _I, _I, _VP, _I, _VP, _F, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP],
     "da_moe_top": [_VP, _I, _VP, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_softcap": [_VP, ctypes.c_long, _F, _VP],
     "da_moe_route": [_VP, _VP, _I, _VP, _I, _I, _I, _I, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP],
@@ -585,11 +586,12 @@ def attention_rel_ref(q: torch.Tensor, cache_slot: torch.Tensor, block_table: to
                       positions: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int, v_head_dim: int, page: int,
                       scale: float, window: Optional[int], dist_bias: Optional[torch.Tensor], temp_coef: float,
                       temp_every: int, out: torch.Tensor, softcap: float = 0.0, keep_first: int = 0,
-                      sink: Optional[torch.Tensor] = None, gate_col: int = -1) -> torch.Tensor:
+                      sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: int = 0) -> torch.Tensor:
     """Plain paged attention with a bias by distance (``dist_bias`` [Hq, n_dist] float32, the last column for every
     larger distance), a query temperature by position, values of their own size, a cap on the scores
     (``softcap * tanh(score / softcap)``) and, with a window, ``keep_first`` first keys that stay visible.  ``sink``
-    (float32 [Hq]): exp(sink[h]) joins the softmax's denominator; ``gate_col`` >= 0: out * logistic(gate), the gate's
+    (float32 [Hq]): exp(sink[h]) joins the softmax's denominator; ``chunk`` (in place of a window): a row sees the keys of
+    its own chunk of so many positions; ``gate_col`` >= 0: out * logistic(gate), the gate's
     Hq * Dv entries lying in q's rows from that column on (q is then wider than its Hq * D query entries)."""
     _dev(q, cache_slot, block_table, seq_of_token, positions, dist_bias, out, sink)
     gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, n_heads * head_dim, n_heads * v_head_dim, q, "attention")
@@ -611,7 +613,7 @@ def attention_rel_ref(q: torch.Tensor, cache_slot: torch.Tensor, block_table: to
         n_dist = dist_bias.shape[1]
     _check(_lib().da_attn_rel_ref(_ptr(q), q.stride(0), _ptr(cache_slot), _dt(q), _ptr(block_table), block_table.shape[1],
                                   _ptr(seq_of_token), _ptr(positions), N, n_heads, n_kv_heads, head_dim, v_head_dim, page,
-                                  float(scale), int(window or 0), _ptr(dist_bias), n_dist, float(temp_coef),
+                                  float(scale), int(window or 0), int(chunk or 0), _ptr(dist_bias), n_dist, float(temp_coef),
                                   int(temp_every), float(softcap), int(keep_first if window else 0), _ptr(sink),
                                   gate_ptr, gate_ld, _ptr(out), out.stride(0), _stream()))
     return out
@@ -1041,10 +1043,10 @@ def attention_window(q: torch.Tensor, cache_slot: torch.Tensor, block_table: tor
                      seq_lens: torch.Tensor, seq0: int, n_seqs: int, max_query_len: int, n_heads: int, n_kv_heads: int,
                      head_dim: int, v_head_dim: int, page: int, scale: float, window: Optional[int], keep_first: int,
                      softcap: float, out: torch.Tensor, form: int = 0, sink: Optional[torch.Tensor] = None,
-                     gate_col: int = -1) -> torch.Tensor:
+                     gate_col: int = -1, chunk: int = 0) -> torch.Tensor:
     """Attention of the sequences ``seq0 .. seq0 + n_seqs - 1`` of a step on the matrix cores, in bfloat16, with keys and
     values of their own sizes, a cap on the scores and, with a window, ``keep_first`` first keys that stay visible.
-    ``form``: 0 leaves the workgroup's row blocks to the kernel's rule; 1, 2 or 4 fixes them."""
+    ``chunk`` (in place of a window): a row sees the keys of its own chunk of so many positions only.  ``form``: 0 leaves the workgroup's row blocks to the kernel's rule; 1, 2 or 4 fixes them."""
     _dev(q, cache_slot, block_table, q_start, seq_lens, out, sink)
     _rows_2d(q, "q"); _rows_2d(out, "out")
     gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, n_heads * head_dim, n_heads * v_head_dim, q, "attention_window")
@@ -1059,7 +1061,7 @@ def attention_window(q: torch.Tensor, cache_slot: torch.Tensor, block_table: tor
           and seq_lens.numel() >= seq0 + n_seqs, "attention_window: q_start must be int32 [S+1] and seq_lens int32 [S]")
     _check(_lib().da_attn_window(_ptr(q), q.stride(0), _ptr(cache_slot), _ptr(block_table), block_table.shape[1],
                                  _ptr(q_start), _ptr(seq_lens), seq0, n_seqs, max_query_len, n_heads, n_kv_heads, head_dim,
-                                 v_head_dim, page, float(scale), int(window or 0), int(keep_first if window else 0),
+                                 v_head_dim, page, float(scale), int(window or 0), int(chunk or 0), int(keep_first if window else 0),
                                  float(softcap), _ptr(sink), gate_ptr, gate_ld, _ptr(out),
                                  out.stride(0), int(form), _stream()))
     return out
@@ -1073,11 +1075,11 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
                         head_dim: int, v_head_dim: int, scale: float, window: Optional[int],
                         dist_bias: Optional[torch.Tensor], temp_coef: float, temp_every: int,
                         out: torch.Tensor, softcap: float = 0.0, keep_first: int = 0,
-                        sink: Optional[torch.Tensor] = None, gate_col: int = -1) -> torch.Tensor:
+                        sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: Optional[int] = None) -> torch.Tensor:
     """Attention of every row of the step with a bias by distance, a query temperature, values of their own
     size, a cap on the scores, first keys that a window keeps, a term without a key in the softmax's denominator
-    (``sink``) and a logistic gate on the result (``gate_col``: where the gate lies in q's rows), each optional; the last two go with the matrix-core
-    kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
+    (``sink``), a logistic gate on the result (``gate_col``: where the gate lies in q's rows) and chunks in place of a window
+    (``chunk``), each optional; the last three go with the matrix-core kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
     bias row that fits the prefill kernel's LDS copy, the one-token sequences go to the decode kernel and the
     portions to the prefill kernel (their forms with these extras); a cap, kept first keys and values of another size
     go to the matrix-core kernel for those (head sizes up to 128, no bias table, no temperature); 32-bit, the reference
@@ -1096,9 +1098,11 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
         for s_ in range(first, last):
             t = starts[s_ + 1] - starts[s_]
             n = lens[s_]
-            keys += min(n, span + t) if span else n
+            keys += (n - (n - t) // chunk * chunk) if chunk else (min(n, span + t) if span else n)
             rows += t
-            if span:
+            if chunk:
+                pairs += sum((n - t + i) % chunk + 1 for i in range(t))
+            elif span:
                 pairs += sum(min(n - t + i + 1, span) for i in range(t))
             else:
                 pairs += sum(n - t + i + 1 for i in range(t)) if t > 1 else n
@@ -1107,7 +1111,7 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
 
     tuned = (_MODE == "tuned" and q.dtype == torch.bfloat16 and v_head_dim == D and D % 16 == 0
              and softcap == 0.0 and not (window and keep_first) and sink is None and gate_col < 0
-             and D <= PREFILL_REL_MAX_HEAD_DIM and cache_slot.dim() == 5 and q.stride(0) % 8 == 0
+             and not chunk and D <= PREFILL_REL_MAX_HEAD_DIM and cache_slot.dim() == 5 and q.stride(0) % 8 == 0
              and q.data_ptr() % 16 == 0 and (dist_bias is None or dist_bias.shape[1] <= PREFILL_REL_MAX_DIST))
     if tuned:
         if nd:
@@ -1129,17 +1133,17 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
         if nd:
             with _timed("attention_window_decode", *cost(0, nd)):
                 attention_window(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, 0, nd, 1, n_heads, n_kv_heads, D,
-                                 v_head_dim, page, scale, window, keep_first, softcap, out, sink=sink, gate_col=gate_col)
+                                 v_head_dim, page, scale, window, keep_first, softcap, out, sink=sink, gate_col=gate_col, chunk=chunk or 0)
         if ctx.n_seqs > nd:
             with _timed("attention_window", *cost(nd, ctx.n_seqs)):
                 attention_window(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, nd, ctx.n_seqs - nd, ctx.max_query_len,
                                  n_heads, n_kv_heads, D, v_head_dim, page, scale, window, keep_first, softcap, out,
-                                 sink=sink, gate_col=gate_col)
+                                 sink=sink, gate_col=gate_col, chunk=chunk or 0)
         return out
     with _timed("attention_plain", *cost(0, ctx.n_seqs), "fp32" if q.dtype == torch.float32 else "bf16"):
         return attention_rel_ref(q, cache_slot, bt, ctx.seq_of_token, ctx.positions, n_heads, n_kv_heads, head_dim,
                                  v_head_dim, page, scale, window, dist_bias, temp_coef, temp_every, out, softcap, keep_first,
-                                 sink=sink, gate_col=gate_col)
+                                 sink=sink, gate_col=gate_col, chunk=chunk or 0)
 
 
 def gated_linear(ctx, h: torch.Tensor, gate_up: torch.Tensor, mid: torch.Tensor, act: str, limit: float = 0.0) -> torch.Tensor:
@@ -1494,6 +1498,40 @@ def retention(ctx, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, decay:
     return o
 
 
+# ------------------------------------------------------------------------------- gated linear attention
+GLA_MAX_DIM = 256            # key entries a head of gated linear attention (csrc/gla.hip)
+
+
+def gla_walk(ctx, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, raw: torch.Tensor, bias: torch.Tensor, tau: float,
+             q_scale: float, state: torch.Tensor, o: torch.Tensor, n_heads: int, head_dim: int, v_head_dim: int,
+             write: bool = True) -> torch.Tensor:
+    """Per head S <- diag(a) S + k v^T, o = S^T (q_scale q), a = logistic(raw + bias)^(1 / tau), over every sequence of
+    the step, token by token (csrc/gla.hip).  ``qkv`` [N, ...] holds q and k (H * D entries each, from columns ``q_off``
+    and ``k_off``) and v (H * Dv from ``v_off``) in the step's dtype; ``raw`` [N, H * D] and ``bias`` [H * D] 32-bit;
+    ``state`` [slots, >= H * Dv * D] 32-bit is read at each portion's start and, with ``write``, written at its end; ``o``
+    [N, H * Dv] 32-bit."""
+    _dev(qkv, raw, bias, state, o)
+    for t_, nm in ((qkv, "qkv"), (raw, "raw"), (o, "o")):
+        _rows_2d(t_, nm)
+    N, H, D, Dv = qkv.shape[0], n_heads, head_dim, v_head_dim
+    ld = _state_args(state, "gla_walk")
+    _need(1 <= D <= GLA_MAX_DIM, f"gla_walk: a key size of {D} is outside 1..{GLA_MAX_DIM}")
+    _need(min(q_off, k_off, v_off) >= 0 and max(q_off, k_off) + H * D <= qkv.shape[1] and v_off + H * Dv <= qkv.shape[1],
+          "gla_walk: q, k and v leave the row")
+    _need(raw.dtype == bias.dtype == o.dtype == torch.float32 and raw.shape[0] == N and raw.shape[1] >= H * D
+          and bias.is_contiguous() and bias.numel() == H * D and o.shape[0] == N and o.shape[1] >= H * Dv,
+          "gla_walk: raw [N, H * D], bias [H * D] and o [N, H * Dv] must be float32")
+    _need(ld >= H * Dv * D, "gla_walk: the state row is too short")
+    _need(ctx.q_start.numel() >= ctx.n_seqs + 1 and ctx.state_slots.numel() >= ctx.n_seqs, "gla_walk: the step's arrays are too short")
+    nb = N * ((2 * H * D + H * Dv) * qkv.element_size() + (H * D + H * Dv) * 4) + 2 * ctx.n_seqs * H * Dv * D * 4
+    with _timed("gla_walk", nb, 4 * N * H * D * Dv, "fp32"):
+        _check(_lib().da_gla_walk(_ptr(qkv), _dt(qkv), qkv.stride(0), int(q_off), int(k_off), int(v_off), _ptr(raw),
+                                  raw.stride(0), _ptr(bias), float(tau), float(q_scale), _ptr(state), ld,
+                                  _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(o), o.stride(0), ctx.n_seqs, H, D, Dv,
+                                  int(bool(write)), _stream()))
+    return o
+
+
 # ------------------------------------------------------------------------------- short filter and scan
 def _state_args(state: torch.Tensor, name: str):
     _need(state.dtype == torch.float32 and state.dim() == 2 and state.is_contiguous(), f"{name}: the state must be contiguous float32 [slots, row]")
@@ -1592,7 +1630,7 @@ def attn_prepare(raw: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int
     position (``speeds`` float64 [dims / 2]; pairs (2i, 2i + 1) when ``interleaved``, else (i, i + dims / 2)),
     the queries stored in ``q_out`` and keys and values in their cache rows ``slot_map`` (a page of the slot
     holds Hkv * page * D keys, then Hkv * Dv * page values).  ``values_are_keys``: the rows hold q | k only, and a key
-    before its turn is also the value.  ``pass_cols``: so many columns behind q | k | v go over into ``q_out`` behind the
+    before its turn is also the value.  ``n_kv_heads`` 0: the rows hold queries only, and nothing is kept.  ``pass_cols``: so many columns behind q | k | v go over into ``q_out`` behind the
     queries, converted.  ``magnitude`` multiplies sine and cosine."""
     _dev(raw, q_gain, k_gain, positions, speeds, q_out, cache_slot, slot_map)
     _rows_2d(raw, "raw"); _rows_2d(q_out, "q_out")
@@ -1602,10 +1640,12 @@ def attn_prepare(raw: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int
     _need(raw.dtype == torch.float32 and pass_cols >= 0 and raw.shape[1] >= q_cols + k_cols + v_cols + pass_cols,
           "attn_prepare: raw must be float32 [N, q | k | v | what passes]")
     _need(q_out.shape[0] == N and q_out.shape[1] >= q_cols + pass_cols, "attn_prepare: q_out must be [N, Hq * D + what passes]")
-    _need((q_gain is None) == (k_gain is None), "attn_prepare: a norm needs both gains")
+    _need(n_kv_heads > 0 or cache_slot is None, "attn_prepare: rows without keys have nothing to keep")
+    _need(n_kv_heads == 0 or (q_gain is None) == (k_gain is None), "attn_prepare: a norm needs both gains")
     if q_gain is not None:
         nq, nk = (q_cols, k_cols) if whole else (head_dim, head_dim)
-        _need(q_gain.is_contiguous() and k_gain.is_contiguous() and q_gain.numel() == nq and k_gain.numel() == nk,
+        _need(q_gain.is_contiguous() and q_gain.numel() == nq
+              and (n_kv_heads == 0 or (k_gain.is_contiguous() and k_gain.numel() == nk)),
               f"attn_prepare: gains of {nq} and {nk} entries are needed")
     _need(dims % 2 == 0 and 0 <= dims <= min(head_dim, PREPARE_MAX_ROT), f"attn_prepare: {dims} turned entries of {head_dim}")
     if dims:

@@ -83,7 +83,10 @@ class CausalLM:
                     if slot not in needs:
                         raise ValueError(f"layer {call.layer} reads cache slot {slot} that nothing writes")
                     if needs[slot] != need:
-                        raise ValueError(f"layer {call.layer} reads cache slot {slot} of another shape")
+                        join = getattr(needs[slot], "joined", None)       # pages that two masks read
+                        if join is None or type(need) is not type(needs[slot]):
+                            raise ValueError(f"layer {call.layer} reads cache slot {slot} of another shape")
+                        needs[slot] = join(need)
         return needs
 
     # ---- one step ----------------------------------------------------------------------------

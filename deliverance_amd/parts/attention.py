@@ -13,8 +13,10 @@ cap * tanh(score / cap)), and first keys of a sequence that a window never leave
 position i sees j <= i when i - j < window or j < keep_first), values that are the keys before their rotation
 (``values_are_keys``: the projection has no value rows; the kernel that turns the keys also keeps them unturned as
 values), a term without key or value in the softmax's denominator (``sink``: exp(0), or exp of a learned number per
-head), and a logistic gate of one more projection of the input on the heads' results (``out_gate``: its rows are stacked
-behind q | k | v in the same product).
+head), a logistic gate of one more projection of the input on the heads' results (``out_gate``: its rows are stacked
+behind q | k | v in the same product), chunks in place of a window (``chunk``: a row sees the earlier keys of its own chunk
+of positions), and another layer's keys and values (``shared_kv``: the product has query and gate rows only, and the run
+order names the slot that the other layer has written).
 Reference: core/src/main/java/io/teknek/deliverance/generator/CausalSelfAttention.java:226-420
 (projections :266-291, cache write :315-336, scores/softmax/weighted sum :458-532, output
 projection :385-408); the residual add is TransformerBlock.java:176.
@@ -69,7 +71,10 @@ class CausalSelfAttention(Mixer):
         self.v_cols = self.n_kv_heads * self.v_head_dim
         self.o_cols = self.n_heads * self.v_head_dim
         self.values_are_keys = bool(getattr(spec, "values_are_keys", False))
-        self.qkv_cols = self.q_cols + self.kv_cols + (0 if self.values_are_keys else self.v_cols)
+        self.shared_kv = bool(getattr(spec, "shared_kv", False))
+        if self.shared_kv and (self.values_are_keys or spec.qkv_bias):
+            raise ValueError("a layer that reads another layer's keys and values has neither values that are keys nor a bias")
+        self.qkv_cols = self.q_cols + (0 if self.shared_kv else self.kv_cols + (0 if self.values_are_keys else self.v_cols))
         self.out_gate = getattr(spec, "out_gate", None)
         if self.out_gate not in (None, "sigmoid"):
             raise ValueError(f"an output gate is 'sigmoid' or None, not {self.out_gate!r}")
@@ -82,6 +87,9 @@ class CausalSelfAttention(Mixer):
         self.gate_off = self.qkv_cols
         self.scale = float(spec.scale)
         self.window = spec.window
+        self.chunk = getattr(spec, "chunk", None)
+        if self.chunk is not None and (self.window or int(self.chunk) <= 0):
+            raise ValueError(f"chunks of {self.chunk} positions with a window of {self.window}: one of the two, and positive")
         self.qkv_weight = to_matrix(params["qkv_weight"], dtype, device)
         self.out_weight = to_matrix(params["out_weight"], dtype, device)
         self.qkv_bias = to_vector(params.get("qkv_bias"), dtype, device) if spec.qkv_bias else None
@@ -123,25 +131,27 @@ class CausalSelfAttention(Mixer):
         if qn is not None:
             nq, nk = (self.q_cols, self.kv_cols) if qn.whole else (self.head_dim, self.head_dim)
             self.q_gain = to_vector(params["q_norm"], dtype, device)
-            self.k_gain = to_vector(params["k_norm"], dtype, device)
-            if self.q_gain.numel() != nq or self.k_gain.numel() != nk:
-                raise ValueError(f"query and key gains have {self.q_gain.numel()} and {self.k_gain.numel()} entries, "
-                                 f"expected {nq} and {nk}")
+            self.k_gain = None if self.shared_kv else to_vector(params["k_norm"], dtype, device)
+            if self.q_gain.numel() != nq or (self.k_gain is not None and self.k_gain.numel() != nk):
+                raise ValueError(f"query and key gains have {self.q_gain.numel()} and "
+                                 f"{nk if self.k_gain is None else self.k_gain.numel()} entries, expected {nq} and {nk}")
         self.extras = (self.dist_bias is not None or self.temp_every > 0 or self.v_head_dim != self.head_dim
-                       or self.softcap > 0.0 or self.keep_first > 0 or self.sink is not None or self.out_gate is not None)
+                       or self.softcap > 0.0 or self.keep_first > 0 or self.sink is not None or self.out_gate is not None
+                       or self.chunk is not None)
         self.position = None
         if spec.position is not None and spec.position.kind != "none":
             self.position = build_position(spec.position, params.get("position", {}), dtype, device)
 
     def cache_need(self):
         return KVNeed(self.n_kv_heads, self.head_dim, self.window,
-                      None if self.v_head_dim == self.head_dim else self.v_head_dim, keep_first=self.keep_first)
+                      None if self.v_head_dim == self.head_dim else self.v_head_dim, keep_first=self.keep_first,
+                      chunk=self.chunk)
 
     def _epilogue_write(self) -> bool:
         """Whether the q|k|v product may write keys and values to the cache itself (its epilogue assumes
         keys and values of one size)."""
         return (self.position is None and self.v_head_dim == self.head_dim and self.qk_norm is None
-                and self.out_gate is None and not self.values_are_keys)
+                and self.out_gate is None and not self.values_are_keys and not self.shared_kv)
 
     normed_into = True
 
@@ -210,20 +220,22 @@ class CausalSelfAttention(Mixer):
         self._attend(ctx, qkv, x, slot, group, call)
 
     def _prepared(self) -> bool:
-        """Whether queries, keys and values go through ``ops.attn_prepare`` (a norm of queries and keys, or values
-        that are the keys; a rotation or no position encoding)."""
-        if self.qk_norm is None and not self.values_are_keys:
+        """Whether queries, keys and values go through ``ops.attn_prepare`` (a norm of queries and keys, values that
+        are the keys, or another layer's keys; a rotation or no position encoding)."""
+        if self.qk_norm is None and not self.values_are_keys and not self.shared_kv:
             return False
         if self.position is not None and not hasattr(self.position, "speeds"):
-            raise ValueError("queries and keys with a norm, or keys that are values, take a rotation or no position encoding")
+            raise ValueError("queries and keys with a norm, keys that are values or another layer's keys take a rotation or no position encoding")
         return True
 
     def _prepare(self, ctx: StepContext, raw: torch.Tensor, slot: torch.Tensor, group: int, call) -> torch.Tensor:
         """[queries | gate] in the compute dtype from the product's 32-bit rows; keys and values into the cache."""
+        if self.shared_kv and call.write:
+            raise ValueError("a layer without keys and values of its own cannot write its cache slot")
         rot = self.position
         norm = self.qk_norm
         q = ctx.buf("q_ready", raw.shape[0], self.q_cols + self.gate_cols, ctx.dtype)
-        ops.attn_prepare(raw, self.n_heads, self.n_kv_heads, self.head_dim, self.v_head_dim,
+        ops.attn_prepare(raw, self.n_heads, 0 if self.shared_kv else self.n_kv_heads, self.head_dim, self.v_head_dim,
                          None if norm is None else self.q_gain, None if norm is None else self.k_gain,
                          0.0 if norm is None else norm.eps, True if norm is None else norm.whole, ctx.positions,
                          None if rot is None else rot.speeds, 0 if rot is None else rot.dims,
@@ -255,7 +267,7 @@ class CausalSelfAttention(Mixer):
             ops.paged_attention_rel(ctx, qkv if self.out_gate else qkv[:, :self.q_cols], slot, group, self.n_heads, self.n_kv_heads, self.head_dim,
                                     self.v_head_dim, self.scale, self.window, self.dist_bias, self.temp_coef,
                                     self.temp_every, o, softcap=self.softcap, keep_first=self.keep_first, sink=self.sink,
-                                    gate_col=gate_off if self.out_gate else -1)
+                                    gate_col=gate_off if self.out_gate else -1, chunk=self.chunk)
         else:
             ops.paged_attention(ctx, qkv[:, :self.q_cols], slot, group, self.n_heads, self.scale, self.window, o)
         if ctx.debug_hook is not None:      # the reference's stage names (CausalSelfAttention.java:299-301,384)

@@ -28,7 +28,7 @@ The reference wires the same roles through constructor arguments of one block cl
 """
 from __future__ import annotations
 
-from dataclasses import dataclass
+from dataclasses import dataclass, replace
 from typing import Callable, Dict, List, Optional, Tuple
 
 import torch
@@ -39,13 +39,27 @@ class KVNeed:
     """Pages of keys (``head_dim`` a head) and values (``v_head_dim`` a head; None: the keys' size).
     ``values_in_keys``: nothing is kept for the values, they are the first ``v_head_dim`` entries of the key rows
     (a page is then ``n_kv_heads * page`` rows of ``head_dim`` entries, token by token).
-    ``keep_first``: with a window, the first so many positions of a sequence stay readable for good."""
+    ``keep_first``: with a window, the first so many positions of a sequence stay readable for good.
+    ``chunk``: in place of a window, a row reads the keys of its own chunk of so many positions only."""
     n_kv_heads: int
     head_dim: int
     window: Optional[int] = None
     v_head_dim: Optional[int] = None
     values_in_keys: bool = False
     keep_first: int = 0
+    chunk: Optional[int] = None
+
+    def joined(self, other: "KVNeed") -> "KVNeed":
+        """The need of a cache slot that serves two layers with masks of their own: what either of them still reads is
+        kept.  (A chunk of n positions lies inside a window of n.)  Sizes must agree."""
+        if (self.n_kv_heads, self.head_dim, self.v_head_dim, self.values_in_keys) != \
+                (other.n_kv_heads, other.head_dim, other.v_head_dim, other.values_in_keys):
+            raise ValueError(f"one cache slot cannot serve {self} and {other}")
+        keep = max(self.keep_first, other.keep_first)
+        if (self.window, self.chunk) == (other.window, other.chunk):
+            return replace(self, keep_first=keep)
+        spans = [n.chunk or n.window for n in (self, other)]
+        return replace(self, chunk=None, window=None if None in spans else max(spans), keep_first=keep)
 
 
 @dataclass(frozen=True)

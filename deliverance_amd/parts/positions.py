@@ -3,6 +3,7 @@
 to queries and keys (its rotary step is skipped: core/.../generator/CausalSelfAttention.java:341)."""
 from __future__ import annotations
 
+from ..config.specs import LinearSpeedsSpec
 from .base import PositionEncoding, register_position, to_vector
 
 
@@ -51,7 +52,8 @@ def ramped_speeds(speeds, dims: int, base: float, scaling):
 class RotaryPositions(PositionEncoding):
     """Pairs of a vector's first ``dims`` entries turned by position * base^(-2i / dims) (``RotarySpec``).  The
     speeds are worked out once in double precision; the kernel takes the sine and cosine of the double angle.
-    With ``spec.scaling`` the speeds are ramped (``ramped_speeds``) and the turned pairs grow by ``magnitude``."""
+    With ``spec.scaling`` the speeds are divided by one factor (``LinearSpeedsSpec``), or ramped (``ramped_speeds``), in
+    which case the turned pairs grow by ``magnitude``."""
 
     def __init__(self, spec, params=None, dtype=None, device=None):
         import torch
@@ -63,7 +65,11 @@ class RotaryPositions(PositionEncoding):
         speeds = [self.base ** (-2.0 * i / self.dims) for i in range(self.dims // 2)]
         self.magnitude = 1.0
         scaling = getattr(spec, "scaling", None)
-        if scaling is not None and self.dims:
+        if isinstance(scaling, LinearSpeedsSpec):
+            if not (float(scaling.factor) > 0.0):
+                raise ValueError(f"speed scaling needs a positive factor, found {scaling.factor}")
+            speeds = [f / float(scaling.factor) for f in speeds]
+        elif scaling is not None and self.dims:
             speeds, self.magnitude = ramped_speeds(speeds, self.dims, self.base, scaling)
         self.speeds = torch.tensor(speeds or [0.0], dtype=torch.float64, device=device)
 
