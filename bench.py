@@ -18,7 +18,8 @@ its fraction of the roofline; `--no-extra` leaves those two out.  Prints ONE JSO
 vocabulary, feed-forward parameters that a token uses): decode at batch 1, 8 and 64 and the prefill of 2 x 1,024
 tokens for both, at the layer sizes of GPT-2 124M and 355M, one JSON line; with `--profile-stages` also both
 models' kernel tables (stderr).  `--design pedatar` does the same for a third design beside Virudra (the closest
-of the engine's models to it), `--design pafolorn` for a fourth beside Pedatar, and `--design salivik` for a fifth beside Pedatar.
+of the engine's models to it), `--design pafolorn` for a fourth beside Pedatar, `--design salivik` for a fifth beside Pedatar, and
+`--design luvatar` for a sixth beside Pafolorn.
 """
 import argparse
 import json
@@ -463,6 +464,111 @@ def salivik_compare(args):
     return 0
 
 
+def luvatar_config(name, n_positions=1024):
+    """A Luvatar of GPT-2 ``name``'s sizes: as many layers, gated linear attention and chunked attention in turn.  Gated
+    linear attention: GPT-2's heads with 64 key and 64 value entries each, tau 16, decays through a low rank of 16.
+    Attention: GPT-2's heads of 64 entries on a quarter as many key heads, all entries rotated with speeds divided by 4,
+    chunks of 1,024 positions; every second attention layer reads the keys and values of the one before it.  Gated
+    feed-forwards of 8/3 of the width, which holds what GPT-2's of four times the width holds."""
+    g = MODELS[name]
+    E, H = g["n_embd"], g["n_head"]
+    gla = {"heads": H, "dim": 64, "vdim": 64, "tau": 16.0, "a_rank": 16}
+    att = {"heads": H, "kv_heads": H // 4, "dim": 64, "vdim": 64, "scale": 64 ** -0.5, "mask": {"size": 1024},
+           "rot": {"base": 10000.0, "dims": 64, "scaling": {"factor": 4.0}}}
+    mlp = {"kind": "dense", "ff": 8 * E // 3 // 64 * 64}
+    layers = [{"type": "gla", "mixer": gla, "mlp": mlp} if i % 2 == 0 else
+              {"type": "attention", "mixer": att if i % 4 == 1 else dict(att, kv_from=i - 2), "mlp": mlp}
+              for i in range(g["n_layer"])]
+    return {"architecture": "Luvatar", "vocab": 50257, "width": E, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "layers": layers, "max_positions": n_positions,
+            # what decode_run and prefill_run read
+            "vocab_size": 50257, "n_positions": n_positions, "n_layer": g["n_layer"], "n_embd": E}
+
+
+def _luvatar_layer_params(c, L):
+    E, m = c["width"], L["mixer"]
+    qk, v = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+    if L["type"] == "gla":
+        n = E * (2 * qk + 2 * v) + v * E + m["a_rank"] * (E + qk)
+    else:
+        n = E * (qk + v) + v * E + (0 if m.get("kv_from") is not None else E * m["kv_heads"] * (m["dim"] + m["vdim"]))
+    return n + (3 * E * L["mlp"]["ff"] if L["mlp"] else 0)
+
+
+def luvatar_step_bytes(c, el, batch, ctx_mean):
+    """What a decode step must read: every matrix once, the states of gated linear attention (read and written, 32-bit),
+    and the keys and values of the chunks' parts behind a position (half a chunk on average, once a chunk is full)."""
+    n, extra = c["vocab"] * c["width"], 0
+    for L in c["layers"]:
+        n += _luvatar_layer_params(c, L)
+        m = L["mixer"]
+        if L["type"] == "gla":
+            extra += batch * 2 * 4 * m["heads"] * m["vdim"] * m["dim"]
+        else:
+            size = m["mask"]["size"]
+            seen = ctx_mean / 2 if ctx_mean < size else (ctx_mean - ctx_mean // size * size)
+            extra += batch * seen * m["kv_heads"] * (m["dim"] + m["vdim"]) * el
+    return n * el + extra
+
+
+def luvatar_step_flops(c, seq_lens_new):
+    """Matrix-product flops of a step (the parameters a token uses, twice), the attention's two products over the keys
+    that each row sees, and gated linear attention's four operations a state entry and token."""
+    n = sum(seq_lens_new)
+    fl = 2 * len(seq_lens_new) * c["width"] * c["vocab"]
+    for L in c["layers"]:
+        fl += 2 * n * _luvatar_layer_params(c, L)
+        m = L["mixer"]
+        if L["type"] == "gla":
+            fl += 4 * n * m["heads"] * m["vdim"] * m["dim"]
+        else:
+            pairs = sum(sum(i % m["mask"]["size"] + 1 for i in range(t)) for t in seq_lens_new)
+            fl += 2 * pairs * m["heads"] * (m["dim"] + m["vdim"])
+    return fl
+
+
+def luvatar_compare(args):
+    """Decode and prefill of Luvatar beside Pafolorn (the closest of the engine's models: a linear recurrence with a decay
+    per key channel, bounded attention with normalised queries and keys, a norm behind each part and none in front, the
+    embedding table as the head) at the layer sizes of GPT-2 124M and 355M; one JSON line."""
+    import numpy as np
+    el, dkey = 2, "bf16"
+    out = {"metric": "decode tok/s at batch 8 of Luvatar at GPT-2 124M layer sizes (beside Pafolorn at the same sizes: see points)",
+           "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": dkey, "steps": args.steps, "warmup": args.warmup,
+           "data": "synthetic (random weights drawn on the GPU, uniform-random token ids)", "points": {}, "points_frac": {}}
+    of = {"pafolorn": (pafolorn_config, pafolorn_step_bytes, pafolorn_step_flops),
+          "luvatar": (luvatar_config, luvatar_step_bytes, luvatar_step_flops)}
+    for size in ("124m", "355m"):
+        for design in ("pafolorn", "luvatar"):
+            rng = np.random.default_rng(0)
+            config, nbytes, flops = of[design]
+            cfg = config(size)
+            model = engine_from_gpu_weights(cfg, "bfloat16", 64, kernels=args.kernels)
+            key = f"{design}_{size}"
+            for b in (1, 8, 64):
+                steps = min(args.steps, 128)
+                d, cm = decode_run(model, cfg, rng, b, args.prompt_len, steps, 8)
+                out["points"][f"{key}_decode_b{b}"] = round(b * steps / d, 1)
+                out["points_frac"][f"{key}_decode_b{b}"] = round(nbytes(cfg, el, b, cm) / (d / steps) / 1e9 / HBM_GBS, 4)
+            for n, length in ((2, 1024), (8, 1024)):
+                pf = prefill_run(model, cfg, rng, dkey, n, length, flops=flops(cfg, [length] * n))
+                out["points"][f"{key}_prefill_{n * length}"] = pf["value"]
+                out["points_frac"][f"{key}_prefill_{n * length}"] = pf["frac"]
+            if args.profile_stages:
+                print(f"==== {key}", file=sys.stderr)
+                kernel_table(model, cfg, rng, args.batch, args.prompt_len)
+            del model
+    out["value"] = out["points"]["luvatar_124m_decode_b8"]
+    out["config"] = {"model": "luvatar beside pafolorn at gpt2-124m and gpt2-355m layer sizes", "global_batch": 8,
+                     "prompt_len": args.prompt_len,
+                     "luvatar": "gated linear attention (GPT-2's heads, 64 x 64 states, decays through a low rank of 16) and "
+                                "attention inside chunks of 1,024 positions (GPT-2's heads on a quarter as many key heads, all "
+                                "entries rotated, sink, output gate; every second one on the keys and values of the one before) in "
+                                "turn; gated feed-forwards of 8/3 width", "parallelism": "single-gpu"}
+    print(json.dumps(out))
+    return 0
+
+
 def design_compare(args):
     """Decode and prefill of another design beside its like at equal sizes; one JSON line."""
     if args.design == "pedatar":
@@ -471,6 +577,8 @@ def design_compare(args):
         return pafolorn_compare(args)
     if args.design == "salivik":
         return salivik_compare(args)
+    if args.design == "luvatar":
+        return luvatar_compare(args)
     return virudra_compare(args)
 
 
@@ -677,11 +785,11 @@ def main():
     ap.add_argument("--pool-tokens", type=int, default=None,
                     help="mixed workload: tokens of cache the pool holds (default: every request at full length; fewer force "
                          "requests out of the cache and back, which the line reports as preemptions)")
-    ap.add_argument("--design", default="gpt2", choices=["gpt2", "virudra", "pedatar", "pafolorn", "salivik"],
+    ap.add_argument("--design", default="gpt2", choices=["gpt2", "virudra", "pedatar", "pafolorn", "salivik", "luvatar"],
                     help="virudra: that design beside GPT-2 at equal sizes (decode at batch 1, 8, 64 and the prefill of 2,048 "
                          "tokens, at 124M and 355M layer sizes) instead of the default workload; pedatar: that design beside "
                          "Virudra, likewise; pafolorn: that design beside Pedatar, likewise; "
-                         "salivik: that design beside Pedatar, likewise")
+                         "salivik: that design beside Pedatar, likewise; luvatar: that design beside Pafolorn, likewise")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed"],
                     help="mixed: only the mixed workload, on --model (64 requests with prompts of 16 to 895 tokens arrive at "
                          "once, prompt portions of 512 tokens run beside the decoding of the others, 128 new tokens each)")
@@ -693,7 +801,7 @@ def main():
     import numpy as np
     from deliverance_amd.random_model import random_model
 
-    if args.design in ("virudra", "pedatar", "pafolorn", "salivik"):
+    if args.design != "gpt2":
         return design_compare(args)
     cfg = model_config(args.model, args.layers, args.n_positions)
     full_layers = MODELS[args.model]["n_layer"]

@@ -116,6 +116,12 @@ _ARGTYPES = {
     "da_retention": [_VP, _I, _I, _I, _I, _I, _VP, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP,
                      ctypes.c_long, _VP],
     "da_gla_walk": [_VP, _I, _I, _I, _I, _I, _VP, _I, _VP, _F, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP],
+    "da_gla_serve_takes": [_I, _I, _I],
+    "da_gla_low_takes": [_I],
+    "da_gla_decode": [_VP, _I, _I, _I, _I, _I, _I, _VP, _I, _VP, _I, _VP, _F, _F, _VP, _I, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I,
+                      _I, _I, _I, _I, _I, _I, _VP],
+    "da_gla_chunked": [_VP, _I, _I, _I, _I, _I, _I, _VP, _I, _VP, _I, _VP, _F, _F, _VP, _I, _F, _VP, ctypes.c_long, _VP, _VP, _VP, _I,
+                       _I, _I, _I, _I, _I, _I, _I, _VP, ctypes.c_long, _VP],
     "da_moe_top": [_VP, _I, _VP, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_softcap": [_VP, ctypes.c_long, _F, _VP],
     "da_moe_route": [_VP, _VP, _I, _VP, _I, _I, _I, _I, _VP, _VP, _VP, _I, _I, _VP, _VP, _VP],
@@ -1530,6 +1536,66 @@ def gla_walk(ctx, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, raw: to
                                   _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(o), o.stride(0), ctx.n_seqs, H, D, Dv,
                                   int(bool(write)), _stream()))
     return o
+
+
+GLA_CHUNK = 64               # tokens of a chunk of the form for portions
+
+
+def gla_serve_takes(proj: torch.Tensor, state: torch.Tensor, head_dim: int, v_head_dim: int) -> bool:
+    """Whether the forms for bfloat16 serving take these sizes (and the kernel mode allows them)."""
+    return (_MODE == "tuned" and proj.dtype == torch.bfloat16 and state.data_ptr() % 16 == 0
+            and bool(_lib().da_gla_serve_takes(head_dim, v_head_dim, state.stride(0))))
+
+
+def gla_low_takes(rank: int, up: torch.Tensor) -> bool:
+    """Whether those forms multiply a low rank of so many numbers up themselves."""
+    return up.dtype == torch.bfloat16 and up.data_ptr() % 8 == 0 and bool(_lib().da_gla_low_takes(rank))
+
+
+def gla_serve(ctx, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_off: int, low_off: int,
+              up: Optional[torch.Tensor], raw: Optional[torch.Tensor], bias: torch.Tensor, tau: float, q_scale: float,
+              gain: torch.Tensor, eps: float, state: torch.Tensor, y: torch.Tensor, n_heads: int, head_dim: int,
+              v_head_dim: int, write: bool = True) -> torch.Tensor:
+    """Gated linear attention of a step in bfloat16 serving, up to the output projection's input: the recurrence of
+    ``gla_walk``, then every head's read-out over its root mean square, times ``gain`` [Dv] and silu(gate).  ``proj``
+    [N, ...] holds q, k, v, the gate (H * Dv from ``gate_off``) and, with ``up`` [H * D, rank], the low rank's numbers
+    from ``low_off``; else ``raw`` [N, H * D] holds the decays' arguments.  One-token sequences and portions go to a
+    kernel (or three) each; ``y`` [N, H * Dv] in bfloat16."""
+    _dev(proj, up, raw, bias, gain, state, y)
+    _rows_2d(proj, "proj"); _rows_2d(y, "y")
+    N, H, D, Dv = proj.shape[0], n_heads, head_dim, v_head_dim
+    ld = _state_args(state, "gla_serve")
+    rank = 0 if up is None else up.shape[1]
+    _need(proj.dtype == y.dtype == torch.bfloat16 and y.shape[0] == N and y.shape[1] >= H * Dv, "gla_serve: proj and y must be bfloat16 of N rows")
+    _need(min(q_off, k_off, v_off, gate_off) >= 0 and max(q_off, k_off) + H * D <= proj.shape[1]
+          and max(v_off, gate_off) + H * Dv <= proj.shape[1], "gla_serve: q, k, v and gate leave the row")
+    _need((up is None) != (raw is None), "gla_serve: the decays' arguments come as rows or from a low rank")
+    if up is not None:
+        _need(up.dtype == torch.bfloat16 and up.is_contiguous() and up.shape[0] == H * D
+              and low_off >= 0 and low_off + rank <= proj.shape[1], "gla_serve: up must be bfloat16 [H * D, rank]")
+    else:
+        _rows_2d(raw, "raw")
+        _need(raw.dtype == torch.float32 and raw.shape[0] == N and raw.shape[1] >= H * D, "gla_serve: raw must be float32 [N, H * D]")
+    _need(bias.dtype == torch.float32 and bias.is_contiguous() and bias.numel() == H * D and gain.is_contiguous()
+          and gain.numel() == Dv, "gla_serve: bias [H * D] float32 and gain [Dv]")
+    _need(ld >= H * Dv * D, "gla_serve: the state row is too short")
+    _need(ctx.q_start.numel() >= ctx.n_seqs + 1 and ctx.state_slots.numel() >= ctx.n_seqs, "gla_serve: the step's arrays are too short")
+    args = (_ptr(proj), proj.stride(0), int(q_off), int(k_off), int(v_off), int(gate_off), int(low_off), _ptr(up), rank,
+            _ptr(raw), 0 if raw is None else raw.stride(0), _ptr(bias), float(tau), float(q_scale), _ptr(gain), _dt(gain), float(eps),
+            _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(y), y.stride(0))
+    nd, S = ctx.n_decode, ctx.n_seqs
+    per = ((2 * H * D + 3 * H * Dv + rank) * 2 + (0 if raw is None else H * D * 4), 2 * H * Dv * D * 4)   # bytes a token, a sequence
+    if nd:
+        with _timed("gla_decode", nd * (per[0] + per[1]), 4 * nd * H * D * Dv, "fp32"):
+            _check(_lib().da_gla_decode(*args, 0, nd, H, D, Dv, int(bool(write)), _stream()))
+    if S > nd:
+        longest = int(ctx.max_query_len)
+        cells = (S - nd) * -(-longest // GLA_CHUNK) * H * D * (Dv + 1)
+        scratch = ctx.buf("gla_scratch", 1, cells, torch.float32) if cells else None
+        with _timed("gla_chunked", (N - nd) * per[0] + (S - nd) * per[1], 4 * (N - nd) * H * D * Dv, "fp32"):
+            _check(_lib().da_gla_chunked(*args, nd, S - nd, H, D, Dv, int(bool(write)), longest, _ptr(scratch),
+                                         0 if scratch is None else scratch.numel(), _stream()))
+    return y
 
 
 # ------------------------------------------------------------------------------- short filter and scan

@@ -12,7 +12,7 @@ state is one 32-bit row [ S: heads x v_head_dim x head_dim ]; kernels find it th
 so decode steps can be recorded.
 
 Products of a step: [q | k | v | gate | the decay's low rank] in the compute dtype (one product), the low rank's second
-factor, and the output projection.
+factor (in bfloat16 serving inside the recurrence's kernels for ranks up to 32), and the output projection.
 """
 from __future__ import annotations
 
@@ -65,14 +65,24 @@ class GatedLinearAttention(Mixer):
         N = h.shape[0]
         proj = ctx.buf("gla_in", N, self.in_weight.shape[0], ctx.dtype)
         ops.linear(h, self.in_weight, None, proj)
-        raw = ctx.buf("gla_decay", N, self.qk_cols, torch.float32)          # unrounded sums
-        ops.linear(proj[:, self.low_off:self.low_off + self.rank], self.decay_up, None, raw)
-        o = ctx.buf("gla_o", N, self.v_cols, torch.float32)
-        ops.gla_walk(ctx, proj, 0, self.qk_cols, self.v_off, raw, self.decay_bias, self.tau, self.q_scale,
-                     ctx.cache.state[call.cache], o, self.H, self.D, self.Dv, write=call.write)
+        state = ctx.cache.state[call.cache]
         y = ctx.buf("gla_y", N, self.v_cols, ctx.dtype)
-        ops.delta_gate_norm(o, proj[:, self.gate_off:self.gate_off + self.v_cols], self.out_norm, self.eps, "silu", self.H,
-                            self.Dv, y)
+        serve = ops.gla_serve_takes(proj, state, self.D, self.Dv)
+        raw = None
+        if not (serve and ops.gla_low_takes(self.rank, self.decay_up)):
+            raw = ctx.buf("gla_decay", N, self.qk_cols, torch.float32)      # unrounded sums
+            ops.linear(proj[:, self.low_off:self.low_off + self.rank], self.decay_up, None, raw)
+        if serve:
+            # the decays, the recurrence, the read-out's norm and the gate together
+            ops.gla_serve(ctx, proj, 0, self.qk_cols, self.v_off, self.gate_off, self.low_off,
+                          self.decay_up if raw is None else None, raw, self.decay_bias, self.tau, self.q_scale, self.out_norm,
+                          self.eps, state, y, self.H, self.D, self.Dv, write=call.write)
+        else:
+            o = ctx.buf("gla_o", N, self.v_cols, torch.float32)
+            ops.gla_walk(ctx, proj, 0, self.qk_cols, self.v_off, raw, self.decay_bias, self.tau, self.q_scale, state, o,
+                         self.H, self.D, self.Dv, write=call.write)
+            ops.delta_gate_norm(o, proj[:, self.gate_off:self.gate_off + self.v_cols], self.out_norm, self.eps, "silu",
+                                self.H, self.Dv, y)
         if ctx.debug_hook is not None:
             ctx.emit(call.layer, "attention_value", y)
         ops.linear(y, self.out_weight, None, x, accumulate=ctx.part_accumulate)

@@ -142,6 +142,7 @@ namespace simt {
 void mfma_32x32x16(const void* a, const void* b, float* c);
 void mfma_16x16x32(const void* a, const void* b, float* c);
 void mfma_4x4x4(const void* a, const void* b, float* c);
+void mfma_16x16x4_f32(const void* a, const void* b, float* c);
 }
 static inline simt_floatx16 simt_mfma_32x32x16(simt_bf16x8 a, simt_bf16x8 b, simt_floatx16 c) {
   simt::mfma_32x32x16(&a, &b, (float*)&c);
@@ -155,6 +156,11 @@ static inline simt_floatx4 simt_mfma_4x4x4(simt_shortx4 a, simt_shortx4 b, simt_
   simt::mfma_4x4x4(&a, &b, (float*)&c);
   return c;
 }
+static inline simt_floatx4 simt_mfma_16x16x4_f32(float a, float b, simt_floatx4 c) {
+  simt::mfma_16x16x4_f32(&a, &b, (float*)&c);
+  return c;
+}
+#define __builtin_amdgcn_mfma_f32_16x16x4f32(a, b, c, x, y, z) simt_mfma_16x16x4_f32((a), (b), (c))
 #define __builtin_amdgcn_mfma_f32_32x32x16_bf16(a, b, c, x, y, z) simt_mfma_32x32x16((a), (b), (c))
 #define __builtin_amdgcn_mfma_f32_16x16x32_bf16(a, b, c, x, y, z) simt_mfma_16x16x32((a), (b), (c))
 #define __builtin_amdgcn_mfma_f32_4x4x4bf16_1k(a, b, c, x, y, z) simt_mfma_4x4x4((a), (b), (c))

@@ -179,6 +179,18 @@ void mfma_4x4x4(const void* a, const void* b, float* c) {
   }
 }
 
+// 16x16x4 in 32-bit: lane l gives row / column l % 16 and k = l / 16; it receives rows 4 * (l / 16) + r, column l % 16.
+void mfma_16x16x4_f32(const void* a, const void* b, float* c) {
+  frag_publish(a, b, 4);
+  const int l = lane_id(), col = l % 16;
+  for (int r = 0; r < 4; ++r) {
+    const int row = 4 * (l / 16) + r;
+    float s = c[r];
+    for (int k = 0; k < 4; ++k) s += *(const float*)frag_a(row + 16 * k) * *(const float*)frag_b(col + 16 * k);
+    c[r] = s;
+  }
+}
+
 int dpp_source(int lane, int ctrl) {
   const int row = lane & ~15, in_row = lane & 15;
   if (ctrl >= 0 && ctrl <= 0xFF) return (lane & ~3) | ((ctrl >> (2 * (lane & 3))) & 3);     // quad_perm
