@@ -1580,21 +1580,23 @@ def gla_serve(ctx, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_
           and gain.numel() == Dv, "gla_serve: bias [H * D] float32 and gain [Dv]")
     _need(ld >= H * Dv * D, "gla_serve: the state row is too short")
     _need(ctx.q_start.numel() >= ctx.n_seqs + 1 and ctx.state_slots.numel() >= ctx.n_seqs, "gla_serve: the step's arrays are too short")
-    args = (_ptr(proj), proj.stride(0), int(q_off), int(k_off), int(v_off), int(gate_off), int(low_off), _ptr(up), rank,
-            _ptr(raw), 0 if raw is None else raw.stride(0), _ptr(bias), float(tau), float(q_scale), _ptr(gain), _dt(gain), float(eps),
-            _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(y), y.stride(0))
+
+    def args():
+        return (_ptr(proj), proj.stride(0), int(q_off), int(k_off), int(v_off), int(gate_off), int(low_off), _ptr(up), rank,
+                _ptr(raw), 0 if raw is None else raw.stride(0), _ptr(bias), float(tau), float(q_scale), _ptr(gain), _dt(gain),
+                float(eps), _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(y), y.stride(0))
+
     nd, S = ctx.n_decode, ctx.n_seqs
     per = ((2 * H * D + 3 * H * Dv + rank) * 2 + (0 if raw is None else H * D * 4), 2 * H * Dv * D * 4)   # bytes a token, a sequence
     if nd:
         with _timed("gla_decode", nd * (per[0] + per[1]), 4 * nd * H * D * Dv, "fp32"):
-            _check(_lib().da_gla_decode(*args, 0, nd, H, D, Dv, int(bool(write)), _stream()))
+            _check(_lib().da_gla_decode(*args(), 0, nd, H, D, Dv, int(bool(write)), _stream()))
     if S > nd:
         longest = int(ctx.max_query_len)
-        cells = (S - nd) * -(-longest // GLA_CHUNK) * H * D * (Dv + 1)
-        scratch = ctx.buf("gla_scratch", 1, cells, torch.float32) if cells else None
+        scratch = ctx.buf("gla_scratch", (S - nd) * -(-longest // GLA_CHUNK), H * D * (Dv + 1), torch.float32)
         with _timed("gla_chunked", (N - nd) * per[0] + (S - nd) * per[1], 4 * (N - nd) * H * D * Dv, "fp32"):
-            _check(_lib().da_gla_chunked(*args, nd, S - nd, H, D, Dv, int(bool(write)), longest, _ptr(scratch),
-                                         0 if scratch is None else scratch.numel(), _stream()))
+            _check(_lib().da_gla_chunked(*args(), nd, S - nd, H, D, Dv, int(bool(write)), longest, _ptr(scratch),
+                                         scratch.numel(), _stream()))
     return y
 
 

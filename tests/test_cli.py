@@ -86,6 +86,21 @@ def test_random_then_inspect_a_design_with_a_loop_of_layers(tmp_path):
     assert "l0.mix.v" in p.stdout and "l2.mix.v" not in p.stdout and "embed.norm" in p.stdout
 
 
+def test_random_then_inspect_a_design_with_layers_on_others_keys(tmp_path):
+    """... and on a Luvatar configuration: a layer on another's keys and values has neither tensors nor a slot for them."""
+    from luvatar_models import CONFIG_A
+    cfg = tmp_path / "config.json"
+    cfg.write_text(json.dumps(CONFIG_A))
+    out = tmp_path / "model"
+    p = run("random", "--config", str(cfg), "--seed", "8", "--out", str(out))
+    assert p.returncode == 0, p.stderr
+    p = run("inspect", str(out))
+    assert p.returncode == 0, p.stderr
+    assert f"architecture Luvatar: 4 layers, width {CONFIG_A['width']}, vocabulary {CONFIG_A['vocab']}" in p.stdout
+    assert "4 layer calls, 4 cache slots" in p.stdout
+    assert "l1.mix.a2.b" in p.stdout and "l0.mix.k.norm" in p.stdout and "l2.mix.sink" in p.stdout and "l2.mix.k" not in p.stdout
+
+
 def test_help_names_the_reference_options():
     p = run("generate", "--help")
     for opt in ("--model", "--working-dtype", "--max-tokens", "--temperature", "--seed", "--warmup-cases", "--max-cases",

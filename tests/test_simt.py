@@ -53,6 +53,12 @@ RUNS = {
                ["tests/test_salivik_gpu.py", "-n", "3", "-m", QUICK, "-k",
                 "not (portions and sizes0) and not token_by_token and not (mixed_batches and (S or float32)) "
                 "and not ((portions or whole_prompts) and S and float32)"],
+    # a sixth design's kernels and parts (gated linear attention's walk and its forms for serving, attention inside
+    # chunks and on another layer's keys) and its models through the step function
+    "luvatar": ["tests/test_luvatar_gpu.py", "-n", "4"] if FULL else
+               ["tests/test_luvatar_gpu.py", "-n", "3", "-m", QUICK, "-k",
+                "not (portions and sizes0) and not (edge and float32) and not ((portions or whole_prompts) and A and float32) "
+                "and not (mixed_batches and float32)"],
     "replay": ["tests/test_replay_gpu.py", "-n", "4"] if FULL else
               ["tests/test_replay_gpu.py", "-n", "2", "-k", "(mixed and (A or B) and not 32) or want_subset or errors_leave or first_tokens"],
     # inner sizes of 32 in an engine step: qkv and fc of seed 11 (and, in the full run, proj of seed 5)
