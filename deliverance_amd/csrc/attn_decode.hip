@@ -20,7 +20,10 @@
 // Compiled a second time with DEC_REL (attn_decode_rel.hip) the kernel also takes what some designs put on the
 // scores: a bias by the distance between query and key (a table [Hq][n_dist], 32-bit, the last entry for every
 // larger distance) and a query temperature 1 + t_coef * ln(floor((p + 1) / t_every) + 1) that multiplies the
-// scale.  The plain build has none of that code.
+// scale; chunks of positions in place of a window (a row sees the keys of its own chunk only); a sink, one number a head
+// whose exponential joins the softmax's denominator, without a key or a value and not scaled; and a gate, rows like out,
+// of which o is multiplied with the logistic function.  The last two act once, after everything has been merged.  The
+// plain build has none of that code.
 #include "common.h"
 
 #define DEC_MAX_D 256
@@ -28,20 +31,41 @@
 #ifdef DEC_REL
 #define DEC_KERNEL attn_decode_rel_kernel
 #define DEC_MERGE_KERNEL attn_decode_rel_merge_kernel
-#define DEC_REL_PARAMS , const float* __restrict__ rel_bias, int n_dist, float t_coef, int t_every
-#define DEC_REL_DECL , const float* rel_bias, int n_dist, float t_coef, int t_every
-#define DEC_REL_ARGS , rel_bias, n_dist, t_coef, t_every
+#define DEC_REL_PARAMS , const float* __restrict__ rel_bias, int n_dist, float t_coef, int t_every, int chunk DEC_END_PARAMS
+#define DEC_REL_DECL , const float* rel_bias, int n_dist, float t_coef, int t_every, int chunk, const float* sink, const bf16_t* gate, int gate_ld
+#define DEC_REL_ARGS , rel_bias, n_dist, t_coef, t_every, chunk DEC_END_ARGS
+#define DEC_END_PARAMS , const float* __restrict__ sink, const bf16_t* __restrict__ gate, int gate_ld
+#define DEC_END_ARGS , sink, gate, gate_ld
 #else
 #define DEC_KERNEL attn_decode_kernel
 #define DEC_MERGE_KERNEL attn_decode_merge_kernel
 #define DEC_REL_PARAMS
 #define DEC_REL_DECL
 #define DEC_REL_ARGS
+#define DEC_END_PARAMS
+#define DEC_END_ARGS
 #endif
 
 // e^x by the hardware's exp2 (two instructions; the library's expf is a dozen, and the merge of 16 wavefronts'
 // partial results takes 16 of them on the one wavefront that everything waits for)
 __device__ __forceinline__ float dec_exp(float x) { return __builtin_amdgcn_exp2f(x * 1.4426950408889634f); }
+
+#ifdef DEC_REL
+// What a finished row is multiplied with, from its maximum and its sum of weights: one over the sum, which the sink
+// joins; `shrink` is what its term makes of the weights' common scale.
+__device__ __forceinline__ float dec_inverse(float mm, float ll, bool with_sink, float s0) {
+  float shrink = 1.f;
+  if (with_sink) {
+    const float m_all = fmaxf(mm, s0);
+    shrink = mm == -INFINITY ? 0.f : dec_exp(mm - m_all);
+    ll = ll * shrink + dec_exp(s0 - m_all);
+  }
+  return ll > 0.f ? shrink / ll : 0.f;
+}
+__device__ __forceinline__ float dec_gate(float z) {
+  return __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-1.4426950408889634f * z));
+}
+#endif
 
 // Long contexts with few (sequence, head) pairs: the keys are also split over workgroups.  Workgroup
 // (pair, j) takes the keys j * span .. (j + 1) * span - 1 (span a multiple of 64) and leaves its
@@ -98,9 +122,20 @@ DEC_KERNEL(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ ca
       btv0[g] = bt[pg < max_blocks ? pg : max_blocks - 1];
     }
   }
+#ifdef DEC_REL
+  // asked for here, used at the end
+  const int gd = t < D ? t : 0;
+  const bf16_t graw = !SPLIT && gate ? gate[(size_t)s * gate_ld + h * D + gd] : (bf16_t)0;
+  const float s0 = !SPLIT && sink ? sink[h] : 0.f;
+#endif
   // the row's position is seq_lens[s] - 1; it sees the keys lo..p (of which this workgroup takes its share)
   const int p_row = seq_lens[s] - 1;
+#ifdef DEC_REL
+  const int lo_row = chunk > 0 ? (p_row > 0 ? p_row / chunk * chunk : 0)
+                               : ((window > 0 && p_row - window + 1 > 0) ? p_row - window + 1 : 0);
+#else
   const int lo_row = (window > 0 && p_row - window + 1 > 0) ? p_row - window + 1 : 0;
+#endif
   const int p = SPLIT ? (p_row < split0 + span - 1 ? p_row : split0 + span - 1) : p_row;
   const int lo = SPLIT ? (lo_row > split0 ? lo_row : split0) : lo_row;
 #ifdef DEC_REL
@@ -324,6 +359,17 @@ DEC_KERNEL(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ ca
     if (t == 0) { mine[D] = mm; mine[D + 1] = ll; }
     return;
   }
+#ifdef DEC_REL
+  const float inv = dec_inverse(mm, ll, sink != nullptr, s0);
+  if (t < D) {                                      // (a workgroup has at least 512 threads)
+    float o = 0.f;
+#pragma unroll
+    for (int w2 = 0; w2 < DEC_WAVES; ++w2) o += part_acc[w2][t] * f[w2];
+    o *= inv;
+    if (gate) o *= dec_gate(bf16_to_f32(graw));
+    out[(size_t)s * out_ld + h * D + t] = f32_to_bf16(o);
+  }
+#else
   const float inv = ll > 0.f ? 1.0f / ll : 0.f;     // a sequence of length 0 (padding) gives zeros
   for (int d = t; d < D; d += DEC_WAVES * DA_WAVE) {
     float o = 0.f;
@@ -331,12 +377,13 @@ DEC_KERNEL(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ ca
     for (int w2 = 0; w2 < DEC_WAVES; ++w2) o += part_acc[w2][d] * f[w2];
     out[(size_t)s * out_ld + h * D + d] = f32_to_bf16(o * inv);
   }
+#endif
 }
 
 // The partial results of a (sequence, head) pair, merged in ascending order of the shares.
 __global__ void __launch_bounds__(256)
 DEC_MERGE_KERNEL(const float* __restrict__ partial, int n_splits, int Hq, int D,
-                         bf16_t* __restrict__ out, int out_ld) {
+                         bf16_t* __restrict__ out, int out_ld DEC_END_PARAMS) {
   const int s = blockIdx.x / Hq, h = blockIdx.x % Hq;
   const float* mine = partial + (size_t)blockIdx.x * n_splits * (D + 2);
   float mm = -INFINITY;
@@ -346,13 +393,20 @@ DEC_MERGE_KERNEL(const float* __restrict__ partial, int n_splits, int Hq, int D,
     const float mj = mine[(size_t)j * (D + 2) + D];
     ll += mine[(size_t)j * (D + 2) + D + 1] * (mj == -INFINITY ? 0.f : dec_exp(mj - mm));
   }
+#ifdef DEC_REL
+  const float inv = dec_inverse(mm, ll, sink != nullptr, sink ? sink[h] : 0.f);
+#else
   const float inv = ll > 0.f ? 1.0f / ll : 0.f;
+#endif
   for (int d = threadIdx.x; d < D; d += blockDim.x) {
     float o = 0.f;
     for (int j = 0; j < n_splits; ++j) {
       const float mj = mine[(size_t)j * (D + 2) + D];
       o += mine[(size_t)j * (D + 2) + d] * (mj == -INFINITY ? 0.f : dec_exp(mj - mm));
     }
+#ifdef DEC_REL
+    if (gate) o *= dec_gate(bf16_to_f32(gate[(size_t)s * gate_ld + h * D + d]));
+#endif
     out[(size_t)s * out_ld + h * D + d] = f32_to_bf16(o * inv);
   }
 }
@@ -397,7 +451,7 @@ static int decode_launch(const void* q, int q_ld, const void* cache, const int* 
 #undef LAUNCH3
   if (n_splits > 1)
     hipLaunchKernelGGL(DEC_MERGE_KERNEL, dim3(S * Hq), dim3(D <= 64 ? 64 : (D <= 128 ? 128 : 256)), 0, st,
-                       partial, n_splits, Hq, D, (bf16_t*)out, out_ld);
+                       partial, n_splits, Hq, D, (bf16_t*)out, out_ld DEC_END_ARGS);
   return 0;
 }
 
@@ -413,10 +467,12 @@ static int rel_checks(const float* rel_bias, int n_dist, int t_every) {
 extern "C" int da_attn_decode_rel(const void* q, int q_ld, const void* cache, const int* block_table,
                                   int max_blocks, const int* seq_lens, int S, int Hq, int Hkv, int D, int page,
                                   float scale, int window, const float* rel_bias, int n_dist, float t_coef,
-                                  int t_every, void* out, int out_ld, int n_splits, void* workspace,
-                                  long workspace_bytes, void* stream) {
+                                  int t_every, int chunk, const float* sink, const void* gate, int gate_ld, void* out,
+                                  int out_ld, int n_splits, void* workspace, long workspace_bytes, void* stream) {
   if (decode_checks(q, q_ld, cache, max_blocks, S, Hq, Hkv, D, page, window, out_ld)) return 1;
   if (rel_checks(rel_bias, n_dist, t_every)) return 1;
+  DA_REQUIRE(chunk >= 0 && (chunk == 0 || window == 0), "attn_decode_rel: a window or chunks, not both");
+  DA_REQUIRE(!gate || gate_ld >= Hq * D, "attn_decode_rel: the gate's rows are too short");
   int span = 0;
   if (n_splits > 1) {
     DA_REQUIRE(n_splits <= 64, "attn_decode_rel: %d shares (2 to 64 are taken)", n_splits);
@@ -428,7 +484,8 @@ extern "C" int da_attn_decode_rel(const void* q, int q_ld, const void* cache, co
   }
   if (S == 0) return 0;
   decode_launch(q, q_ld, cache, block_table, max_blocks, seq_lens, S, Hq, Hkv, D, page, scale, window, out, out_ld,
-                n_splits > 1 ? n_splits : 1, span, (float*)workspace, (hipStream_t)stream, rel_bias, n_dist, t_coef, t_every);
+                n_splits > 1 ? n_splits : 1, span, (float*)workspace, (hipStream_t)stream, rel_bias, n_dist, t_coef, t_every,
+                chunk, sink, (const bf16_t*)gate, gate_ld);
   DA_CHECK_LAUNCH("attn_decode_rel");
   return 0;
 }

@@ -15,11 +15,92 @@
 //
 // A page of the cache slot holds Hkv * page * D keys (rows of D), then Hkv * Dv * page values (dimension-major);
 // slot_map[n] = page id * page + row, or -1 for a token whose keys are not kept.  One workgroup a token.
+//
+// Where norms are per head (or there are none), pairs are neighbours and rows are even, a second kernel does the same
+// with a head on 16, 32 or 64 neighbouring lanes, a lane a pair: the row is read once in 8-byte pieces, the norm's sum
+// goes over the head's lanes, and a lane works its sine and cosine out once for all of its heads.
 #include "common.h"
 
 #define PREP_THREADS 256
 #define PREP_MAX_HALF 128
 #define PREP_MAX_GROUPS 256
+
+// Sine and cosine of a double angle, in 32-bit: whole turns are taken off in double (2 pi as the sum of two doubles).
+__device__ __forceinline__ void prep_sincos(double a, float* s, float* c) {
+  const double n = rint(a * 0.15915494309189535);
+  const double r = fma(-n, 2.4492935982947064e-16, fma(-n, 6.283185307179586, a));
+  sincosf((float)r, s, c);
+}
+
+__device__ __forceinline__ void prep_store2(float* p, float a, float b) { *(float2*)p = make_float2(a, b); }
+__device__ __forceinline__ void prep_store2(bf16_t* p, float a, float b) { *(uint32_t*)p = pack2_bf16(a, b); }
+
+template <typename T, int LPH>
+__global__ void __launch_bounds__(PREP_THREADS)
+attn_prepare_heads_kernel(const float* __restrict__ raw, int ld, int Hq, int Hkv, int D, int Dv, const void* __restrict__ gq,
+                          int gq_dtype, const void* __restrict__ gk, int gk_dtype, float eps, const int* __restrict__ positions,
+                          const double* __restrict__ speeds, int dims, T* __restrict__ q_out, int q_ld, T* __restrict__ cache,
+                          const int* __restrict__ slot_map, int page, int pass_cols, float mag) {
+  constexpr int AT_ONCE = PREP_THREADS / LPH;          // heads side by side
+  constexpr int AHEAD = 4;                             // heads whose entries a lane asks for at once
+  const int n = blockIdx.x, t = threadIdx.x, i = t % LPH, g = t / LPH;
+  const float* row = raw + (size_t)n * ld;
+  const bool ok = 2 * i < D;
+  const int d = ok ? 2 * i : 0;
+  const int total = Hq + Hkv;
+  const int slot = (cache != nullptr && slot_map != nullptr) ? slot_map[n] : -1;
+  float gain[2][2] = {{1.f, 1.f}, {1.f, 1.f}};         // [queries, keys]
+  if (gq != nullptr) {
+    gain[0][0] = load_param(gq, gq_dtype, d); gain[0][1] = load_param(gq, gq_dtype, d + 1);
+    if (gk != nullptr) { gain[1][0] = load_param(gk, gk_dtype, d); gain[1][1] = load_param(gk, gk_dtype, d + 1); }
+  }
+  float2 x[AHEAD];
+  auto fetch = [&](int h0) {
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const int h = h0 + u * AT_ONCE + g;
+      x[u] = *(const float2*)(row + (size_t)(h < total ? h : 0) * D + d);
+    }
+  };
+  fetch(0);
+  float cs = 1.f, sn = 0.f;
+  if (2 * i < dims) {
+    prep_sincos((double)positions[n] * speeds[i], &sn, &cs);
+    cs *= mag; sn *= mag;
+  }
+  const long long pg = slot >= 0 ? slot / page : 0;
+  const int prow = slot >= 0 ? slot % page : 0;
+  T* kbase = cache + pg * ((long long)Hkv * page * (D + Dv));
+  for (int h0 = 0; h0 < total; h0 += AHEAD * AT_ONCE) {
+    if (h0) fetch(h0);
+#pragma unroll
+    for (int u = 0; u < AHEAD; ++u) {
+      const int h = h0 + u * AT_ONCE + g;
+      const bool is_q = h < Hq;
+      float a = ok ? x[u].x : 0.f, b = ok ? x[u].y : 0.f;
+      if (gq != nullptr) {
+        const float inv = 1.0f / sqrtf(group_sum<LPH>(fmaf(a, a, b * b)) / (float)D + eps);
+        a *= inv * (is_q ? gain[0][0] : gain[1][0]);
+        b *= inv * (is_q ? gain[0][1] : gain[1][1]);
+      }
+      const float ra = a * cs - b * sn, rb = b * cs + a * sn;
+      if (ok && h < total) {
+        if (is_q) prep_store2(q_out + (size_t)n * q_ld + h * D + d, ra, rb);
+        else if (slot >= 0) prep_store2(kbase + ((long long)(h - Hq) * page + prow) * D + d, ra, rb);
+      }
+    }
+  }
+  if (slot >= 0) {
+    const float* v = row + (size_t)total * D;
+    T* vb = kbase + (long long)Hkv * page * D;
+    for (int idx = t; idx < Hkv * Dv; idx += PREP_THREADS) from_f32(&vb[(long long)idx * page + prow], v[idx]);
+  }
+  const float* extra = row + (size_t)total * D + Hkv * Dv;
+  for (int idx = 2 * t; idx < pass_cols; idx += 2 * PREP_THREADS) {
+    const float2 e = *(const float2*)(extra + idx);
+    prep_store2(q_out + (size_t)n * q_ld + Hq * D + idx, e.x, e.y);
+  }
+}
 
 template <typename T>
 __global__ void __launch_bounds__(PREP_THREADS)
@@ -39,10 +120,10 @@ attn_prepare_kernel(const float* __restrict__ raw, int ld, int Hq, int Hkv, int 
   if (dims > 0) {
     const double p = (double)positions[n];
     for (int i = threadIdx.x; i < half; i += PREP_THREADS) {
-      double s, c;
-      sincos(p * speeds[i], &s, &c);
-      cs[i] = (float)c * mag;
-      sn[i] = (float)s * mag;
+      float s, c;
+      prep_sincos(p * speeds[i], &s, &c);
+      cs[i] = c * mag;
+      sn[i] = s * mag;
     }
   }
   if (normed) {
@@ -118,6 +199,26 @@ extern "C" int da_attn_prepare(const float* raw, int ld, int Hq, int Hkv, int D,
   DA_REQUIRE(whole || Hq + Hkv <= PREP_MAX_GROUPS, "attn_prepare: %d heads, %d norms are taken", Hq + Hkv, PREP_MAX_GROUPS);
   DA_REQUIRE(q_out != nullptr, "attn_prepare: the queries need a place");
   if (N == 0) return 0;
+  const int el = out_dtype == DA_BF16 ? 4 : 8;           // bytes of a pair of results
+  if (!whole && !v_from_k && (interleaved || dims == 0) && D % 2 == 0 && D <= 128 && (Hkv * Dv) % 2 == 0 && pass_cols % 2 == 0 &&
+      ld % 2 == 0 && q_ld % 2 == 0 && page % 2 == 0 && (uintptr_t)raw % 8 == 0 && (uintptr_t)q_out % el == 0 && (uintptr_t)cache % el == 0) {
+#define PREP_HEADS(T, L)                                                                                                     \
+  hipLaunchKernelGGL((attn_prepare_heads_kernel<T, L>), dim3(N), dim3(PREP_THREADS), 0, (hipStream_t)stream, raw, ld, Hq, Hkv, D, \
+                     Dv, gq, gq_dtype, gk, gk_dtype, eps, positions, speeds, dims, (T*)q_out, q_ld, (T*)cache, slot_map, page,    \
+                     pass_cols, mag)
+#define PREP_LANES(T)                        \
+  do {                                       \
+    if (D <= 32) PREP_HEADS(T, 16);          \
+    else if (D <= 64) PREP_HEADS(T, 32);     \
+    else PREP_HEADS(T, 64);                  \
+  } while (0)
+    if (out_dtype == DA_BF16) PREP_LANES(bf16_t);
+    else PREP_LANES(float);
+#undef PREP_LANES
+#undef PREP_HEADS
+    DA_CHECK_LAUNCH("attn_prepare");
+    return 0;
+  }
   if (out_dtype == DA_BF16)
     hipLaunchKernelGGL(attn_prepare_kernel<bf16_t>, dim3(N), dim3(PREP_THREADS), 0, (hipStream_t)stream, raw, ld, Hq, Hkv, D,
                        Dv, gq, gq_dtype, gk, gk_dtype, eps, whole, positions, speeds, dims, interleaved, (bf16_t*)q_out, q_ld,

@@ -95,7 +95,7 @@ _ARGTYPES = {
     "da_can_fuse_ln": [_I, _I, _I],
     "da_run_step": [_VP, _VP],
     "da_top_logprobs": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP],
-    "da_attn_decode_rel": [_VP, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _VP, _I, _I, _VP, ctypes.c_long, _VP],
+    "da_attn_decode_rel": [_VP, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _I, _VP, _VP, _I, _VP, _I, _I, _VP, ctypes.c_long, _VP],
     "da_attn_prefill_rel": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _VP, _I, _I, _VP],
     "da_rmsnorm": [_VP, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
     "da_rmsnorm_add": [_VP, _VP, _I, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
@@ -1004,9 +1004,15 @@ def _rel_bias_args(dist_bias, n_heads, name):
 def attention_decode_rel(q: torch.Tensor, cache_slot: torch.Tensor, block_table: torch.Tensor, seq_lens: torch.Tensor,
                          n_seqs: int, n_heads: int, scale: float, window: Optional[int],
                          dist_bias: Optional[torch.Tensor], temp_coef: float, temp_every: int, out: torch.Tensor,
-                         n_splits: int = 1, workspace: Optional[torch.Tensor] = None) -> torch.Tensor:
-    """``attention_decode`` with a bias by distance and a query temperature on the scores."""
-    Hkv, page, D = _attn_common(q, cache_slot, block_table, n_heads, out, "attention_decode_rel")
+                         n_splits: int = 1, workspace: Optional[torch.Tensor] = None, chunk: int = 0,
+                         sink: Optional[torch.Tensor] = None, gate_col: int = -1) -> torch.Tensor:
+    """``attention_decode`` with a bias by distance and a query temperature on the scores, chunks of positions in place
+    of a window, a sink (float32 [Hq]) and a gate that lies in q's rows from column ``gate_col`` on (q is then wider than
+    its Hq * D query entries)."""
+    cols = out.shape[1]
+    Hkv, page, D = _attn_common(q[:, :cols], cache_slot, block_table, n_heads, out, "attention_decode_rel")
+    gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, cols, cols, q, "attention_decode_rel")
+    _dev(sink)
     _need(q.shape[0] >= n_seqs and out.shape[0] >= n_seqs and block_table.shape[0] >= n_seqs,
           "attention_decode_rel: fewer rows than sequences")
     _need(seq_lens.dtype == torch.int32 and seq_lens.numel() >= n_seqs, "attention_decode_rel: seq_lens must be int32 [S]")
@@ -1020,8 +1026,8 @@ def attention_decode_rel(q: torch.Tensor, cache_slot: torch.Tensor, block_table:
         ws_bytes = workspace.numel() * 4
     _check(_lib().da_attn_decode_rel(_ptr(q), q.stride(0), _ptr(cache_slot), _ptr(block_table), block_table.shape[1],
                                      _ptr(seq_lens), n_seqs, n_heads, Hkv, D, page, float(scale), int(window or 0),
-                                     bias_ptr, n_dist, float(temp_coef), int(temp_every), _ptr(out), out.stride(0),
-                                     int(n_splits), _ptr(workspace) if n_splits > 1 else None, ws_bytes, _stream()))
+                                     bias_ptr, n_dist, float(temp_coef), int(temp_every), int(chunk), _ptr(sink), gate_ptr,
+                                     gate_ld, _ptr(out), out.stride(0), int(n_splits), _ptr(workspace) if n_splits > 1 else None, ws_bytes, _stream()))
     return out
 
 
@@ -1085,7 +1091,7 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
     """Attention of every row of the step with a bias by distance, a query temperature, values of their own
     size, a cap on the scores, first keys that a window keeps, a term without a key in the softmax's denominator
     (``sink``), a logistic gate on the result (``gate_col``: where the gate lies in q's rows) and chunks in place of a window
-    (``chunk``), each optional; the last three go with the matrix-core kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
+    (``chunk``), each optional; the last three go with the decode kernel, the matrix-core kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
     bias row that fits the prefill kernel's LDS copy, the one-token sequences go to the decode kernel and the
     portions to the prefill kernel (their forms with these extras); a cap, kept first keys and values of another size
     go to the matrix-core kernel for those (head sizes up to 128, no bias table, no temperature); 32-bit, the reference
@@ -1115,19 +1121,25 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
         return (keys * n_kv_heads * (D + v_head_dim) * el + rows * n_heads * (D + v_head_dim) * el,
                 2 * pairs * n_heads * (D + v_head_dim))
 
-    tuned = (_MODE == "tuned" and q.dtype == torch.bfloat16 and v_head_dim == D and D % 16 == 0
-             and softcap == 0.0 and not (window and keep_first) and sink is None and gate_col < 0
-             and not chunk and D <= PREFILL_REL_MAX_HEAD_DIM and cache_slot.dim() == 5 and q.stride(0) % 8 == 0
-             and q.data_ptr() % 16 == 0 and (dist_bias is None or dist_bias.shape[1] <= PREFILL_REL_MAX_DIST))
+    # what the decode kernel takes; the prefill kernel beside it takes the same without chunks, sink and gate
+    decode_tuned = (_MODE == "tuned" and q.dtype == torch.bfloat16 and v_head_dim == D and D % 16 == 0
+                    and softcap == 0.0 and not (window and keep_first)
+                    and D <= PREFILL_REL_MAX_HEAD_DIM and cache_slot.dim() == 5 and q.stride(0) % 8 == 0
+                    and q.data_ptr() % 16 == 0 and (dist_bias is None or dist_bias.shape[1] <= PREFILL_REL_MAX_DIST))
+    tuned = decode_tuned and sink is None and gate_col < 0 and not chunk
+
+    def decode_rows():
+        n_splits = decode_splits(nd, n_heads, bt.shape[1], page)
+        ws = None
+        if n_splits > 1:
+            ws = ctx.buf("decode_partial", 1, decode_workspace_floats(nd, n_heads, D, n_splits), torch.float32)
+        with _timed("attention_decode", *cost(0, nd)):
+            attention_decode_rel(q, cache_slot, bt, ctx.seq_lens, nd, n_heads, scale, window, dist_bias, temp_coef,
+                                 temp_every, out, n_splits, ws, chunk=chunk or 0, sink=sink, gate_col=gate_col)
+
     if tuned:
         if nd:
-            n_splits = decode_splits(nd, n_heads, bt.shape[1], page)
-            ws = None
-            if n_splits > 1:
-                ws = ctx.buf("decode_partial", 1, decode_workspace_floats(nd, n_heads, D, n_splits), torch.float32)
-            with _timed("attention_decode", *cost(0, nd)):
-                attention_decode_rel(q, cache_slot, bt, ctx.seq_lens, nd, n_heads, scale, window, dist_bias, temp_coef,
-                                     temp_every, out, n_splits, ws)
+            decode_rows()
         if ctx.n_seqs > nd:
             with _timed("attention_prefill", *cost(nd, ctx.n_seqs)):
                 attention_prefill_rel(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, nd, ctx.n_seqs - nd,
@@ -1135,8 +1147,11 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
         return out
     if (_MODE == "tuned" and q.dtype == torch.bfloat16 and dist_bias is None and temp_every == 0
             and attention_window_takes(D, v_head_dim, page) and q.stride(0) % 8 == 0 and q.data_ptr() % 16 == 0):
-        # decode rows (four key phases a row) and portions (row blocks by the longest portion) in a launch each
-        if nd:
+        # decode rows (the decode kernel, or four key phases a row) and portions (row blocks by the longest portion) in a
+        # launch each
+        if nd and decode_tuned:
+            decode_rows()
+        elif nd:
             with _timed("attention_window_decode", *cost(0, nd)):
                 attention_window(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, 0, nd, 1, n_heads, n_kv_heads, D,
                                  v_head_dim, page, scale, window, keep_first, softcap, out, sink=sink, gate_col=gate_col, chunk=chunk or 0)

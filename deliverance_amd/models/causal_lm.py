@@ -15,6 +15,7 @@ import torch
 
 from ..config.specs import ModelConfig
 from ..kernels import ops
+from ..parts.norms import STREAM_ITSELF
 from ..parts import Block, StepContext, build_norm, build_position, to_matrix, to_vector
 from ..registry import Architecture, ModelSupport, read_config_json
 from ..weights.loader import load_declared
@@ -110,11 +111,13 @@ class CausalLM:
             # [stream | embedding output] in the compute dtype; the right half is written once a step
             both = ctx.buf("input_mix", N, 2 * self.config.width, ctx.dtype)
             ops.concat_rows(x, both, self.config.width)
-        for call in self.config.schedule:
+        h = None                                        # a block's input that the block before has made
+        for call, after in zip(self.config.schedule, (*self.config.schedule[1:], None)):
             if getattr(call, "mix_input", False):       # x <- W [x; embedding output]
                 ops.concat_rows(x, both, 0)
                 ops.linear(both, self.input_mix, None, x)
-            self.blocks[call.layer].forward(ctx, x, call)
+            ahead = after is not None and not getattr(after, "mix_input", False) and self.blocks[after.layer].takes_stream_ahead()
+            h = self.blocks[call.layer].forward(ctx, x, call, h_ready=h, next_pre=STREAM_ITSELF if ahead else None)
             if debug:
                 ctx.emit(call.layer, "layer_output", x)
         logits = ctx.buf("logits", n_want, self.config.vocab_size, torch.float32)

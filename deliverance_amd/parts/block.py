@@ -91,28 +91,41 @@ class Block:
                 ops.copy_rows(out, x, accumulate=True, scale=self.residual_multiplier)
         return None
 
-    def forward(self, ctx: StepContext, x: torch.Tensor, call) -> None:
+    def takes_stream_ahead(self) -> bool:
+        """Whether the block's first part reads the stream itself: the norm at the end of the block before can then
+        convert it in passing (``forward(next_pre=STREAM_ITSELF)`` there, ``h_ready`` here)."""
+        return self.pre_mixer_norm is None
+
+    def forward(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None, next_pre=None):
+        """Runs the block.  ``h_ready``: the mixer's input, when the block before has made it.  ``next_pre``: what the
+        block behind wants of the new stream (``STREAM_ITSELF`` or None); returns it when the block's last norm could make
+        it in the same pass, else None."""
+        if ctx.debug_hook is not None or self.post_block_norm is not None:
+            next_pre = None
         fused = getattr(self.mixer, "forward_normed", None)
         h_ff = self._part(ctx, x, self.pre_mixer_norm, self.post_mixer_norm,
                           lambda h, into: self.mixer.forward(ctx, h, into, call),
                           None if fused is None else (lambda norm, into: fused(ctx, norm, x, call) if into is None
                                                       else fused(ctx, norm, x, call, into=into)), part=self.mixer,
-                          scale=self.mixer_scale,
-                          next_pre=None if self.feed_forward is None or ctx.debug_hook is not None else
-                          (self.pre_ff_norm if self.pre_ff_norm is not None else STREAM_ITSELF))
+                          h_ready=h_ready, scale=self.mixer_scale,
+                          next_pre=next_pre if self.feed_forward is None else (None if ctx.debug_hook is not None else
+                          (self.pre_ff_norm if self.pre_ff_norm is not None else STREAM_ITSELF)))
         if ctx.debug_hook is not None:
             ctx.emit(call.layer, "post_attention_residual", x)
         if self.feed_forward is not None:
             fused = getattr(self.feed_forward, "forward_normed", None)
-            self._part(ctx, x, self.pre_ff_norm, self.post_ff_norm,
-                       lambda h, into: self.feed_forward.forward(ctx, h, into),
-                       None if fused is None else (lambda norm, into: fused(ctx, norm, x) if into is None
-                                                   else fused(ctx, norm, x, into=into)), part=self.feed_forward,
-                       h_ready=h_ff, scale=self.ff_scale)
+            h_next = self._part(ctx, x, self.pre_ff_norm, self.post_ff_norm,
+                                lambda h, into: self.feed_forward.forward(ctx, h, into),
+                                None if fused is None else (lambda norm, into: fused(ctx, norm, x) if into is None
+                                                            else fused(ctx, norm, x, into=into)), part=self.feed_forward,
+                                h_ready=h_ff, scale=self.ff_scale, next_pre=next_pre)
             if ctx.debug_hook is not None:
                 chosen = getattr(self.feed_forward, "last_choice", None)
                 if chosen is not None:             # a routed feed-forward: the experts of every row, [N, top]
                     ctx.emit(call.layer, "expert_choice", chosen)
                 ctx.emit(call.layer, "post_ff_residual", x)
+        else:
+            h_next = h_ff
         if self.post_block_norm is not None:                # the stream itself, normalised in place
             ops.copy_rows(self.post_block_norm.forward(ctx, x, out_name="post_norm", out_dtype=torch.float32), x)
+        return h_next

@@ -57,8 +57,8 @@ RUNS = {
     # chunks and on another layer's keys) and its models through the step function
     "luvatar": ["tests/test_luvatar_gpu.py", "-n", "4"] if FULL else
                ["tests/test_luvatar_gpu.py", "-n", "3", "-m", QUICK, "-k",
-                "not (portions and sizes0) and not (edge and float32) and not ((portions or whole_prompts) and A and float32) "
-                "and not (mixed_batches and float32)"],
+                "not float32 and not (portions and (sizes0 or A)) and not token_by_token and not (mixed_batches and (A or C)) "
+                "and not (edge and True and not 56)"],
     "replay": ["tests/test_replay_gpu.py", "-n", "4"] if FULL else
               ["tests/test_replay_gpu.py", "-n", "2", "-k", "(mixed and (A or B) and not 32) or want_subset or errors_leave or first_tokens"],
     # inner sizes of 32 in an engine step: qkv and fc of seed 11 (and, in the full run, proj of seed 5)
