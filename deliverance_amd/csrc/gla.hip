@@ -214,6 +214,7 @@ struct GlaServeArgs {
   bf16_t* y; int y_ld;                // [N, H * Dv]
   int H, D, Dv, write, seq0, n_seqs;
   float q_scale, inv_tau, eps;
+  int whole_qk, whole_v, whole_low;   // four entries of q and k, of v, of the low rank's numbers lie 8-byte aligned
   int n_chunks;                       // chunks of the longest portion
   float* ends;                        // [n_seqs, n_chunks, H, Dv, D]: chunks' end states, then their start states
   float* chunk_decay;                 // [n_seqs, n_chunks, H, D]
@@ -338,62 +339,131 @@ struct GlaLds {
   int thin[GLA_NBLK];
 };
 
+// Four neighbouring entries of a row of proj; `whole`: one 8-byte load (the same for the whole launch).
+__device__ __forceinline__ uint2 gla_load4(const bf16_t* row, int at, int count, bool whole) {
+  if (whole) return *(const uint2*)(row + (at < count ? at : 0));
+  uint32_t e[4];
+#pragma unroll
+  for (int i = 0; i < 4; ++i) e[i] = row[at + i < count ? at + i : 0];
+  return make_uint2(e[0] | (e[1] << 16), e[2] | (e[3] << 16));
+}
+// ... with zeros for what lies behind the row's last entry, or everywhere
+__device__ __forceinline__ uint2 gla_keep4(uint2 x, int at, int count, bool any) {
+  if (!any || at >= count) return make_uint2(0, 0);
+  if (at + 1 >= count) x.x &= 0xffffu;
+  if (at + 2 >= count) x.y = 0;
+  else if (at + 3 >= count) x.y &= 0xffffu;
+  return x;
+}
+__device__ __forceinline__ float4 gla_widen4(uint2 x) {
+  return make_float4(__uint_as_float(x.x << 16), __uint_as_float(x.x & 0xffff0000u), __uint_as_float(x.y << 16),
+                     __uint_as_float(x.y & 0xffff0000u));
+}
+
 template <int DT, int VT, bool OUT>
 __device__ __forceinline__ void gla_prepare(const GlaServeArgs& A, GlaLds<DT, VT, OUT>& L, int h, int n0, int n) {
   constexpr int DP = DT * 16, DS = DP + 4, VP = VT * 16, VS = VP + 4;
-  constexpr int ITEMS = GLA_NBLK * DP;
+  constexpr int ITEMS = GLA_NBLK * DP, PER = ITEMS > 256 ? ITEMS / 256 : 1;
+  constexpr int UP4 = GLA_LOW_MAX / 4, LOWN = GLA_CHUNK * UP4 / 256;
   static_assert(GLA_CHUNK * DS >= GLA_CHUNK * GLA_LOW_MAX, "the low rank's numbers lie where the logarithms go");
   const int t = threadIdx.x;
-  if (t < GLA_NBLK) L.thin[t] = 0;
+  // Every load first, from places that exist: keys, queries, values and the low rank's numbers in pieces of four
+  // entries, then this thread's rows of the low rank's second matrix and their bias.
+  uint2 rk[DT], rq[OUT ? DT : 1], rv[VT], rl[LOWN], up[PER][UP4];
+  float bias[PER], zr[PER][GLA_BLK];
+#pragma unroll
+  for (int u = 0; u < DT; ++u) {
+    const int idx = t + 256 * u, tok = idx / (DP / 4), d = idx % (DP / 4) * 4;
+    const bf16_t* row = A.proj + (size_t)(n0 + (tok < n ? tok : 0)) * A.ld + h * A.D;
+    rk[u] = gla_load4(row + A.k_off, d, A.D, A.whole_qk);
+    if (OUT) rq[u] = gla_load4(row + A.q_off, d, A.D, A.whole_qk);
+  }
+#pragma unroll
+  for (int u = 0; u < VT; ++u) {
+    const int idx = t + 256 * u, tok = idx / (VP / 4), d = idx % (VP / 4) * 4;
+    rv[u] = gla_load4(A.proj + (size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.v_off + h * A.Dv, d, A.Dv, A.whole_v);
+  }
   if (A.up) {
-    for (int i = t; i < GLA_CHUNK * A.rank; i += 256) {
-      const int tok = i / A.rank, r = i % A.rank;
-      L.la[tok * GLA_LOW_MAX + r] = bf16_to_f32(A.proj[(size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.low_off + r]);
+#pragma unroll
+    for (int u = 0; u < LOWN; ++u) {
+      const int idx = t + 256 * u, tok = idx / UP4, r = idx % UP4 * 4;
+      rl[u] = gla_load4(A.proj + (size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.low_off, r, A.rank, A.whole_low);
     }
   }
-  for (int i = t; i < GLA_CHUNK * VP; i += 256) {
-    const int tok = i / VP, d = i % VP;
-    const bool ok = tok < n && d < A.Dv;
-    const bf16_t x = A.proj[(size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.v_off + h * A.Dv + (d < A.Dv ? d : 0)];
-    L.v[tok * VS + d] = ok ? x : (bf16_t)0;
-  }
-  lds_barrier();
-  constexpr int PER = ITEMS > 256 ? ITEMS / 256 : 1;
-  float z[PER][GLA_BLK];
-  bf16_t q[PER][GLA_BLK], k[PER][GLA_BLK];
 #pragma unroll
   for (int u = 0; u < PER; ++u) {
     const int it = t + 256 * u, b = it / DP, d = it % DP, dc = h * A.D + (d < A.D ? d : 0);
+    bias[u] = A.bias[dc];
+    if (A.up) {
+#pragma unroll
+      for (int r = 0; r < UP4; ++r)
+        if (4 * r < A.rank) up[u][r] = *(const uint2*)(A.up + (size_t)dc * A.rank + 4 * r);
+    } else {
+#pragma unroll
+      for (int i = 0; i < GLA_BLK; ++i) {
+        const int tok = b * GLA_BLK + i;
+        zr[u][i] = A.raw[(size_t)(n0 + (tok < n ? tok : 0)) * A.raw_ld + dc];
+      }
+    }
+  }
+  if (t < GLA_NBLK) L.thin[t] = 0;
+  // keys and queries as they are go where the scaled keys will be, the low rank's numbers where the logarithms will be
+  bf16_t* raw_k = (bf16_t*)L.kh;
+  bf16_t* raw_q = raw_k + GLA_CHUNK * DS;
+#pragma unroll
+  for (int u = 0; u < DT; ++u) {
+    const int idx = t + 256 * u, tok = idx / (DP / 4), d = idx % (DP / 4) * 4;
+    *(uint2*)(raw_k + tok * DS + d) = gla_keep4(rk[u], d, A.D, tok < n);
+    if (OUT) *(uint2*)(raw_q + tok * DS + d) = gla_keep4(rq[u], d, A.D, tok < n);
+  }
+#pragma unroll
+  for (int u = 0; u < VT; ++u) {
+    const int idx = t + 256 * u, tok = idx / (VP / 4), d = idx % (VP / 4) * 4;
+    *(uint2*)(L.v + tok * VS + d) = gla_keep4(rv[u], d, A.Dv, tok < n);
+  }
+  if (A.up) {
+#pragma unroll
+    for (int u = 0; u < LOWN; ++u) {
+      const int idx = t + 256 * u, tok = idx / UP4, r = idx % UP4 * 4;
+      if (r < A.rank) *(float4*)(L.la + tok * GLA_LOW_MAX + r) = gla_widen4(rl[u]);
+    }
+  }
+  lds_barrier();
+  bf16_t k[PER][GLA_BLK], q[PER][OUT ? GLA_BLK : 1];
+  float z[PER][GLA_BLK];
+#pragma unroll
+  for (int u = 0; u < PER; ++u) {
+    const int it = t + 256 * u, b = it / DP, d = it % DP;
     if (it < ITEMS) {
 #pragma unroll
       for (int i = 0; i < GLA_BLK; ++i) {
-        const int tok = b * GLA_BLK + i, nn = n0 + (tok < n ? tok : 0);
-        k[u][i] = A.proj[(size_t)nn * A.ld + A.k_off + dc];
-        if (OUT) q[u][i] = A.proj[(size_t)nn * A.ld + A.q_off + dc];
-        z[u][i] = A.up ? 0.f : A.raw[(size_t)nn * A.raw_ld + dc];
+        k[u][i] = raw_k[(b * GLA_BLK + i) * DS + d];
+        if (OUT) q[u][i] = raw_q[(b * GLA_BLK + i) * DS + d];
+        z[u][i] = A.up ? 0.f : zr[u][i];
       }
       if (A.up) {
-        for (int r = 0; r < A.rank; r += 4) {
-          const uint2 w = *(const uint2*)(A.up + (size_t)dc * A.rank + r);
-          const float w0 = bf16_to_f32((bf16_t)(w.x & 0xffffu)), w1 = bf16_to_f32((bf16_t)(w.x >> 16));
-          const float w2 = bf16_to_f32((bf16_t)(w.y & 0xffffu)), w3 = bf16_to_f32((bf16_t)(w.y >> 16));
 #pragma unroll
-          for (int i = 0; i < GLA_BLK; ++i) {
-            const float4 a = *(const float4*)(L.la + (b * GLA_BLK + i) * GLA_LOW_MAX + r);
-            z[u][i] = fmaf(w0, a.x, fmaf(w1, a.y, fmaf(w2, a.z, fmaf(w3, a.w, z[u][i]))));
+        for (int r = 0; r < UP4; ++r) {
+          if (4 * r < A.rank) {
+            const float4 w = gla_widen4(up[u][r]);
+#pragma unroll
+            for (int i = 0; i < GLA_BLK; ++i) {
+              const float4 a = *(const float4*)(L.la + (b * GLA_BLK + i) * GLA_LOW_MAX + 4 * r);
+              z[u][i] = fmaf(w.x, a.x, fmaf(w.y, a.y, fmaf(w.z, a.z, fmaf(w.w, a.w, z[u][i]))));
+            }
           }
         }
       }
-      const float bias = A.bias[dc];
       float run = 0.f;
 #pragma unroll
       for (int i = 0; i < GLA_BLK; ++i) {
-        if (b * GLA_BLK + i < n && d < A.D) run += gla_log2_decay<true>(z[u][i] + bias, A.inv_tau);
+        const float dec = gla_log2_decay<true>(z[u][i] + bias[u], A.inv_tau);
+        run += b * GLA_BLK + i < n && d < A.D ? dec : 0.f;
         z[u][i] = run;                              // the running logarithm since the block's start
       }
     }
   }
-  if (OUT) lds_barrier();                           // the low rank's numbers have been read
+  lds_barrier();                                    // everything parked has been read
 #pragma unroll
   for (int u = 0; u < PER; ++u) {
     const int it = t + 256 * u, b = it / DP, d = it % DP;
@@ -402,12 +472,11 @@ __device__ __forceinline__ void gla_prepare(const GlaServeArgs& A, GlaLds<DT, VT
       L.G[b * DP + d] = __builtin_amdgcn_exp2f(end);
       if (OUT && end < GLA_THIN) L.thin[b] = 1;
 #pragma unroll
-      for (int i = 0; i < GLA_BLK; ++i) {
+      for (int i = 0; i < GLA_BLK; ++i) {           // (keys and queries of what does not exist are zeros)
         const int tok = b * GLA_BLK + i;
-        const bool ok = tok < n && d < A.D;
-        L.kh[tok * DS + d] = ok ? bf16_to_f32(k[u][i]) * __builtin_amdgcn_exp2f(end - z[u][i]) : 0.f;
+        L.kh[tok * DS + d] = bf16_to_f32(k[u][i]) * __builtin_amdgcn_exp2f(end - z[u][i]);
         if (OUT) {
-          L.qh[tok * DS + d] = ok ? bf16_to_f32(q[u][i]) * (A.q_scale * __builtin_amdgcn_exp2f(z[u][i])) : 0.f;
+          L.qh[tok * DS + d] = bf16_to_f32(q[u][i]) * (A.q_scale * __builtin_amdgcn_exp2f(z[u][i]));
           L.la[tok * DS + d] = z[u][i];
         }
       }
@@ -523,6 +592,19 @@ gla_output_kernel(GlaServeArgs A) {
 #pragma unroll
       for (int dt = 0; dt < DT; ++dt) s0[vt][dt] = start_piece(vt, dt);
   }
+  // the gates and gains of this lane's part of rows 4 hi + r
+  bf16_t gate[VT][4];
+  float gain[VT];
+#pragma unroll
+  for (int vt = 0; vt < VT; ++vt) {
+    const int vc = vt * 16 + lo < A.Dv ? vt * 16 + lo : 0;
+    gain[vt] = load_param(A.gain, A.gain_dtype, vc);
+#pragma unroll
+    for (int r = 0; r < 4; ++r) {
+      const int tok = w * GLA_BLK + 4 * hi + r;
+      gate[vt][r] = A.proj[(size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.g_off + h * A.Dv + vc];
+    }
+  }
   gla_prepare<DT, VT, true>(A, L, h, n0, n);
   if (w * GLA_BLK >= n) return;
   // this wavefront's rows: block w of the chunk; row lo of it as a matrix operand
@@ -614,13 +696,12 @@ gla_output_kernel(GlaServeArgs A) {
     for (int vt = 0; vt < VT; ++vt) ss = fmaf(o[vt][r], o[vt][r], ss);
     const float inv = 1.0f / sqrtf(group_sum<16>(ss) / (float)A.Dv + A.eps);
     const int tok = w * GLA_BLK + 4 * hi + r;
-    const bf16_t* grow = A.proj + (size_t)(n0 + (tok < n ? tok : 0)) * A.ld + A.g_off + h * A.Dv;
 #pragma unroll
     for (int vt = 0; vt < VT; ++vt) {
-      const int v = vt * 16 + lo, vc = v < A.Dv ? v : 0;
-      const float gate = bf16_to_f32(grow[vc]), gain = load_param(A.gain, A.gain_dtype, vc);
-      const float g = gate * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-GLA_LOG2E * gate));
-      if (tok < n && v < A.Dv) A.y[(size_t)(n0 + tok) * A.y_ld + h * A.Dv + v] = f32_to_bf16(o[vt][r] * inv * gain * g);
+      const int v = vt * 16 + lo;
+      const float gt = bf16_to_f32(gate[vt][r]);
+      const float g = gt * __builtin_amdgcn_rcpf(1.0f + __builtin_amdgcn_exp2f(-GLA_LOG2E * gt));
+      if (tok < n && v < A.Dv) A.y[(size_t)(n0 + tok) * A.y_ld + h * A.Dv + v] = f32_to_bf16(o[vt][r] * inv * gain[vt] * g);
     }
   }
 }
@@ -650,6 +731,10 @@ static int gla_serve_args(GlaServeArgs& A, const char* what, const void* proj, i
   A.up = (const bf16_t*)up; A.rank = rank; A.raw = raw; A.raw_ld = raw_ld; A.bias = bias; A.gain = gain; A.gain_dtype = gain_dtype;
   A.state = state; A.state_ld = state_ld; A.state_slots = state_slots; A.q_start = q_start; A.y = (bf16_t*)y; A.y_ld = y_ld;
   A.H = H; A.D = D; A.Dv = Dv; A.write = write; A.seq0 = seq0; A.n_seqs = n_seqs; A.q_scale = q_scale; A.inv_tau = 1.0f / tau;
+  const bool rows = ld % 4 == 0 && (uintptr_t)proj % 8 == 0;
+  A.whole_qk = rows && q_off % 4 == 0 && k_off % 4 == 0;
+  A.whole_v = rows && v_off % 4 == 0 && Dv % 4 == 0;
+  A.whole_low = rows && low_off % 4 == 0;
   A.eps = eps; A.n_chunks = 0; A.ends = nullptr; A.chunk_decay = nullptr;
   return 0;
 }
