@@ -21,7 +21,7 @@ from typing import Callable, Dict, Hashable, List, Optional, Sequence, Union
 import torch
 
 from ..config.engine_config import EngineConfig
-from ..kernels import ops
+from ..kernels import build, ops
 from ..models.causal_lm import CausalLM, load_model
 from ..profiler import InferenceProfiler
 from ..sampling.params import GeneratorParameters
@@ -63,6 +63,7 @@ class CausalLanguageModel:
     def __init__(self, model: CausalLM, engine_config: EngineConfig):
         if not torch.cuda.is_available():
             raise RuntimeError("deliverance_amd runs on a GPU only; no device is visible")
+        build.ensure([*model.kernel_units(), "sample"])
         self.model = model
         self.config = model.config
         self.engine_config = engine_config

@@ -153,16 +153,25 @@ _ARGTYPES = {
 _LIB = None
 
 
+class _EntryPoints:
+    """Entry points by name; each is looked up, and given its argument types, when it is first used."""
+
+    def __init__(self, library):
+        self._library = library
+
+    def __getattr__(self, name):
+        fn = getattr(self._library, name)
+        fn.argtypes = _ARGTYPES[name]
+        fn.restype = ctypes.c_int
+        setattr(self, name, fn)
+        return fn
+
+
 def _lib():
-    """The kernel library with its argument types declared (conversion is then cheap and checked)."""
+    """The kernels' entry points with their argument types declared (conversion is then cheap and checked)."""
     global _LIB
     if _LIB is None:
-        lib = build.load()
-        for name, types in _ARGTYPES.items():
-            fn = getattr(lib, name)
-            fn.argtypes = types
-            fn.restype = ctypes.c_int
-        _LIB = lib
+        _LIB = _EntryPoints(build.load())
     return _LIB
 
 
@@ -1554,6 +1563,7 @@ def gla_walk(ctx, qkv: torch.Tensor, q_off: int, k_off: int, v_off: int, raw: to
 
 
 GLA_CHUNK = 64               # tokens of a chunk of the form for portions
+GLA_SERVE_MAX_DIM = 128      # key and value entries a head of the forms for serving
 
 
 def gla_serve_takes(proj: torch.Tensor, state: torch.Tensor, head_dim: int, v_head_dim: int) -> bool:

@@ -61,6 +61,22 @@ class CausalLM:
         """Whether every part allows a decode step to be replayed from a recorded HIP graph."""
         return all(b.mixer.graph_safe and (b.feed_forward is None or b.feed_forward.graph_safe) for b in self.blocks)
 
+    def kernel_units(self) -> List[str]:
+        """The kernel units that the model's steps call: what a first call in a fresh checkout compiles, side by side."""
+        names = ["rowwise", "dispatch"] + (["gemm_mfma", "gemm_wide", "gemm_fused"] if self.dtype == torch.bfloat16 else ["gemm_ref"])
+        norms = [self.final_norm, self.embed_norm]
+        for b in self.blocks:
+            norms += [b.pre_mixer_norm, b.post_mixer_norm, b.pre_ff_norm, b.post_ff_norm, b.post_block_norm]
+            names += list(b.mixer.kernel_units(self.dtype))
+            if b.feed_forward is not None:
+                names += list(b.feed_forward.kernel_units(self.dtype))
+            if b.mixer_scale is not None or b.ff_scale is not None:
+                names.append("elementwise")
+        names += [u for n in norms if n is not None for u in n.kernel_units]
+        if self.input_mix is not None or self.config.logit_softcap > 0.0:
+            names.append("elementwise")
+        return sorted(set(names))
+
     # ---- what the cache must provide -----------------------------------------------------
     def cache_needs(self) -> Dict[int, object]:
         """cache slot -> KVNeed / StateNeed of the layer call that writes it."""

@@ -147,6 +147,22 @@ class CausalSelfAttention(Mixer):
                       None if self.v_head_dim == self.head_dim else self.v_head_dim, keep_first=self.keep_first,
                       chunk=self.chunk)
 
+    def kernel_units(self, dtype):
+        out = ("attn_prepare",) if self._prepared() else (() if self.position is None else ("attn_latent",))
+        if self.v_head_dim != self.head_dim and not self._prepared():
+            out += ("attn_rel",)
+        D = self.head_dim
+        if dtype != torch.bfloat16:
+            return out + (("attn_rel",) if self.extras else ("attn_ref",))
+        if not self.extras:
+            return out + (("attn_decode", "attn_prefill") if D % 16 == 0 else ("attn_ref",))
+        scores_only = self.v_head_dim == D and D % 16 == 0 and D <= 128 and self.softcap == 0.0 and not self.keep_first
+        if scores_only and self.sink is None and self.out_gate is None and self.chunk is None:
+            return out + ("attn_decode_rel", "attn_prefill_rel")
+        if D % 8 or max(D, self.v_head_dim) > 128 or self.dist_bias is not None or self.temp_every:
+            return out + ("attn_rel",)
+        return out + ("attn_window",) + (("attn_decode_rel",) if scores_only else ())
+
     def _epilogue_write(self) -> bool:
         """Whether the q|k|v product may write keys and values to the cache itself (its epilogue assumes
         keys and values of one size)."""

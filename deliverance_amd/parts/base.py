@@ -156,6 +156,10 @@ class Arena:
 
 
 class Norm:
+    # The kernel units (kernels/build.py) that the norm's steps call; a model's are compiled together before its first
+    # step.  (A unit that is not named is compiled when it is first called.)
+    kernel_units: Tuple[str, ...] = ()
+
     def forward(self, ctx: StepContext, x: torch.Tensor, rows: Optional[torch.Tensor] = None,
                 n_rows: Optional[int] = None, out_name: str = "norm",
                 out_dtype: Optional[torch.dtype] = None) -> torch.Tensor:
@@ -173,6 +177,10 @@ class Mixer:
     # once as a HIP graph and replayed.  A mixer that reads ctx.*_host must leave this False.
     graph_safe = False
 
+    def kernel_units(self, dtype: torch.dtype) -> Tuple[str, ...]:
+        """The kernel units that the mixer's steps call beyond the matrix products (see ``Norm.kernel_units``)."""
+        return ()
+
     def cache_need(self):
         return None
 
@@ -182,6 +190,9 @@ class Mixer:
 
 class FeedForward:
     graph_safe = False
+
+    def kernel_units(self, dtype: torch.dtype) -> Tuple[str, ...]:
+        return ()
 
     def forward(self, ctx: StepContext, h: torch.Tensor, x: torch.Tensor) -> None:
         raise NotImplementedError

@@ -92,6 +92,9 @@ class GatedDeltaRule(Mixer):
         self.s_elems = H * Dv * D
         self.conv_off = self.s_elems                 # where the filters' inputs start in a state row
 
+    def kernel_units(self, dtype):
+        return ("delta", "ssm")
+
     def cache_need(self):
         return StateNeed(self.s_elems + (self.taps - 1) * self.conv_cols)
 

@@ -68,6 +68,9 @@ class GatedFeedForward(FeedForward):
         if tuple(self.down_weight.shape) != (self.width, self.inner):
             raise ValueError(f"down weight is {list(self.down_weight.shape)}, expected {[self.width, self.inner]}")
 
+    def kernel_units(self, dtype):
+        return ("elementwise",)
+
     def forward(self, ctx: StepContext, h: torch.Tensor, x: torch.Tensor) -> None:
         N = h.shape[0]
         mid = ctx.buf("ff_mid", N, self.inner, ctx.dtype)
@@ -149,6 +152,9 @@ class ExpertsFeedForward(FeedForward):
                 DenseFeedForwardSpec("dense", self.width, spec.shared_inner, spec.shared_activation or self.activation,
                                      bias=False),
                 {"fc_weight": params["shared_up_weight"], "proj_weight": params["shared_down_weight"]}, dtype, device)
+
+    def kernel_units(self, dtype):
+        return ("moe", "elementwise") + (() if self.shared is None else self.shared.kernel_units(dtype))
 
     def forward(self, ctx: StepContext, h: torch.Tensor, x: torch.Tensor) -> None:
         ids = weights = None

@@ -58,6 +58,10 @@ class GatedLinearAttention(Mixer):
         self.v_off, self.gate_off = 2 * self.qk_cols, 2 * self.qk_cols + self.v_cols
         self.low_off = self.gate_off + self.v_cols
 
+    def kernel_units(self, dtype):
+        serve = dtype == torch.bfloat16 and self.D % 4 == 0 and max(self.D, self.Dv) <= ops.GLA_SERVE_MAX_DIM
+        return ("gla",) if serve else ("gla", "delta")
+
     def cache_need(self):
         return StateNeed(self.H * self.Dv * self.D)
 

@@ -62,6 +62,9 @@ class LatentAttention(Mixer):
         if self.rotary.dims > self.dr:
             raise ValueError(f"{self.rotary.dims} turned entries, the rotated piece has {self.dr}")
 
+    def kernel_units(self, dtype):
+        return ("attn_latent",) + (("attn_latent_mfma", "gemm_heads") if dtype == torch.bfloat16 else ())
+
     def cache_need(self):
         return KVNeed(1, self.row_dim, self.window, self.kv_rank, values_in_keys=True)
 

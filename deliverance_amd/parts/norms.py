@@ -41,6 +41,7 @@ class RmsNorm(Norm):
     """The row divided by its root mean square (eps inside the root), times ``gain_offset + weight``; all in
     32-bit.  Behind a part it can do three things in one pass over the row (``add_into``): normalise the
     part's output, add it to the residual stream, and normalise the new stream for the part that follows."""
+    kernel_units = ("norm_rms",)
 
     def __init__(self, spec, params, dtype, device):
         self.width = spec.width

@@ -32,6 +32,9 @@ class ParallelMixer(Mixer):
     def graph_safe(self) -> bool:
         return all(b.graph_safe for b in self.branches)
 
+    def kernel_units(self, dtype):
+        return tuple(u for b in self.branches for u in b.kernel_units(dtype))
+
     def cache_need(self):
         return tuple(b.cache_need() for b in self.branches)
 

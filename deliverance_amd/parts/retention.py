@@ -56,6 +56,9 @@ class Retention(Mixer):
             raise ValueError(f"{self.rotary.dims} turned entries, a head has {D}")
         self.v_off, self.gate_off = 2 * self.qk_cols, 2 * self.qk_cols + self.v_cols
 
+    def kernel_units(self, dtype):
+        return ("retention", "delta") + (("attn_latent",) if self.rotary is not None and self.rotary.dims else ())
+
     def cache_need(self):
         return StateNeed(self.H * self.Dv * self.D)
 

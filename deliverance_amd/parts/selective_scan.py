@@ -42,6 +42,9 @@ class SelectiveScan(Mixer):
         self.out_weight = to_matrix(shaped("out_weight", (E, I)), dtype, device)
         self.conv_off = I * n                      # where the filter's inputs start in a state row
 
+    def kernel_units(self, dtype):
+        return ("ssm",)
+
     def cache_need(self):
         return StateNeed(self.inner * self.state + (self.taps - 1) * self.inner)
 

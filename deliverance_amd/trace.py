@@ -36,11 +36,13 @@ class TraceSession:
         from . import models  # noqa: F401  (registers the architectures)
         from .config.engine_config import KERNEL_MODES
         from .engine.device_cache import DeviceCache
+        from .kernels import build
         from .models.causal_lm import load_model
         if kernels not in KERNEL_MODES:
             raise ValueError(f"kernels must be one of {KERNEL_MODES}")
         tdtype = {"bfloat16": torch.bfloat16, "float32": torch.float32}[dtype]
         self.model = load_model(model_dir, tdtype, device)
+        build.ensure(self.model.kernel_units())
         # A request's count is rounded up to a multiple of 64, so max_tokens / page_size pages
         # hold every live request whatever its length.
         self.cache = DeviceCache(self.model.cache_needs(), tdtype, device, page_size, max(max_tokens, 64),
@@ -111,10 +113,6 @@ def main(argv=None) -> int:
 
     say("importing torch")
     import torch
-    from .kernels import build
-    if build.library_path() is None:
-        say("compiling the HIP kernels (first call)")
-    build.load()
     if not torch.cuda.is_available():
         say("no GPU is visible; trace_run drives the GPU engine and has no other path")
         return 3
