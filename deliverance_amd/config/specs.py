@@ -112,6 +112,9 @@ class AttentionSpec:
     # no keys and values of its own: the run order gives this layer another layer's cache slot to read (``write`` off);
     # there is no key or value matrix, no key gain, and heads, sizes and rotation are the other layer's
     shared_kv: bool = False
+    # one number a query head that a score loses for every position of distance between query and key (after the scale,
+    # which does not multiply it): s - distance_slopes[h] * (i - j)
+    distance_slopes: Optional[Tuple[float, ...]] = None
 
     @property
     def value_dim(self) -> int:
@@ -230,6 +233,23 @@ class SelectiveScanSpec:
 
 
 @dataclass(frozen=True)
+class RealGatedRecurrenceSpec:
+    """A linear recurrence with one real number of state a channel and a decay that the input sets.  Two branches of
+    ``channels`` entries: y = act(W_y h + b_y) and u, a projection W_x h + b_x that passes a causal filter of
+    ``conv_taps`` taps a channel (with a bias, no activation).  u is cut into ``blocks`` equal parts; in part b two square
+    matrices with biases give r = logistic(A_b u_b + ..) and i = logistic(I_b u_b + ..).  Per channel
+    ln a = -``decay_strength`` * r * softplus(lam),  S <- a S + sqrt(1 - a^2) * i * u, from S = 0.  The output is the
+    projection of S * y back to the width.  The state (S and the filter's last inputs) is 32-bit."""
+    kind: str            # "real_gated_recurrence"
+    width: int
+    channels: int
+    blocks: int
+    conv_taps: int
+    decay_strength: float
+    activation: str = "gelu_pytorch_tanh"
+
+
+@dataclass(frozen=True)
 class DeltaRuleSpec:
     """A gated delta-rule mixer.  Per value head a matrix S (``head_dim`` x ``v_head_dim``, 32-bit) is carried from
     token to token: S <- g * S (a decay in (0, 1) for every row of S), u = beta * (v - S^T k), S <- S + k u^T,
@@ -295,8 +315,14 @@ class ExpertsFeedForwardSpec:
     else down(act(up h)).  ``weight_on``: "output" (weight * expert(h)) or "input" (expert(weight * h)).
     ``router == "softmax_top"``: logits z = matrix h + bias (32-bit); the ``top`` largest logits are used (the lower
     index wins a tie), with the softmax over just those as weights.
+    ``router == "softmax_all"``: s = the softmax over all logits; the ``top`` largest entries of s + correction (a vector,
+    32-bit) are used, with s without the correction over the chosen ones' sum (+ 1e-20) as weights.  ``groups`` > 0: the
+    entries form so many equal groups of neighbours, a group counts as its largest s + correction, and only entries of
+    the ``groups_kept`` best groups can be chosen.  ``identity``: so many more router outputs behind the experts' name
+    experts that hand the input on as it is.
     ``shared_inner`` > 0: one more feed-forward of that many columns runs for every token with weight 1 and is
-    added; it is ungated, or (``shared_gated``) of the gated form with ``shared_limit``.  ``limit``: the constant of
+    added; it is ungated, or (``shared_gated``) of the gated form with ``shared_limit``; ``shared_token_gate``: times
+    the logistic function of one more row of the input.  ``limit``: the constant of
     the activation "glu_capped" (``GatedFeedForwardSpec``)."""
     kind: str            # "experts"
     width: int
@@ -315,6 +341,10 @@ class ExpertsFeedForwardSpec:
     shared_gated: bool = False
     shared_limit: float = 0.0
     router_bias: bool = False
+    groups: int = 0
+    groups_kept: int = 0
+    identity: int = 0
+    shared_token_gate: bool = False
 
 
 @dataclass(frozen=True)
@@ -341,6 +371,9 @@ class LayerSpec:
     # element, after the norm behind it and before it joins the stream (parameters "mixer_scale", "ff_scale")
     mixer_scale: bool = False
     ff_scale: bool = False
+    # both parts read the one norm in front (``pre_mixer_norm``) and join the stream together:
+    # h = norm(x), x += mixer(h) + ff(h)
+    parallel: bool = False
 
 
 @dataclass(frozen=True)
@@ -350,12 +383,16 @@ class LayerCall:
     ``layer`` indexes ``ModelConfig.layers`` (a layer may be named twice), ``cache`` is
     the cache slot its mixer uses, and ``write`` is False when the mixer only reads a
     slot that another call has filled in the same step.  ``mix_input``: right before this
-    call the stream becomes W [stream; embedding output] (``ModelConfig.input_mix``).
+    call the stream becomes W [stream; embedding output] (``ModelConfig.input_mix``).  ``add_input``: right before this
+    call the embedding output is added to the stream; ``add_step``: and then row ``add_step`` of the model's step
+    vectors (``ModelConfig.step_vectors``).
     """
     layer: int
     cache: int
     write: bool = True
     mix_input: bool = False
+    add_input: bool = False
+    add_step: Optional[int] = None
 
 
 @dataclass(frozen=True)
@@ -383,6 +420,9 @@ class ModelConfig:
     # a matrix [width, 2 width] (parameter "input_mix") that run-order entries with ``mix_input`` apply to the
     # stream beside the embedding output (the stream's half first)
     input_mix: bool = False
+    # so many vectors of the model's width (parameter "step_vectors" [n, width]) that run-order entries with
+    # ``add_step`` add to the stream
+    step_vectors: int = 0
 
     @property
     def n_cache_slots(self) -> int:

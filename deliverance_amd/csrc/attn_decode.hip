@@ -20,7 +20,7 @@
 // Compiled a second time with DEC_REL (attn_decode_rel.hip) the kernel also takes what some designs put on the
 // scores: a bias by the distance between query and key (a table [Hq][n_dist], 32-bit, the last entry for every
 // larger distance) and a query temperature 1 + t_coef * ln(floor((p + 1) / t_every) + 1) that multiplies the
-// scale; chunks of positions in place of a window (a row sees the keys of its own chunk only); a sink, one number a head
+// scale; a slope per head that a score loses for every position of distance; chunks of positions in place of a window (a row sees the keys of its own chunk only); a sink, one number a head
 // whose exponential joins the softmax's denominator, without a key or a value and not scaled; and a gate, rows like out,
 // of which o is multiplied with the logistic function.  The last two act once, after everything has been merged.  The
 // plain build has none of that code.
@@ -31,9 +31,9 @@
 #ifdef DEC_REL
 #define DEC_KERNEL attn_decode_rel_kernel
 #define DEC_MERGE_KERNEL attn_decode_rel_merge_kernel
-#define DEC_REL_PARAMS , const float* __restrict__ rel_bias, int n_dist, float t_coef, int t_every, int chunk DEC_END_PARAMS
-#define DEC_REL_DECL , const float* rel_bias, int n_dist, float t_coef, int t_every, int chunk, const float* sink, const bf16_t* gate, int gate_ld
-#define DEC_REL_ARGS , rel_bias, n_dist, t_coef, t_every, chunk DEC_END_ARGS
+#define DEC_REL_PARAMS , const float* __restrict__ rel_bias, int n_dist, const float* __restrict__ slopes, float t_coef, int t_every, int chunk DEC_END_PARAMS
+#define DEC_REL_DECL , const float* rel_bias, int n_dist, const float* slopes, float t_coef, int t_every, int chunk, const float* sink, const bf16_t* gate, int gate_ld
+#define DEC_REL_ARGS , rel_bias, n_dist, slopes, t_coef, t_every, chunk DEC_END_ARGS
 #define DEC_END_PARAMS , const float* __restrict__ sink, const bf16_t* __restrict__ gate, int gate_ld
 #define DEC_END_ARGS , sink, gate, gate_ld
 #else
@@ -140,6 +140,7 @@ DEC_KERNEL(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ ca
   const int lo = SPLIT ? (lo_row > split0 ? lo_row : split0) : lo_row;
 #ifdef DEC_REL
   const float* brow = rel_bias ? rel_bias + (size_t)h * n_dist : nullptr;
+  const float slope = slopes ? slopes[h] : 0.f;
   const float qscale = t_every > 0 ? scale * (1.0f + t_coef * logf((float)((p_row + 1) / t_every + 1))) : scale;
 #else
   const float qscale = scale;
@@ -227,9 +228,10 @@ DEC_KERNEL(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ ca
     // the bias of the key whose score this lane will keep, asked for beside the keys and values (a key past the
     // row's own position has no distance: it reads entry 0 and is dropped with its score)
     float brel = 0.f;
+    if (slopes) brel = -slope * (float)(p_row - (c0 + piece * G + sub));
     if (brow) {
       const int dist = p_row - (c0 + piece * G + sub);
-      brel = brow[dist < 0 ? 0 : (dist < n_dist ? dist : n_dist - 1)];
+      brel += brow[dist < 0 ? 0 : (dist < n_dist ? dist : n_dist - 1)];
     }
 #endif
     // nothing moves across this line: the compiler would otherwise push the value loads down behind
@@ -466,8 +468,8 @@ static int rel_checks(const float* rel_bias, int n_dist, int t_every) {
 // and `workspace` holds the partial results.
 extern "C" int da_attn_decode_rel(const void* q, int q_ld, const void* cache, const int* block_table,
                                   int max_blocks, const int* seq_lens, int S, int Hq, int Hkv, int D, int page,
-                                  float scale, int window, const float* rel_bias, int n_dist, float t_coef,
-                                  int t_every, int chunk, const float* sink, const void* gate, int gate_ld, void* out,
+                                  float scale, int window, const float* rel_bias, int n_dist, const float* slopes,
+                                  float t_coef, int t_every, int chunk, const float* sink, const void* gate, int gate_ld, void* out,
                                   int out_ld, int n_splits, void* workspace, long workspace_bytes, void* stream) {
   if (decode_checks(q, q_ld, cache, max_blocks, S, Hq, Hkv, D, page, window, out_ld)) return 1;
   if (rel_checks(rel_bias, n_dist, t_every)) return 1;
@@ -484,7 +486,7 @@ extern "C" int da_attn_decode_rel(const void* q, int q_ld, const void* cache, co
   }
   if (S == 0) return 0;
   decode_launch(q, q_ld, cache, block_table, max_blocks, seq_lens, S, Hq, Hkv, D, page, scale, window, out, out_ld,
-                n_splits > 1 ? n_splits : 1, span, (float*)workspace, (hipStream_t)stream, rel_bias, n_dist, t_coef, t_every,
+                n_splits > 1 ? n_splits : 1, span, (float*)workspace, (hipStream_t)stream, rel_bias, n_dist, slopes, t_coef, t_every,
                 chunk, sink, (const bf16_t*)gate, gate_ld);
   DA_CHECK_LAUNCH("attn_decode_rel");
   return 0;

@@ -6,6 +6,7 @@
 //   s_j = cap((q . k_j) * scale * temp(p)) + bias[h][min(p - j, n_dist - 1)]
 //   temp(p) = 1 + t_coef * ln(floor((p + 1) / t_every) + 1)          (1 when t_every is 0)
 //   cap(s) = softcap * tanh(s / softcap)                              (s itself when softcap is 0)
+// `slopes` (optional, [Hq], 32-bit): s_j also loses slopes[h] * (p - j).
 // With `chunk` c (in place of a window) the keys are j in [floor(p / c) c, p].
 // With a window w the keys are j in [p - w + 1, p] and, with keep_first, also j < keep_first: the first keys of a
 // sequence stay visible at their true positions.
@@ -30,8 +31,8 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
                     const int* __restrict__ block_table, int max_blocks,
                     const int* __restrict__ seq_of_token, const int* __restrict__ positions,
                     int Hq, int Hkv, int D, int Dv, int page, float scale, int window, int chunk,
-                    const float* __restrict__ bias, int n_dist, float t_coef, int t_every, float softcap, int keep_first,
-                    const float* __restrict__ sink, const T* __restrict__ gate, int gate_ld,
+                    const float* __restrict__ bias, int n_dist, const float* __restrict__ slopes, float t_coef, int t_every,
+                    float softcap, int keep_first, const float* __restrict__ sink, const T* __restrict__ gate, int gate_ld,
                     T* __restrict__ out, int out_ld) {
   __shared__ float qs[REL_MAX_D];
   __shared__ float ps[DA_WAVE];
@@ -44,6 +45,7 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
   const long long page_elems = (long long)Hkv * page * (D + Dv);
   const long long v0 = (long long)Hkv * page * D + (long long)hk * page * Dv;
   const float* brow = bias ? bias + (size_t)h * n_dist : nullptr;
+  const float slope = slopes ? slopes[h] : 0.f;
   const float temp = t_every > 0 ? 1.0f + t_coef * logf((float)((p + 1) / t_every + 1)) : 1.0f;
   const float qscale = scale * temp;
 
@@ -77,6 +79,7 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
         const int dist = p - key;
         s += brow[dist < n_dist ? dist : n_dist - 1];
       }
+      if (slopes) s -= slope * (float)(p - key);
     }
     const float m_new = fmaxf(m, wave_max(s));
     const float e = valid ? expf(s - m_new) : 0.f;
@@ -123,7 +126,7 @@ attn_rel_ref_kernel(const T* __restrict__ q, int q_ld, const T* __restrict__ cac
 extern "C" int da_attn_rel_ref(const void* q, int q_ld, const void* cache, int dtype, const int* block_table,
                                int max_blocks, const int* seq_of_token, const int* positions, int N, int Hq, int Hkv,
                                int D, int Dv, int page, float scale, int window, int chunk, const float* bias, int n_dist,
-                               float t_coef, int t_every, float softcap, int keep_first, const float* sink,
+                               const float* slopes, float t_coef, int t_every, float softcap, int keep_first, const float* sink,
                                const void* gate, int gate_ld, void* out, int out_ld, void* stream) {
   DA_REQUIRE(N >= 0 && Hq > 0 && Hkv > 0 && D > 0 && Dv > 0 && page > 0, "attn_rel_ref: bad sizes");
   DA_REQUIRE(Hq % Hkv == 0, "attn_rel_ref: %d query heads are not a multiple of %d key heads", Hq, Hkv);
@@ -139,12 +142,12 @@ extern "C" int da_attn_rel_ref(const void* q, int q_ld, const void* cache, int d
   if (dtype == DA_BF16)
     hipLaunchKernelGGL(attn_rel_ref_kernel<bf16_t>, dim3(N * Hq), dim3(DA_WAVE), 0, (hipStream_t)stream,
                        (const bf16_t*)q, q_ld, (const bf16_t*)cache, block_table, max_blocks, seq_of_token, positions,
-                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
+                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, slopes, t_coef, t_every, softcap, keep_first, sink,
                        (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld);
   else
     hipLaunchKernelGGL(attn_rel_ref_kernel<float>, dim3(N * Hq), dim3(DA_WAVE), 0, (hipStream_t)stream,
                        (const float*)q, q_ld, (const float*)cache, block_table, max_blocks, seq_of_token, positions,
-                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, t_coef, t_every, softcap, keep_first, sink,
+                       Hq, Hkv, D, Dv, page, scale, window, chunk, bias, n_dist, slopes, t_coef, t_every, softcap, keep_first, sink,
                        (const float*)gate, gate_ld, (float*)out, out_ld);
   DA_CHECK_LAUNCH("attn_rel_ref");
   return 0;

@@ -6,6 +6,7 @@
 // `chunk` in place of a window, when j <= p and floor(j / chunk) = floor(p / chunk);
 //   s_j = cap((q . k_j) * scale),  cap(s) = softcap * tanh(s / softcap)   (s itself when softcap is 0)
 //   o   = sum_j softmax(s)_j v_j                                           (scores, weights and sums in 32-bit)
+// `slopes` (optional, [Hq], 32-bit): s_j loses slopes[h] * (p - j), after the cap.
 // `sink` (optional, [Hq], 32-bit): the softmax's denominator also holds exp(sink[h]), a term without a key or a
 // value that is not scaled; it joins once, after the phases have been merged.  `gate` (optional, rows like out):
 // o <- o * logistic(gate), in the store.
@@ -51,8 +52,8 @@ __global__ void __launch_bounds__(AW_WAVES * DA_WAVE)
 attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restrict__ cache,
                    const int* __restrict__ block_table, int max_blocks, const int* __restrict__ q_start,
                    const int* __restrict__ seq_lens, int seq0, int Hq, int Hkv, int D, int Dv, int page, float scale,
-                   int window, int chunk, int keep_first, float softcap, const float* __restrict__ sink,
-                   const bf16_t* __restrict__ gate, int gate_ld, bf16_t* __restrict__ out, int out_ld, int RB) {
+                   int window, int chunk, int keep_first, float softcap, const float* __restrict__ slopes,
+                   const float* __restrict__ sink, const bf16_t* __restrict__ gate, int gate_ld, bf16_t* __restrict__ out, int out_ld, int RB) {
   constexpr int PER = DT * 16 + 2;
   __shared__ float mg[3 * PER * DA_WAVE];              // (KP - 1) * RB <= 3 partial results
   const int KP = AW_WAVES / RB;
@@ -71,6 +72,7 @@ attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restr
   const long long page_elems = (long long)Hkv * page * (D + Dv);
   const bf16_t* kbase = cache + (long long)hk * page * D;
   const bf16_t* vbase = cache + (long long)Hkv * page * D + (long long)hk * Dv * page;
+  const float slope2 = slopes ? slopes[h] * AW_LOG2E : 0.f;       // in the base-2 domain
   const int kfw = window > 0 ? keep_first : 0;
   // the first position that a row at position p sees (apart from kept first keys)
   auto low_of = [&](int p) -> int {
@@ -176,6 +178,7 @@ attn_window_kernel(const bf16_t* __restrict__ q, int q_ld, const bf16_t* __restr
       } else {
         v = sc[r] * (scale * AW_LOG2E);
       }
+      v -= slope2 * (float)(pq - key);
       const bool seen = key <= pq && (key >= p_low || key < kfw);
       v = seen ? v : -INFINITY;
       sc[r] = v;
@@ -300,7 +303,7 @@ extern "C" int da_attn_window_takes(int D, int Dv, int page) {
 extern "C" int da_attn_window(const void* q, int q_ld, const void* cache, const int* block_table, int max_blocks,
                               const int* q_start, const int* seq_lens, int seq0, int n_seqs, int max_query_len, int Hq,
                               int Hkv, int D, int Dv, int page, float scale, int window, int chunk, int keep_first, float softcap,
-                              const float* sink, const void* gate, int gate_ld, void* out, int out_ld, int form,
+                              const float* slopes, const float* sink, const void* gate, int gate_ld, void* out, int out_ld, int form,
                               void* stream) {
   DA_REQUIRE(n_seqs >= 0 && Hq > 0 && Hkv > 0 && max_query_len >= 0, "attn_window: bad sizes");
   DA_REQUIRE(form == 0 || form == 1 || form == 2 || form == 4, "attn_window: form %d (0 leaves the choice to the rule; 1, 2 or 4 row blocks)", form);
@@ -326,7 +329,7 @@ extern "C" int da_attn_window(const void* q, int q_ld, const void* cache, const 
 #define AW_GO(N, M)                                                                                                  \
   hipLaunchKernelGGL((attn_window_kernel<N, M>), grid, block, 0, (hipStream_t)stream, (const bf16_t*)q, q_ld,        \
                      (const bf16_t*)cache, block_table, max_blocks, q_start, seq_lens, seq0, Hq, Hkv, D, Dv, page,   \
-                     scale, window, chunk, keep_first, softcap, sink, (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld, RB)
+                     scale, window, chunk, keep_first, softcap, slopes, sink, (const bf16_t*)gate, gate_ld, (bf16_t*)out, out_ld, RB)
 #define AW_VALUES(N)                 \
   do {                               \
     if (Dv <= 32) AW_GO(N, 1);       \

@@ -4,6 +4,7 @@
 //   da_concat_rows dst[r, off + c] = src[r, c]                      a 32-bit matrix into columns of a wider one
 //   da_softcap     v <- cap * tanh(v / cap)                         in place, 32-bit
 //   da_scale_add_rows  dst[r, c] += mult * scale[c] * src[r, c]     a learned scale per channel, 32-bit
+//   da_add_rows    dst[r, c] += src[r, c] + vec[c]                  either may be absent, 32-bit
 #include "common.h"
 
 template <typename T, bool FAST>
@@ -79,5 +80,23 @@ extern "C" int da_concat_rows(const float* src, void* dst, int dtype, int ld, in
     hipLaunchKernelGGL(concat_rows_kernel<float>, dim3(da_ceil_div(n, 256)), dim3(256), 0, (hipStream_t)stream, src,
                        (float*)dst, ld, off, n, E);
   DA_CHECK_LAUNCH("concat_rows");
+  return 0;
+}
+
+__global__ void add_rows_kernel(float* __restrict__ dst, const float* __restrict__ src, const float* __restrict__ vec, long n, int E) {
+  const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
+  if (i >= n) return;
+  float v = dst[i];
+  if (src) v += src[i];
+  if (vec) v += vec[i % E];
+  dst[i] = v;
+}
+
+extern "C" int da_add_rows(float* dst, const float* src, const float* vec, int R, int E, void* stream) {
+  DA_REQUIRE(R >= 0 && E > 0 && (src || vec) && src != dst, "add_rows: bad sizes, or nothing to add");
+  if (R == 0) return 0;
+  const long n = (long)R * E;
+  hipLaunchKernelGGL(add_rows_kernel, dim3(da_ceil_div(n, 256)), dim3(256), 0, (hipStream_t)stream, dst, src, vec, n, E);
+  DA_CHECK_LAUNCH("add_rows");
   return 0;
 }

@@ -7,7 +7,10 @@
 //                   given a pair are also written out a slot
 //   da_moe_gated    mid[slot] = act(Wg_e a[row]) * (Wu_e a[row])      (plain kernel, any dtype)
 //   da_moe_down     out[slot] = Wd_e mid[slot]                        (plain kernel, 32-bit out)
-//   da_moe_combine  y[n] (+)= sum_k weight_k * out[slot(n, k)]        k ascending
+//   da_moe_combine  y[n] (+)= sum_k weight_k * out[slot(n, k)]        k ascending; a pair without a slot adds weight_k
+//                   times the token's input where there are experts that hand it on, and a shared feed-forward's result
+//                   joins times a logistic gate
+//   da_moe_top, da_moe_choose   from router logits to expert ids and weights
 //
 // Everything the grid depends on comes from the step's shape (tokens x top, experts); which tiles are
 // used is decided on the device, so a step can be recorded.  A pair's result does not depend on its slot:
@@ -284,6 +287,96 @@ extern "C" int da_moe_top_logistic(const float* z, int ldz, int N, int E, int to
   return da_moe_top(z, ldz, nullptr, 0, N, E, top, 0, renorm, ids, weights, stream);
 }
 
+// The choice by a softmax over all E outputs: s = softmax(z), c = s + correction; the `top` largest c are chosen (the lower
+// index wins a tie), with s over the chosen ones' sum (+ 1e-20) as weights.  groups > 0: the outputs are so many equal runs
+// of neighbours, a run counts as its largest c, and only entries of the `keep` best runs can be chosen (the lower run wins
+// a tie).  A wavefront a token, an output every 64th a lane; c and the runs' largest wait in LDS.
+// (EC: outputs that LDS has room for.)
+#define MC_WAVES 4
+template <int EC>
+__global__ void __launch_bounds__(MC_WAVES * DA_WAVE)
+moe_choose_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ correction, int N, int E, int top, int groups,
+                  int keep, int* __restrict__ ids, float* __restrict__ weights) {
+  __shared__ float mc_lds[MC_WAVES][3][EC];
+  const int lane = threadIdx.x % DA_WAVE, wave = threadIdx.x / DA_WAVE;
+  const int n = blockIdx.x * MC_WAVES + wave;
+  if (n >= N) return;                                  // (wavefronts do not wait for one another)
+  float *c = mc_lds[wave][0], *sc = mc_lds[wave][1], *gm = mc_lds[wave][2];      // choice scores, softmax scores, the runs' largest
+  const float* row = z + (size_t)n * ldz;
+  auto wave_fence = [] {                               // LDS of this wavefront only
+    __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
+    __builtin_amdgcn_wave_barrier();
+    __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
+  };
+  float m = -INFINITY;
+  for (int e = lane; e < E; e += DA_WAVE) m = fmaxf(m, row[e]);
+  m = wave_max(m);
+  float sum = 0.f;
+  for (int e = lane; e < E; e += DA_WAVE) {
+    const float v = expf(row[e] - m);
+    sc[e] = v;
+    sum += v;
+  }
+  sum = wave_sum(sum);
+  for (int e = lane; e < E; e += DA_WAVE) {
+    const float v = sc[e] / sum;
+    sc[e] = v;
+    c[e] = v + correction[e];
+  }
+  wave_fence();
+  if (groups > 0) {
+    const int size = E / groups;
+    for (int q = lane; q < groups; q += DA_WAVE) {
+      float v = -INFINITY;
+      for (int e = 0; e < size; ++e) v = fmaxf(v, c[q * size + e]);
+      gm[q] = v;
+    }
+    wave_fence();
+    for (int q = lane; q < groups; q += DA_WAVE) {
+      int ahead = 0;                                   // runs that come before this one
+      for (int k = 0; k < groups; ++k) ahead += gm[k] > gm[q] || (gm[k] == gm[q] && k < q);
+      if (ahead >= keep)
+        for (int e = 0; e < size; ++e) c[q * size + e] = -INFINITY;
+    }
+    wave_fence();
+  }
+  float chosen = 0.f;
+  auto better = [](float a, int ai, float b, int bi) { return a > b || (a == b && ai < bi); };
+  for (int k = 0; k < top; ++k) {
+    float bv = -INFINITY;
+    int be = lane < E ? lane : E - 1;
+    for (int e = lane; e < E; e += DA_WAVE)
+      if (better(c[e], e, bv, be)) { bv = c[e]; be = e; }
+    wave_best(bv, be, better);
+    chosen += sc[be];
+    if (lane == 0) {
+      ids[(size_t)n * top + k] = be;
+      c[be] = -INFINITY;                               // taken
+    }
+    wave_fence();
+    if (lane == 0) weights[(size_t)n * top + k] = sc[be];
+  }
+  if (lane == 0)
+    for (int k = 0; k < top; ++k) weights[(size_t)n * top + k] /= chosen + 1e-20f;
+}
+
+extern "C" int da_moe_choose(const float* z, int ldz, const float* correction, int N, int E, int top, int groups, int keep,
+                             int* ids, float* weights, void* stream) {
+  DA_REQUIRE(N >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E && correction, "moe_choose: bad sizes");
+  DA_REQUIRE(groups == 0 || (groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= E / groups * keep),
+             "moe_choose: top %d of %d outputs in %d groups of which %d are kept", top, E, groups, keep);
+  if (N == 0) return 0;
+#define MC_GO(EC)                                                                                                            \
+  hipLaunchKernelGGL((moe_choose_kernel<EC>), dim3(da_ceil_div(N, MC_WAVES)), dim3(MC_WAVES * DA_WAVE), 0, (hipStream_t)stream, \
+                     z, ldz, correction, N, E, top, groups, keep, ids, weights)
+  if (E <= 64) MC_GO(64);
+  else if (E <= 256) MC_GO(256);
+  else MC_GO(MOE_MAX_EXPERTS);
+#undef MC_GO
+  DA_CHECK_LAUNCH("moe_choose");
+  return 0;
+}
+
 // slot_weight[slot_of_pair[i]] = weights[i]: a pair's weight where its slot's row is
 __global__ void moe_slot_weights_kernel(const int* __restrict__ slot_of_pair, const float* __restrict__ weights, int P,
                                         float* __restrict__ slot_weight) {
@@ -302,10 +395,13 @@ extern "C" int da_moe_slot_weights(const int* slot_of_pair, const float* weights
   return 0;
 }
 
-// y[n] (+)= sum_k weight(n, k) * out[slot_of_pair[n * top + k]]; weights: per pair, or one for all
+// y[n] (+)= sum_k weight(n, k) * out[slot_of_pair[n * top + k]]; weights: per pair, or one for all.  h (optional): a pair
+// without a slot adds weight * h[n], an expert that hands its input on.  shared (optional): + logistic(gate[n]) * shared[n].
+template <typename T>
 __global__ void moe_combine_kernel(const float* __restrict__ out, int ldo, const int* __restrict__ slot_of_pair,
                                    const float* __restrict__ weights, float uniform, int top, float* __restrict__ y,
-                                   int ldy, int N, int width, int accumulate) {
+                                   int ldy, int N, int width, int accumulate, const T* __restrict__ h, int ldh,
+                                   const float* __restrict__ shared, int lds, const float* __restrict__ gate, int ldg) {
   const long i = (long)blockIdx.x * blockDim.x + threadIdx.x;
   if (i >= (long)N * width) return;
   const int n = (int)(i / width), c = (int)(i % width);
@@ -313,17 +409,26 @@ __global__ void moe_combine_kernel(const float* __restrict__ out, int ldo, const
   for (int k = 0; k < top; ++k) {
     const int slot = slot_of_pair[n * top + k];
     if (slot >= 0) s += (weights ? weights[n * top + k] : uniform) * out[(size_t)slot * ldo + c];
+    else if (h) s += (weights ? weights[n * top + k] : uniform) * to_f32(h[(size_t)n * ldh + c]);
   }
+  if (shared) s += shared[(size_t)n * lds + c] / (1.f + expf(-gate[(size_t)n * ldg]));
   float* dst = y + (size_t)n * ldy + c;
   *dst = accumulate ? *dst + s : s;
 }
 
 extern "C" int da_moe_combine(const float* out, int ldo, const int* slot_of_pair, const float* weights, float uniform,
-                              int top, float* y, int ldy, int N, int width, int accumulate, void* stream) {
+                              int top, float* y, int ldy, int N, int width, int accumulate, const void* h, int h_dtype, int ldh,
+                              const float* shared, int lds, const float* gate, int ldg, void* stream) {
   DA_REQUIRE(N >= 0 && width > 0 && top > 0 && ldo >= width && ldy >= width, "moe_combine: bad sizes");
+  DA_REQUIRE((!h || ldh >= width) && (!shared || (lds >= width && gate && ldg > 0)), "moe_combine: the input's or the shared result's rows");
   if (N == 0) return 0;
-  hipLaunchKernelGGL(moe_combine_kernel, dim3(da_ceil_div((long)N * width, 256)), dim3(256), 0, (hipStream_t)stream, out,
-                     ldo, slot_of_pair, weights, uniform, top, y, ldy, N, width, accumulate);
+  const dim3 grid(da_ceil_div((long)N * width, 256));
+  if (h && h_dtype == DA_BF16)
+    hipLaunchKernelGGL(moe_combine_kernel<bf16_t>, grid, dim3(256), 0, (hipStream_t)stream, out, ldo, slot_of_pair, weights,
+                       uniform, top, y, ldy, N, width, accumulate, (const bf16_t*)h, ldh, shared, lds, gate, ldg);
+  else
+    hipLaunchKernelGGL(moe_combine_kernel<float>, grid, dim3(256), 0, (hipStream_t)stream, out, ldo, slot_of_pair, weights,
+                       uniform, top, y, ldy, N, width, accumulate, (const float*)h, ldh, shared, lds, gate, ldg);
   DA_CHECK_LAUNCH("moe_combine");
   return 0;
 }

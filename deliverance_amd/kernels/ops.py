@@ -95,13 +95,13 @@ _ARGTYPES = {
     "da_can_fuse_ln": [_I, _I, _I],
     "da_run_step": [_VP, _VP],
     "da_top_logprobs": [_VP, _I, _I, _I, _VP, _I, _VP, _VP, _VP],
-    "da_attn_decode_rel": [_VP, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _I, _VP, _VP, _I, _VP, _I, _I, _VP, ctypes.c_long, _VP],
+    "da_attn_decode_rel": [_VP, _I, _VP, _VP, _I, _VP, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _VP, _F, _I, _I, _VP, _VP, _I, _VP, _I, _I, _VP, ctypes.c_long, _VP],
     "da_attn_prefill_rel": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _F, _I, _VP, _I, _F, _I, _VP, _I, _I, _VP],
     "da_rmsnorm": [_VP, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
     "da_rmsnorm_add": [_VP, _VP, _I, _VP, _VP, _I, _F, _F, _VP, _I, _I, _I, _VP],
-    "da_attn_rel_ref": [_VP, _I, _VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _I, _I, _VP, _I, _F, _I, _F, _I, _VP, _VP, _I,
+    "da_attn_rel_ref": [_VP, _I, _VP, _I, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _F, _I, _I, _VP, _I, _VP, _F, _I, _F, _I, _VP, _VP, _I,
                         _VP, _I, _VP],
-    "da_attn_window": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _VP, _VP, _I, _VP, _I, _I,
+    "da_attn_window": [_VP, _I, _VP, _VP, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _F, _I, _I, _I, _F, _VP, _VP, _VP, _I, _VP, _I, _I,
                        _VP],
     "da_attn_window_takes": [_I, _I, _I],
     "da_attn_prepare": [_VP, _I, _I, _I, _I, _I, _VP, _I, _VP, _I, _F, _I, _VP, _VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _I, _I, _F,
@@ -148,7 +148,15 @@ _ARGTYPES = {
     "da_conv_state_update": [_VP, _I, _I, _VP, ctypes.c_long, _I, _VP, _VP, _I, _I, _I, _VP],
     "da_selective_scan": [_VP, _I, _I, _VP, _I, _VP, _I, _I, _I, _VP, _I, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP,
                           _VP, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
-    "da_moe_combine": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _I, _VP],
+    "da_moe_combine": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _I, _VP, _I, _I, _VP, _I, _VP, _I, _VP],
+    "da_moe_choose": [_VP, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP, _VP],
+    "da_add_rows": [_VP, _VP, _VP, _I, _I, _VP],
+    "da_rglru_walk": [_VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _VP],
+    "da_rglru_serve_takes": [_I],
+    "da_rglru_chunk_tokens": [],
+    "da_rglru_decode": [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _VP],
+    "da_rglru_portion": [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
+                         _VP, ctypes.c_long, _VP],
 }
 _LIB = None
 
@@ -400,6 +408,19 @@ def concat_rows(src: torch.Tensor, dst: torch.Tensor, col: int) -> torch.Tensor:
     return dst
 
 
+def add_rows(dst: torch.Tensor, src: Optional[torch.Tensor], vec: Optional[torch.Tensor]) -> torch.Tensor:
+    """dst[r, c] += src[r, c] + vec[c], all 32-bit; either may be None."""
+    _dev(dst, src, vec)
+    R, E = dst.shape
+    _need(dst.dtype == torch.float32 and dst.is_contiguous() and dst.dim() == 2, "add_rows: dst must be contiguous float32 [R, E]")
+    _need(src is None or (src.dtype == torch.float32 and src.is_contiguous() and src.dim() == 2 and src.shape[1] == E and src.shape[0] >= R),
+          "add_rows: src must be contiguous float32 [R, E]")
+    _need(vec is None or (vec.dtype == torch.float32 and vec.is_contiguous() and vec.numel() == E), "add_rows: vec must be float32 [E]")
+    with _timed("add_rows", _nbytes(dst) * (2 if src is None else 3), dst.numel() * 2, "fp32"):
+        _check(_lib().da_add_rows(_ptr(dst), _ptr(src), _ptr(vec), R, E, _stream()))
+    return dst
+
+
 def softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
     """logits <- cap * tanh(logits / cap), in place."""
     _dev(logits)
@@ -492,17 +513,30 @@ def moe_down_ref(mid: torch.Tensor, row_of_slot: torch.Tensor, tile_expert: torc
 
 
 def moe_combine(out: torch.Tensor, slot_of_pair: torch.Tensor, weights: Optional[torch.Tensor], uniform: float,
-                top: int, y: torch.Tensor, accumulate: bool) -> torch.Tensor:
-    """y[n] (+)= sum_k weight * out[slot_of_pair[n, k]] with ``weights[n, k]`` or the one weight ``uniform``."""
-    _dev(out, slot_of_pair, weights, y)
+                top: int, y: torch.Tensor, accumulate: bool, h: Optional[torch.Tensor] = None,
+                shared: Optional[torch.Tensor] = None, shared_logit: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """y[n] (+)= sum_k weight * out[slot_of_pair[n, k]] with ``weights[n, k]`` or the one weight ``uniform``.  With ``h``
+    [N, width] a pair without a slot adds weight * h[n]; with ``shared`` [N, width] and ``shared_logit`` [N, 1] (both
+    32-bit) logistic(shared_logit[n]) * shared[n] joins."""
+    _dev(out, slot_of_pair, weights, y, h, shared, shared_logit)
     _rows_2d(out, "out"); _rows_2d(y, "y")
     N, width = y.shape
     _need(out.dtype == torch.float32 and y.dtype == torch.float32 and out.shape[1] == width, "moe_combine: float32 [.., width]")
     _need(slot_of_pair.dtype == torch.int32 and slot_of_pair.numel() >= N * top, "moe_combine: a slot a pair")
     _need(weights is None or (weights.dtype == torch.float32 and weights.numel() >= N * top), "moe_combine: a weight a pair")
-    with _timed("moe_combine", (top + 2) * N * width * 4, top * N * width, "fp32"):
+    if h is not None:
+        _rows_2d(h, "h")
+        _need(h.shape[0] >= N and h.shape[1] == width, "moe_combine: the input must be [N, width]")
+    _need((shared is None) == (shared_logit is None), "moe_combine: a shared result needs its gate")
+    if shared is not None:
+        _rows_2d(shared, "shared")
+        _need(shared.dtype == shared_logit.dtype == torch.float32 and shared.shape[0] >= N and shared.shape[1] == width
+              and shared_logit.dim() == 2 and shared_logit.shape[0] >= N, "moe_combine: float32 [N, width] with a gate [N, 1]")
+    with _timed("moe_combine", (top + 2) * N * width * 4 + _nbytes(shared), top * N * width, "fp32"):
         _check(_lib().da_moe_combine(_ptr(out), out.stride(0), _ptr(slot_of_pair), _ptr(weights), float(uniform), top,
-                                     _ptr(y), y.stride(0), N, width, int(accumulate), _stream()))
+                                     _ptr(y), y.stride(0), N, width, int(accumulate), _ptr(h), 0 if h is None else _dt(h),
+                                     0 if h is None else h.stride(0), _ptr(shared), 0 if shared is None else shared.stride(0),
+                                     _ptr(shared_logit), 0 if shared is None else shared_logit.stride(0), _stream()))
     return y
 
 
@@ -601,15 +635,17 @@ def attention_rel_ref(q: torch.Tensor, cache_slot: torch.Tensor, block_table: to
                       positions: torch.Tensor, n_heads: int, n_kv_heads: int, head_dim: int, v_head_dim: int, page: int,
                       scale: float, window: Optional[int], dist_bias: Optional[torch.Tensor], temp_coef: float,
                       temp_every: int, out: torch.Tensor, softcap: float = 0.0, keep_first: int = 0,
-                      sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: int = 0) -> torch.Tensor:
+                      sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: int = 0,
+                      slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Plain paged attention with a bias by distance (``dist_bias`` [Hq, n_dist] float32, the last column for every
     larger distance), a query temperature by position, values of their own size, a cap on the scores
     (``softcap * tanh(score / softcap)``) and, with a window, ``keep_first`` first keys that stay visible.  ``sink``
     (float32 [Hq]): exp(sink[h]) joins the softmax's denominator; ``chunk`` (in place of a window): a row sees the keys of
-    its own chunk of so many positions; ``gate_col`` >= 0: out * logistic(gate), the gate's
+    its own chunk of so many positions; ``slopes`` (float32 [Hq]): a score loses slopes[h] * distance; ``gate_col`` >= 0: out * logistic(gate), the gate's
     Hq * Dv entries lying in q's rows from that column on (q is then wider than its Hq * D query entries)."""
-    _dev(q, cache_slot, block_table, seq_of_token, positions, dist_bias, out, sink)
+    _dev(q, cache_slot, block_table, seq_of_token, positions, dist_bias, out, sink, slopes)
     gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, n_heads * head_dim, n_heads * v_head_dim, q, "attention")
+    _slopes_arg(slopes, n_heads, "attention")
     _rows_2d(q, "q"); _rows_2d(out, "out")
     N = q.shape[0]
     _need(cache_slot.is_contiguous() and cache_page_elems(cache_slot) == n_kv_heads * page * (head_dim + v_head_dim),
@@ -628,7 +664,7 @@ def attention_rel_ref(q: torch.Tensor, cache_slot: torch.Tensor, block_table: to
         n_dist = dist_bias.shape[1]
     _check(_lib().da_attn_rel_ref(_ptr(q), q.stride(0), _ptr(cache_slot), _dt(q), _ptr(block_table), block_table.shape[1],
                                   _ptr(seq_of_token), _ptr(positions), N, n_heads, n_kv_heads, head_dim, v_head_dim, page,
-                                  float(scale), int(window or 0), int(chunk or 0), _ptr(dist_bias), n_dist, float(temp_coef),
+                                  float(scale), int(window or 0), int(chunk or 0), _ptr(dist_bias), n_dist, _ptr(slopes), float(temp_coef),
                                   int(temp_every), float(softcap), int(keep_first if window else 0), _ptr(sink),
                                   gate_ptr, gate_ld, _ptr(out), out.stride(0), _stream()))
     return out
@@ -643,6 +679,11 @@ def _sink_gate_args(sink, gate_col, n_heads, q_cols, cols, q, name):
         return None, 0
     _need(gate_col >= q_cols and gate_col + cols <= q.shape[1], f"{name}: the gate's columns leave q's rows or meet the queries")
     return _ptr(q) + gate_col * q.element_size(), q.stride(0)
+
+
+def _slopes_arg(slopes, n_heads, name):
+    _need(slopes is None or (slopes.dtype == torch.float32 and slopes.is_contiguous() and slopes.numel() == n_heads),
+          f"{name}: the slopes by distance must be float32 with one entry a query head")
 
 
 # ------------------------------------------------------------------------------- sampling
@@ -1014,14 +1055,16 @@ def attention_decode_rel(q: torch.Tensor, cache_slot: torch.Tensor, block_table:
                          n_seqs: int, n_heads: int, scale: float, window: Optional[int],
                          dist_bias: Optional[torch.Tensor], temp_coef: float, temp_every: int, out: torch.Tensor,
                          n_splits: int = 1, workspace: Optional[torch.Tensor] = None, chunk: int = 0,
-                         sink: Optional[torch.Tensor] = None, gate_col: int = -1) -> torch.Tensor:
-    """``attention_decode`` with a bias by distance and a query temperature on the scores, chunks of positions in place
+                         sink: Optional[torch.Tensor] = None, gate_col: int = -1,
+                         slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
+    """``attention_decode`` with a bias or a slope (``slopes``, float32 [Hq]) by distance and a query temperature on the scores, chunks of positions in place
     of a window, a sink (float32 [Hq]) and a gate that lies in q's rows from column ``gate_col`` on (q is then wider than
     its Hq * D query entries)."""
     cols = out.shape[1]
     Hkv, page, D = _attn_common(q[:, :cols], cache_slot, block_table, n_heads, out, "attention_decode_rel")
     gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, cols, cols, q, "attention_decode_rel")
-    _dev(sink)
+    _slopes_arg(slopes, n_heads, "attention_decode_rel")
+    _dev(sink, slopes)
     _need(q.shape[0] >= n_seqs and out.shape[0] >= n_seqs and block_table.shape[0] >= n_seqs,
           "attention_decode_rel: fewer rows than sequences")
     _need(seq_lens.dtype == torch.int32 and seq_lens.numel() >= n_seqs, "attention_decode_rel: seq_lens must be int32 [S]")
@@ -1035,7 +1078,7 @@ def attention_decode_rel(q: torch.Tensor, cache_slot: torch.Tensor, block_table:
         ws_bytes = workspace.numel() * 4
     _check(_lib().da_attn_decode_rel(_ptr(q), q.stride(0), _ptr(cache_slot), _ptr(block_table), block_table.shape[1],
                                      _ptr(seq_lens), n_seqs, n_heads, Hkv, D, page, float(scale), int(window or 0),
-                                     bias_ptr, n_dist, float(temp_coef), int(temp_every), int(chunk), _ptr(sink), gate_ptr,
+                                     bias_ptr, n_dist, _ptr(slopes), float(temp_coef), int(temp_every), int(chunk), _ptr(sink), gate_ptr,
                                      gate_ld, _ptr(out), out.stride(0), int(n_splits), _ptr(workspace) if n_splits > 1 else None, ws_bytes, _stream()))
     return out
 
@@ -1064,13 +1107,15 @@ def attention_window(q: torch.Tensor, cache_slot: torch.Tensor, block_table: tor
                      seq_lens: torch.Tensor, seq0: int, n_seqs: int, max_query_len: int, n_heads: int, n_kv_heads: int,
                      head_dim: int, v_head_dim: int, page: int, scale: float, window: Optional[int], keep_first: int,
                      softcap: float, out: torch.Tensor, form: int = 0, sink: Optional[torch.Tensor] = None,
-                     gate_col: int = -1, chunk: int = 0) -> torch.Tensor:
+                     gate_col: int = -1, chunk: int = 0, slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of the sequences ``seq0 .. seq0 + n_seqs - 1`` of a step on the matrix cores, in bfloat16, with keys and
     values of their own sizes, a cap on the scores and, with a window, ``keep_first`` first keys that stay visible.
-    ``chunk`` (in place of a window): a row sees the keys of its own chunk of so many positions only.  ``form``: 0 leaves the workgroup's row blocks to the kernel's rule; 1, 2 or 4 fixes them."""
-    _dev(q, cache_slot, block_table, q_start, seq_lens, out, sink)
+    ``chunk`` (in place of a window): a row sees the keys of its own chunk of so many positions only.
+    ``slopes`` (float32 [Hq]): a score loses slopes[h] * distance.  ``form``: 0 leaves the workgroup's row blocks to the kernel's rule; 1, 2 or 4 fixes them."""
+    _dev(q, cache_slot, block_table, q_start, seq_lens, out, sink, slopes)
     _rows_2d(q, "q"); _rows_2d(out, "out")
     gate_ptr, gate_ld = _sink_gate_args(sink, gate_col, n_heads, n_heads * head_dim, n_heads * v_head_dim, q, "attention_window")
+    _slopes_arg(slopes, n_heads, "attention_window")
     _need(q.dtype == cache_slot.dtype == out.dtype == torch.bfloat16, "attention_window: q, cache and out must be bfloat16")
     _need(cache_slot.is_contiguous() and cache_page_elems(cache_slot) == n_kv_heads * page * (head_dim + v_head_dim),
           "attention_window: a page of the cache slot does not hold Hkv * page * (D + Dv) entries")
@@ -1083,7 +1128,7 @@ def attention_window(q: torch.Tensor, cache_slot: torch.Tensor, block_table: tor
     _check(_lib().da_attn_window(_ptr(q), q.stride(0), _ptr(cache_slot), _ptr(block_table), block_table.shape[1],
                                  _ptr(q_start), _ptr(seq_lens), seq0, n_seqs, max_query_len, n_heads, n_kv_heads, head_dim,
                                  v_head_dim, page, float(scale), int(window or 0), int(chunk or 0), int(keep_first if window else 0),
-                                 float(softcap), _ptr(sink), gate_ptr, gate_ld, _ptr(out),
+                                 float(softcap), _ptr(slopes), _ptr(sink), gate_ptr, gate_ld, _ptr(out),
                                  out.stride(0), int(form), _stream()))
     return out
 
@@ -1096,11 +1141,12 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
                         head_dim: int, v_head_dim: int, scale: float, window: Optional[int],
                         dist_bias: Optional[torch.Tensor], temp_coef: float, temp_every: int,
                         out: torch.Tensor, softcap: float = 0.0, keep_first: int = 0,
-                        sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: Optional[int] = None) -> torch.Tensor:
+                        sink: Optional[torch.Tensor] = None, gate_col: int = -1, chunk: Optional[int] = None,
+                        slopes: Optional[torch.Tensor] = None) -> torch.Tensor:
     """Attention of every row of the step with a bias by distance, a query temperature, values of their own
     size, a cap on the scores, first keys that a window keeps, a term without a key in the softmax's denominator
     (``sink``), a logistic gate on the result (``gate_col``: where the gate lies in q's rows) and chunks in place of a window
-    (``chunk``), each optional; the last three go with the decode kernel, the matrix-core kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
+    (``chunk``) and slopes by distance (``slopes``), each optional; the last four go with the decode kernel, the matrix-core kernel for windows or the plain one.  In bfloat16, with keys and values of one size that is a multiple of 16 up to 128 and a
     bias row that fits the prefill kernel's LDS copy, the one-token sequences go to the decode kernel and the
     portions to the prefill kernel (their forms with these extras); a cap, kept first keys and values of another size
     go to the matrix-core kernel for those (head sizes up to 128, no bias table, no temperature); 32-bit, the reference
@@ -1135,7 +1181,7 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
                     and softcap == 0.0 and not (window and keep_first)
                     and D <= PREFILL_REL_MAX_HEAD_DIM and cache_slot.dim() == 5 and q.stride(0) % 8 == 0
                     and q.data_ptr() % 16 == 0 and (dist_bias is None or dist_bias.shape[1] <= PREFILL_REL_MAX_DIST))
-    tuned = decode_tuned and sink is None and gate_col < 0 and not chunk
+    tuned = decode_tuned and sink is None and gate_col < 0 and not chunk and slopes is None
 
     def decode_rows():
         n_splits = decode_splits(nd, n_heads, bt.shape[1], page)
@@ -1144,7 +1190,7 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
             ws = ctx.buf("decode_partial", 1, decode_workspace_floats(nd, n_heads, D, n_splits), torch.float32)
         with _timed("attention_decode", *cost(0, nd)):
             attention_decode_rel(q, cache_slot, bt, ctx.seq_lens, nd, n_heads, scale, window, dist_bias, temp_coef,
-                                 temp_every, out, n_splits, ws, chunk=chunk or 0, sink=sink, gate_col=gate_col)
+                                 temp_every, out, n_splits, ws, chunk=chunk or 0, sink=sink, gate_col=gate_col, slopes=slopes)
 
     if tuned:
         if nd:
@@ -1163,17 +1209,18 @@ def paged_attention_rel(ctx, q: torch.Tensor, cache_slot: torch.Tensor, group: i
         elif nd:
             with _timed("attention_window_decode", *cost(0, nd)):
                 attention_window(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, 0, nd, 1, n_heads, n_kv_heads, D,
-                                 v_head_dim, page, scale, window, keep_first, softcap, out, sink=sink, gate_col=gate_col, chunk=chunk or 0)
+                                 v_head_dim, page, scale, window, keep_first, softcap, out, sink=sink, gate_col=gate_col, chunk=chunk or 0,
+                                 slopes=slopes)
         if ctx.n_seqs > nd:
             with _timed("attention_window", *cost(nd, ctx.n_seqs)):
                 attention_window(q, cache_slot, bt, ctx.q_start, ctx.seq_lens, nd, ctx.n_seqs - nd, ctx.max_query_len,
                                  n_heads, n_kv_heads, D, v_head_dim, page, scale, window, keep_first, softcap, out,
-                                 sink=sink, gate_col=gate_col, chunk=chunk or 0)
+                                 sink=sink, gate_col=gate_col, chunk=chunk or 0, slopes=slopes)
         return out
     with _timed("attention_plain", *cost(0, ctx.n_seqs), "fp32" if q.dtype == torch.float32 else "bf16"):
         return attention_rel_ref(q, cache_slot, bt, ctx.seq_of_token, ctx.positions, n_heads, n_kv_heads, head_dim,
                                  v_head_dim, page, scale, window, dist_bias, temp_coef, temp_every, out, softcap, keep_first,
-                                 sink=sink, gate_col=gate_col, chunk=chunk or 0)
+                                 sink=sink, gate_col=gate_col, chunk=chunk or 0, slopes=slopes)
 
 
 def gated_linear(ctx, h: torch.Tensor, gate_up: torch.Tensor, mid: torch.Tensor, act: str, limit: float = 0.0) -> torch.Tensor:
@@ -1203,6 +1250,24 @@ def moe_top(z: torch.Tensor, bias: Optional[torch.Tensor], top: int, mode: str, 
                                  1 if mode == "softmax" else 0, int(renorm), _ptr(ids), _ptr(weights), _stream()))
 
 
+def moe_choose(z: torch.Tensor, outputs: int, correction: torch.Tensor, top: int, groups: int, groups_kept: int, ids: torch.Tensor,
+               weights: torch.Tensor) -> None:
+    """From 32-bit router logits (the first ``outputs`` columns of z): s = their softmax, the ``top`` largest entries of
+    s + correction (the lower index wins a tie; inside the ``groups_kept`` best of ``groups`` equal groups of neighbours,
+    if there are groups) as ids[n, k] in descending order, and weights[n, k] = s over the chosen ones' sum (+ 1e-20)."""
+    _dev(z, correction, ids, weights)
+    _rows_2d(z, "z")
+    N = z.shape[0]
+    _need(z.dtype == torch.float32 and z.shape[1] >= outputs, "moe_choose: router logits must be float32 [N, >= outputs]")
+    _need(correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == outputs,
+          "moe_choose: the correction must be float32 with one entry an output")
+    _need(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= N * top and weights.dtype == torch.float32
+          and weights.is_contiguous() and weights.numel() >= N * top, "moe_choose: ids int32 and weights float32, [N, top]")
+    with _timed("moe_choose", N * outputs * 4 + N * top * 8, N * outputs * (top + 6), "fp32"):
+        _check(_lib().da_moe_choose(_ptr(z), z.stride(0), _ptr(correction), N, outputs, top, int(groups), int(groups_kept), _ptr(ids),
+                                    _ptr(weights), _stream()))
+
+
 def _moe_mfma_ok(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor) -> bool:
     return (_MODE == "tuned" and h.dtype == torch.bfloat16 and gate_up.dtype == torch.bfloat16 and h.shape[1] % 8 == 0
             and h.stride(0) % 8 == 0 and down.shape[2] % 8 == 0 and h.data_ptr() % 16 == 0
@@ -1226,11 +1291,14 @@ def moe_top_logistic(z: torch.Tensor, top: int, renorm: bool, ids: torch.Tensor,
 def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up: torch.Tensor, down: torch.Tensor,
                     n_experts: int, top: int, weight: float, act: str, x: torch.Tensor, accumulate: bool,
                     ids: Optional[torch.Tensor] = None, pair_weights: Optional[torch.Tensor] = None,
-                    gated: bool = True, weight_input: bool = False, limit: float = 0.0) -> torch.Tensor:
+                    gated: bool = True, weight_input: bool = False, limit: float = 0.0, identity: bool = False,
+                    shared_out: Optional[torch.Tensor] = None, shared_logit: Optional[torch.Tensor] = None) -> torch.Tensor:
     """x (+)= sum_k weight_k * expert_k(h) (or, with ``weight_input``, sum_k expert_k(weight_k * h)): route, two
     grouped products, combine.  The experts of a row come from ``table[token, k]`` or from ``ids[n, k]``; the
     weights are ``pair_weights[n, k]`` or the one ``weight``.  ``gated``: the first matrix of an expert is gate | up
     ([2 inner, width]) and its middle is act(gate h) * (up h); else it is [inner, width] and the middle is act(up h).
+    ``identity``: ids from ``n_experts`` on name experts whose output is h itself.  ``shared_out`` with ``shared_logit``: see
+    ``moe_combine``.
     bfloat16 steps run the grouped products on the matrix cores; 32-bit and the reference mode use the plain ones."""
     N, width = h.shape
     inner = down.shape[2]
@@ -1309,8 +1377,10 @@ def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up
                                             _stream()))
         moe_down_ref(mid, row_of_slot, tile_expert, down, pair_out, tiles)
     if weight_input:               # the weights already sit in the rows
-        return moe_combine(pair_out, slot_of_pair, None, 1.0, top, x, accumulate)
-    return moe_combine(pair_out, slot_of_pair, pair_weights, weight, top, x, accumulate)
+        _need(not identity, "experts: an expert that hands its input on takes its weight on the output")
+        return moe_combine(pair_out, slot_of_pair, None, 1.0, top, x, accumulate, None, shared_out, shared_logit)
+    return moe_combine(pair_out, slot_of_pair, pair_weights, weight, top, x, accumulate, h if identity else None, shared_out,
+                       shared_logit)
 
 
 # ------------------------------------------------------------------------------- rotation, latent attention
@@ -1623,6 +1693,76 @@ def gla_serve(ctx, proj: torch.Tensor, q_off: int, k_off: int, v_off: int, gate_
             _check(_lib().da_gla_chunked(*args(), nd, S - nd, H, D, Dv, int(bool(write)), longest, _ptr(scratch),
                                          scratch.numel(), _stream()))
     return y
+
+
+# ------------------------------------------------------------------------------- recurrence with one number a channel
+def rglru_walk(ctx, u: torch.Tensor, raw: torch.Tensor, block: int, rate: torch.Tensor, y: torch.Tensor, act: str,
+               state: torch.Tensor, out: torch.Tensor, write: bool = True) -> torch.Tensor:
+    """S <- a S + sqrt(1 - a^2) * logistic(i) * u, a = exp(rate * logistic(r)), out = S * act(y), token by token over every
+    sequence of the step (csrc/rglru.hip).  ``u`` [N, C] in the step's dtype; ``raw`` [N, 2 C] 32-bit, block by block of
+    ``block`` channels the r's and then the i's; ``rate`` float32 [C]; the first C entries of ``state``'s rows are read at
+    each portion's start and, with ``write``, written at its end."""
+    _dev(u, raw, rate, y, state, out)
+    for t_, nm in ((u, "u"), (raw, "raw"), (y, "y"), (out, "out")):
+        _rows_2d(t_, nm)
+    N, C = u.shape
+    ld = _state_args(state, "rglru_walk")
+    _need(raw.dtype == torch.float32 and raw.shape[0] == N and raw.shape[1] >= 2 * C, "rglru_walk: raw must be float32 [N, 2 C]")
+    _need(u.dtype == y.dtype == out.dtype and y.shape[0] == N and y.shape[1] >= C and out.shape[0] == N and out.shape[1] >= C,
+          "rglru_walk: u, y and out must be [N, C] of one dtype")
+    _need(rate.dtype == torch.float32 and rate.is_contiguous() and rate.numel() == C and ld >= C and C % block == 0,
+          "rglru_walk: rate float32 [C], state rows of C entries and more")
+    _need(ctx.q_start.numel() >= ctx.n_seqs + 1 and ctx.state_slots.numel() >= ctx.n_seqs, "rglru_walk: the step's arrays are too short")
+    with _timed("rglru_walk", N * C * (3 * u.element_size() + 8) + ctx.n_seqs * C * 8, 12 * N * C, "fp32"):
+        _check(_lib().da_rglru_walk(_ptr(u), _dt(u), u.stride(0), _ptr(raw), raw.stride(0), int(block), _ptr(rate), _ptr(y),
+                                    y.stride(0), ACTIVATIONS[act], _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start),
+                                    _ptr(out), out.stride(0), ctx.n_seqs, C, int(bool(write)), _stream()))
+    return out
+
+
+def rglru_serve_takes(yx: torch.Tensor, block: int) -> bool:
+    """Whether the forms for bfloat16 serving take blocks of so many channels (and the kernel mode allows them)."""
+    return _MODE == "tuned" and yx.dtype == torch.bfloat16 and bool(_lib().da_rglru_serve_takes(int(block)))
+
+
+def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, gate_w: torch.Tensor, gate_b: torch.Tensor,
+                rate: torch.Tensor, act: str, state: torch.Tensor, out: torch.Tensor, write: bool = True) -> torch.Tensor:
+    """The recurrence of a step in bfloat16 serving, from the rows ``yx`` [N, y: C | x: C] to out = S * act(y): the filter
+    of x (``conv_w`` float32 [taps, C], the last row meets the token itself; ``conv_b`` float32 [C]), the blocks' two square
+    matrices (``gate_w`` [blocks, 2 b, b], ``gate_b`` float32 [blocks, 2 b]: r's rows, then i's), and ``rglru_walk``'s
+    recurrence.  One-token sequences and portions go to a launch (or, for portions longer than a chunk, three) each.
+    ``state`` [slots, taps * C]: S, then the filter's last inputs; both move on with ``write``."""
+    _dev(yx, conv_w, conv_b, gate_w, gate_b, rate, state, out)
+    _rows_2d(yx, "yx"); _rows_2d(out, "out")
+    N, (K, C), (blocks, _, bs) = yx.shape[0], conv_w.shape, gate_w.shape
+    ld = _state_args(state, "rglru_serve")
+    _need(yx.dtype == out.dtype == gate_w.dtype == torch.bfloat16 and yx.shape[1] >= 2 * C and out.shape[0] == N and out.shape[1] >= C,
+          "rglru_serve: yx [N, 2 C] and out [N, C] in bfloat16")
+    _need(blocks * bs == C and gate_w.is_contiguous() and gate_w.shape[1] == 2 * bs, "rglru_serve: gate_w must be [blocks, 2 b, b]")
+    for t_, n_, nm in ((conv_w, K * C, "conv_w"), (conv_b, C, "conv_b"), (gate_b, 2 * C, "gate_b"), (rate, C, "rate")):
+        _need(t_.dtype == torch.float32 and t_.is_contiguous() and t_.numel() == n_, f"rglru_serve: {nm} must be float32 of {n_} entries")
+    _need(ld >= K * C, "rglru_serve: the state row is too short")
+    _need(ctx.q_start.numel() >= ctx.n_seqs + 1 and ctx.state_slots.numel() >= ctx.n_seqs, "rglru_serve: the step's arrays are too short")
+
+    def args():
+        return (_ptr(yx), yx.stride(0), _ptr(conv_w), _ptr(conv_b), _ptr(gate_w), _ptr(gate_b), _ptr(rate), ACTIVATIONS[act],
+                _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(out), out.stride(0))
+
+    nd, S = ctx.n_decode, ctx.n_seqs
+    weights = _nbytes(gate_w, gate_b, conv_w, conv_b, rate)
+    if nd:
+        with _timed("rglru_decode", nd * C * (3 * 2 + 2 * K * 4) + weights, nd * C * (4 * bs + 2 * K + 20), "bf16"):
+            _check(_lib().da_rglru_decode(*args(), 0, nd, C, bs, K, int(bool(write)), _stream()))
+    if S > nd:
+        longest = int(ctx.max_query_len)
+        chunks = -(-longest // int(_lib().da_rglru_chunk_tokens()))
+        scratch = None
+        if chunks > 1 or bs > 64:
+            scratch = ctx.buf("rglru_scratch", (S - nd) * (2 * chunks + K - 1), C, torch.float32)
+        with _timed("rglru_portion", (N - nd) * C * 3 * 2 + (S - nd) * C * 2 * K * 4 + weights, (N - nd) * C * (4 * bs + 2 * K + 20), "bf16"):
+            _check(_lib().da_rglru_portion(*args(), nd, S - nd, C, bs, K, int(bool(write)), longest, _ptr(scratch),
+                                           0 if scratch is None else scratch.numel(), _stream()))
+    return out
 
 
 # ------------------------------------------------------------------------------- short filter and scan

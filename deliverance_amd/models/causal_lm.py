@@ -21,6 +21,11 @@ from ..registry import Architecture, ModelSupport, read_config_json
 from ..weights.loader import load_declared
 
 
+def _changes_stream(call) -> bool:
+    """Whether something happens to the stream right before this run-order entry."""
+    return bool(getattr(call, "mix_input", False) or getattr(call, "add_input", False) or getattr(call, "add_step", None) is not None)
+
+
 class CausalLM:
     def __init__(self, config: ModelConfig, params: dict, dtype: torch.dtype, device):
         self.config = config
@@ -47,6 +52,15 @@ class CausalLM:
                 raise ValueError(f"the input mix is {list(self.input_mix.shape)}, expected {[config.width, 2 * config.width]}")
         elif any(getattr(c, "mix_input", False) for c in config.schedule):
             raise ValueError("the run order mixes the stream with the embedding output, but the model has no matrix for it")
+        # vectors [n, width] of which run-order entries add one to the stream (32-bit)
+        self.step_vectors, self.adds_input = None, any(getattr(c, "add_input", False) for c in config.schedule)
+        n_steps = int(getattr(config, "step_vectors", 0))
+        if n_steps:
+            self.step_vectors = params["step_vectors"]["weight"].to(device=device, dtype=torch.float32).contiguous()
+            if tuple(self.step_vectors.shape) != (n_steps, config.width):
+                raise ValueError(f"the step vectors are {list(self.step_vectors.shape)}, expected {[n_steps, config.width]}")
+        if any(c.add_step is not None and not (0 <= c.add_step < n_steps) for c in config.schedule if hasattr(c, "add_step")):
+            raise ValueError(f"the run order names a step vector that is not among the model's {n_steps}")
         head = params["head"]["weight"]
         if head is emb["tokens"] and self.token_table.dtype == dtype:
             self.head_weight = self.token_table            # tied: one buffer, two uses
@@ -73,7 +87,7 @@ class CausalLM:
             if b.mixer_scale is not None or b.ff_scale is not None:
                 names.append("elementwise")
         names += [u for n in norms if n is not None for u in n.kernel_units]
-        if self.input_mix is not None or self.config.logit_softcap > 0.0:
+        if self.input_mix is not None or self.step_vectors is not None or self.adds_input or self.config.logit_softcap > 0.0:
             names.append("elementwise")
         return sorted(set(names))
 
@@ -127,12 +141,18 @@ class CausalLM:
             # [stream | embedding output] in the compute dtype; the right half is written once a step
             both = ctx.buf("input_mix", N, 2 * self.config.width, ctx.dtype)
             ops.concat_rows(x, both, self.config.width)
+        first = None
+        if self.adds_input:                             # the embedding output, as run-order entries add it again
+            first = ops.copy_rows(x, ctx.buf("embedded", N, self.config.width, torch.float32))
         h = None                                        # a block's input that the block before has made
         for call, after in zip(self.config.schedule, (*self.config.schedule[1:], None)):
             if getattr(call, "mix_input", False):       # x <- W [x; embedding output]
                 ops.concat_rows(x, both, 0)
                 ops.linear(both, self.input_mix, None, x)
-            ahead = after is not None and not getattr(after, "mix_input", False) and self.blocks[after.layer].takes_stream_ahead()
+            again, vec = getattr(call, "add_input", False), getattr(call, "add_step", None)
+            if again or vec is not None:                # x <- x + embedding output + step vector
+                ops.add_rows(x, first if again else None, None if vec is None else self.step_vectors[vec])
+            ahead = after is not None and not _changes_stream(after) and self.blocks[after.layer].takes_stream_ahead()
             h = self.blocks[call.layer].forward(ctx, x, call, h_ready=h, next_pre=STREAM_ITSELF if ahead else None)
             if debug:
                 ctx.emit(call.layer, "layer_output", x)

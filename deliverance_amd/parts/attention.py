@@ -15,8 +15,9 @@ position i sees j <= i when i - j < window or j < keep_first), values that are t
 values), a term without key or value in the softmax's denominator (``sink``: exp(0), or exp of a learned number per
 head), a logistic gate of one more projection of the input on the heads' results (``out_gate``: its rows are stacked
 behind q | k | v in the same product), chunks in place of a window (``chunk``: a row sees the earlier keys of its own chunk
-of positions), and another layer's keys and values (``shared_kv``: the product has query and gate rows only, and the run
-order names the slot that the other layer has written).
+of positions), another layer's keys and values (``shared_kv``: the product has query and gate rows only, and the run
+order names the slot that the other layer has written), and slopes by distance (``distance_slopes``: a score loses its
+head's number for every position between query and key).
 Reference: core/src/main/java/io/teknek/deliverance/generator/CausalSelfAttention.java:226-420
 (projections :266-291, cache write :315-336, scores/softmax/weighted sum :458-532, output
 projection :385-408); the residual add is TransformerBlock.java:176.
@@ -117,6 +118,12 @@ class CausalSelfAttention(Mixer):
                 raise ValueError(f"distance-bias table is {list(table.shape)}, expected "
                                  f"{[db.n_buckets or 'rows', self.n_heads]}")
             self.dist_bias = bias_by_distance(table, db.max_distance).to(device)
+        slopes = getattr(spec, "distance_slopes", None)
+        self.slopes = None                            # 32-bit, one a query head
+        if slopes is not None:
+            if len(slopes) != self.n_heads:
+                raise ValueError(f"{len(slopes)} slopes by distance for {self.n_heads} heads")
+            self.slopes = torch.tensor([float(v) for v in slopes], dtype=torch.float32, device=device)
         qt = getattr(spec, "query_temperature", None)
         self.temp_coef, self.temp_every = (float(qt.coef), int(qt.every)) if qt is not None else (0.0, 0)
         if qt is not None and self.temp_every <= 0:
@@ -137,7 +144,7 @@ class CausalSelfAttention(Mixer):
                                  f"{nk if self.k_gain is None else self.k_gain.numel()} entries, expected {nq} and {nk}")
         self.extras = (self.dist_bias is not None or self.temp_every > 0 or self.v_head_dim != self.head_dim
                        or self.softcap > 0.0 or self.keep_first > 0 or self.sink is not None or self.out_gate is not None
-                       or self.chunk is not None)
+                       or self.chunk is not None or self.slopes is not None)
         self.position = None
         if spec.position is not None and spec.position.kind != "none":
             self.position = build_position(spec.position, params.get("position", {}), dtype, device)
@@ -157,7 +164,7 @@ class CausalSelfAttention(Mixer):
         if not self.extras:
             return out + (("attn_decode", "attn_prefill") if D % 16 == 0 else ("attn_ref",))
         scores_only = self.v_head_dim == D and D % 16 == 0 and D <= 128 and self.softcap == 0.0 and not self.keep_first
-        if scores_only and self.sink is None and self.out_gate is None and self.chunk is None:
+        if scores_only and self.sink is None and self.out_gate is None and self.chunk is None and self.slopes is None:
             return out + ("attn_decode_rel", "attn_prefill_rel")
         if D % 8 or max(D, self.v_head_dim) > 128 or self.dist_bias is not None or self.temp_every:
             return out + ("attn_rel",)
@@ -283,7 +290,7 @@ class CausalSelfAttention(Mixer):
             ops.paged_attention_rel(ctx, qkv if self.out_gate else qkv[:, :self.q_cols], slot, group, self.n_heads, self.n_kv_heads, self.head_dim,
                                     self.v_head_dim, self.scale, self.window, self.dist_bias, self.temp_coef,
                                     self.temp_every, o, softcap=self.softcap, keep_first=self.keep_first, sink=self.sink,
-                                    gate_col=gate_off if self.out_gate else -1, chunk=self.chunk)
+                                    gate_col=gate_off if self.out_gate else -1, chunk=self.chunk, slopes=self.slopes)
         else:
             ops.paged_attention(ctx, qkv[:, :self.q_cols], slot, group, self.n_heads, self.scale, self.window, o)
         if ctx.debug_hook is not None:      # the reference's stage names (CausalSelfAttention.java:299-301,384)

@@ -3,7 +3,8 @@ adding into the 32-bit residual stream.
 Reference: core/src/main/java/io/teknek/deliverance/generator/TransformerBlock.java:161-200
 (five optional norm places :26-32; GPT-2 uses the two pre-norms :35-41; a norm after a part acts
 on the part's output before the residual add :172-176,184-188; the part's output may join the stream
-times a constant :260-272; the fifth norm acts on the stream at the block's end :199)."""
+times a constant :260-272; the fifth norm acts on the stream at the block's end :199).  A block whose parts lie side by
+side (``LayerSpec.parallel``) has one norm: both parts read its output and add into the stream."""
 from __future__ import annotations
 
 import torch
@@ -24,6 +25,11 @@ class Block:
         self.post_ff_norm = norm(spec.post_ff_norm, "post_ff_norm")
         self.post_block_norm = norm(getattr(spec, "post_block_norm", None), "post_block_norm")
         self.residual_multiplier = float(getattr(spec, "residual_multiplier", 1.0))
+        self.parallel = bool(getattr(spec, "parallel", False))
+        if self.parallel and (spec.feed_forward is None or self.residual_multiplier != 1.0 or any(
+                n is not None for n in (self.post_mixer_norm, self.pre_ff_norm, self.post_ff_norm, self.post_block_norm))
+                or getattr(spec, "mixer_scale", False) or getattr(spec, "ff_scale", False)):
+            raise ValueError("parts side by side need a feed-forward and take one norm, in front of both, and no scales")
         # A learned scale per channel on a part's result ("layer scale").  Behind a norm that can take it into its
         # gain (``Norm.scaled_by``) it costs nothing; else it is applied while the result joins the stream.
         self.mixer_scale, self.post_mixer_norm = self._scale(spec, params, "mixer_scale", self.post_mixer_norm, dtype, device)
@@ -96,10 +102,26 @@ class Block:
         convert it in passing (``forward(next_pre=STREAM_ITSELF)`` there, ``h_ready`` here)."""
         return self.pre_mixer_norm is None
 
+    def _forward_parallel(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None):
+        """x += mixer(h) + ff(h), h = norm(x): the norm's output is a buffer of its own, so the mixer may add into the
+        stream before the feed-forward reads."""
+        h = h_ready if h_ready is not None else Block._normed(ctx, x, self.pre_mixer_norm)
+        self.mixer.forward(ctx, h, x, call)
+        if ctx.debug_hook is not None:
+            ctx.emit(call.layer, "post_attention_residual", x)
+        self.feed_forward.forward(ctx, h, x)
+        if ctx.debug_hook is not None:
+            chosen = getattr(self.feed_forward, "last_choice", None)
+            if chosen is not None:
+                ctx.emit(call.layer, "expert_choice", chosen)
+            ctx.emit(call.layer, "post_ff_residual", x)
+
     def forward(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None, next_pre=None):
         """Runs the block.  ``h_ready``: the mixer's input, when the block before has made it.  ``next_pre``: what the
         block behind wants of the new stream (``STREAM_ITSELF`` or None); returns it when the block's last norm could make
         it in the same pass, else None."""
+        if self.parallel:
+            return self._forward_parallel(ctx, x, call, h_ready)
         if ctx.debug_hook is not None or self.post_block_norm is not None:
             next_pre = None
         fused = getattr(self.mixer, "forward_normed", None)

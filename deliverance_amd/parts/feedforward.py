@@ -83,10 +83,14 @@ class ExpertsFeedForward(FeedForward):
     with what weights.  ``token_table``: row ``token id`` of an integer table names them, each with weight 1 / top.
     ``logistic_top``: 32-bit logits from a matrix; the ``top`` largest logistic scores, which are the weights.
     ``softmax_top``: 32-bit logits from a matrix and a bias; the ``top`` largest logits, weighted by the softmax over
-    just those.
+    just those.  ``softmax_all``: the softmax over all logits plus a correction decides, inside the best groups if there
+    are groups; the weights are the chosen softmax scores over their sum.  Router outputs behind the experts' name experts
+    that hand the input on (``identity``): they have no matrices and join where the pairs are added up.
     The step's (token, choice) pairs are laid out expert by expert on the device (``ops.moe_route``), two grouped
     products run over that layout, and the pairs' results are added up per token; a weight on the input scales
-    the pair's row in the first product.  A shared expert, if any, runs as a dense feed-forward for every token.
+    the pair's row in the first product.  A shared expert, if any, runs as a dense feed-forward for every token; with a gate
+    a token (``shared_token_gate``, one more row of the router's product) its result goes to a buffer of its own and joins
+    where the pairs are added up.
     Nothing is read back to the host, so a step can be recorded."""
     graph_safe = True
     can_store = True
@@ -100,14 +104,23 @@ class ExpertsFeedForward(FeedForward):
         if self.activation not in ops.ACTIVATIONS:
             raise ValueError(f"unknown activation {self.activation!r}")
         self.limit = float(getattr(spec, "limit", 0.0) or 0.0)
-        if self.router not in ("token_table", "logistic_top", "softmax_top"):
-            raise ValueError(f"unknown router {self.router!r}; known: 'token_table', 'logistic_top', 'softmax_top'")
+        if self.router not in ("token_table", "logistic_top", "softmax_top", "softmax_all"):
+            raise ValueError(f"unknown router {self.router!r}; known: 'token_table', 'logistic_top', 'softmax_top', 'softmax_all'")
+        self.groups, self.groups_kept = int(getattr(spec, "groups", 0)), int(getattr(spec, "groups_kept", 0))
+        self.identity = int(getattr(spec, "identity", 0))
+        self.token_gate = bool(getattr(spec, "shared_token_gate", False)) and bool(getattr(spec, "shared_inner", 0))
+        self.outputs = self.n_experts + self.identity            # the router's
+        if self.router != "softmax_all" and (self.groups or self.identity or self.token_gate):
+            raise ValueError("groups, experts that hand the input on and a shared gate a token go with the router 'softmax_all'")
+        if self.groups and (self.outputs % self.groups or not (1 <= self.groups_kept <= self.groups)):
+            raise ValueError(f"{self.outputs} router outputs in {self.groups} equal groups of which {self.groups_kept} are kept")
         if self.activation == "glu_capped" and not (self.gated and self.limit > 0.0):
             raise ValueError(f"the capped gated form needs gated experts and a positive limit, found {self.limit}")
         if self.weight_on not in ("output", "input"):
             raise ValueError(f"a pair's weight goes on the 'output' or the 'input', not {self.weight_on!r}")
-        if not (1 <= self.top <= self.n_experts):
-            raise ValueError(f"top {self.top} of {self.n_experts} experts")
+        can = self.outputs // self.groups * self.groups_kept if self.groups else self.outputs
+        if not (1 <= self.top <= can):
+            raise ValueError(f"top {self.top} of {can} experts")
         first_rows = (2 if self.gated else 1) * self.inner
         # [experts, 2 inner | inner, width]: gate | up, or up alone
         self.gate_up_weight = to_matrix(params["gate_up_weight" if self.gated else "up_weight"], dtype, device)
@@ -129,9 +142,20 @@ class ExpertsFeedForward(FeedForward):
             if self.weight_on != "output":
                 raise ValueError("a table router gives no weight to put on the input")
         else:
-            self.router_weight = to_matrix(params["router_weight"], dtype, device)     # [experts, width]
-            if tuple(self.router_weight.shape) != (self.n_experts, self.width):
-                raise ValueError(f"router weight is {list(self.router_weight.shape)}, expected {[self.n_experts, self.width]}")
+            router = params["router_weight"]                                           # [outputs, width]
+            if tuple(router.shape) != (self.outputs, self.width):
+                raise ValueError(f"router weight is {list(router.shape)}, expected {[self.outputs, self.width]}")
+            if self.token_gate:                                                        # its row rides behind the router's
+                row = params["shared_token_gate"].reshape(1, -1)
+                if row.shape[1] != self.width:
+                    raise ValueError(f"the shared expert's gate has {row.shape[1]} entries for width {self.width}")
+                router = torch.cat([router, row.to(router.dtype)], 0)
+            self.router_weight = to_matrix(router, dtype, device)
+        self.correction = None
+        if self.router == "softmax_all":
+            self.correction = params["router_correction"].to(device=device, dtype=torch.float32).contiguous()
+            if self.correction.numel() != self.outputs:
+                raise ValueError(f"the correction has {self.correction.numel()} entries for {self.outputs} router outputs")
         self.router_bias = None
         if getattr(spec, "router_bias", False):
             self.router_bias = params["router_bias"].to(device=device, dtype=torch.float32).contiguous()
@@ -160,20 +184,31 @@ class ExpertsFeedForward(FeedForward):
         ids = weights = None
         if self.router_weight is not None:
             N = h.shape[0]
-            z = ctx.buf("moe_logits", N, self.n_experts, torch.float32)      # 32-bit sums of the products
+            z = ctx.buf("moe_logits", N, self.router_weight.shape[0], torch.float32)      # 32-bit sums of the products
             ops.linear(h, self.router_weight, None, z)
             ids = ctx.buf("moe_ids", N, self.top, torch.int32)
             weights = ctx.buf("moe_weights", N, self.top, torch.float32)
-            if self.router == "softmax_top":
+            if self.router == "softmax_all":
+                ops.moe_choose(z, self.outputs, self.correction, self.top, self.groups, self.groups_kept, ids, weights)
+            elif self.router == "softmax_top":
                 ops.moe_top(z, self.router_bias, self.top, "softmax", False, ids, weights)
             else:
                 ops.moe_top(z, self.router_bias, self.top, "logistic", self.renormalize, ids, weights)
         self.last_choice = ids if ctx.debug_hook is not None else None      # handed to the layer debug hook
+        shared_out = None
+        if self.token_gate:
+            shared_out = ctx.buf("moe_shared_out", h.shape[0], self.width, torch.float32)
+            keep, ctx.part_accumulate = ctx.part_accumulate, False
+            try:
+                self.shared.forward(ctx, h, shared_out)
+            finally:
+                ctx.part_accumulate = keep
         ops.experts_forward(ctx, h, self.table, self.gate_up_weight, self.down_weight, self.n_experts, self.top,
                             self.weight, self.activation, x, accumulate=ctx.part_accumulate, ids=ids,
                             pair_weights=weights, gated=self.gated, weight_input=self.weight_on == "input",
-                            limit=self.limit)
-        if self.shared is not None:
+                            limit=self.limit, identity=self.identity > 0, shared_out=shared_out,
+                            shared_logit=z[:, self.outputs:] if self.token_gate else None)
+        if self.shared is not None and not self.token_gate:
             keep = ctx.part_accumulate
             ctx.part_accumulate = True          # the shared expert joins the experts' sum, stored or added above
             try:
