@@ -18,8 +18,8 @@ its fraction of the roofline; `--no-extra` leaves those two out.  Prints ONE JSO
 vocabulary, feed-forward parameters that a token uses): decode at batch 1, 8 and 64 and the prefill of 2 x 1,024
 tokens for both, at the layer sizes of GPT-2 124M and 355M, one JSON line; with `--profile-stages` also both
 models' kernel tables (stderr).  `--design pedatar` does the same for a third design beside Virudra (the closest
-of the engine's models to it), `--design pafolorn` for a fourth beside Pedatar, `--design salivik` for a fifth beside Pedatar, and
-`--design luvatar` for a sixth beside Pafolorn.
+of the engine's models to it), `--design pafolorn` for a fourth beside Pedatar, `--design salivik` for a fifth beside Pedatar,
+`--design luvatar` for a sixth beside Pafolorn, and `--design mogevik` for a seventh beside Salivik.
 """
 import argparse
 import json
@@ -527,19 +527,14 @@ def luvatar_step_flops(c, seq_lens_new):
     return fl
 
 
-def luvatar_compare(args):
-    """Decode and prefill of Luvatar beside Pafolorn (the closest of the engine's models: a linear recurrence with a decay
-    per key channel, bounded attention with normalised queries and keys, a norm behind each part and none in front, the
-    embedding table as the head) at the layer sizes of GPT-2 124M and 355M; one JSON line."""
+def measure_designs(args, out, of):
+    """Decode (batch 1, 8, 64) and prefill (2 and 8 prompts of 1,024) of every design in ``of`` (name -> its configuration,
+    step-bytes and step-flops functions) at the layer sizes of GPT-2 124M and 355M, into ``out["points"]`` and, as fractions
+    of the roofline, ``out["points_frac"]``."""
     import numpy as np
     el, dkey = 2, "bf16"
-    out = {"metric": "decode tok/s at batch 8 of Luvatar at GPT-2 124M layer sizes (beside Pafolorn at the same sizes: see points)",
-           "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": dkey, "steps": args.steps, "warmup": args.warmup,
-           "data": "synthetic (random weights drawn on the GPU, uniform-random token ids)", "points": {}, "points_frac": {}}
-    of = {"pafolorn": (pafolorn_config, pafolorn_step_bytes, pafolorn_step_flops),
-          "luvatar": (luvatar_config, luvatar_step_bytes, luvatar_step_flops)}
     for size in ("124m", "355m"):
-        for design in ("pafolorn", "luvatar"):
+        for design in of:
             rng = np.random.default_rng(0)
             config, nbytes, flops = of[design]
             cfg = config(size)
@@ -558,6 +553,19 @@ def luvatar_compare(args):
                 print(f"==== {key}", file=sys.stderr)
                 kernel_table(model, cfg, rng, args.batch, args.prompt_len)
             del model
+
+
+def luvatar_compare(args):
+    """Decode and prefill of Luvatar beside Pafolorn (the closest of the engine's models: a linear recurrence with a decay
+    per key channel, bounded attention with normalised queries and keys, a norm behind each part and none in front, the
+    embedding table as the head) at the layer sizes of GPT-2 124M and 355M; one JSON line."""
+    dkey = "bf16"
+    out = {"metric": "decode tok/s at batch 8 of Luvatar at GPT-2 124M layer sizes (beside Pafolorn at the same sizes: see points)",
+           "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": dkey, "steps": args.steps, "warmup": args.warmup,
+           "data": "synthetic (random weights drawn on the GPU, uniform-random token ids)", "points": {}, "points_frac": {}}
+    of = {"pafolorn": (pafolorn_config, pafolorn_step_bytes, pafolorn_step_flops),
+          "luvatar": (luvatar_config, luvatar_step_bytes, luvatar_step_flops)}
+    measure_designs(args, out, of)
     out["value"] = out["points"]["luvatar_124m_decode_b8"]
     out["config"] = {"model": "luvatar beside pafolorn at gpt2-124m and gpt2-355m layer sizes", "global_batch": 8,
                      "prompt_len": args.prompt_len,
@@ -565,6 +573,86 @@ def luvatar_compare(args):
                                 "attention inside chunks of 1,024 positions (GPT-2's heads on a quarter as many key heads, all "
                                 "entries rotated, sink, output gate; every second one on the keys and values of the one before) in "
                                 "turn; gated feed-forwards of 8/3 width", "parallelism": "single-gpu"}
+    print(json.dumps(out))
+    return 0
+
+
+def mogevik_config(name, n_positions=1024):
+    """A Mogevik of GPT-2 ``name``'s sizes: as many layer runs, two recurrent layers and an attention layer in turn.
+    Recurrence: as many channels as the width in blocks of GPT-2's heads' number, four taps.  Attention: GPT-2's heads of 64
+    key and 64 value entries on a quarter as many key heads, a window of 512.  Feed-forward: Salivik's sizes (8 gated
+    experts of 2/3 of the width, 2 a token, and a shared one of 4/3 of the width), two more outputs that hand the input on,
+    two groups of which one is kept.  The first three layers run twice (a loop), so the stored layers are three fewer than
+    the runs."""
+    g = MODELS[name]
+    E, H = g["n_embd"], g["n_head"]
+    rec = {"width": E, "blocks": H, "conv": 4}
+    att = {"heads": H, "kv_heads": H // 4, "dim": 64, "vdim": 64, "scale": 64 ** -0.5, "mask": {"size": 512}}
+    f, fs = (2 * E // 3) // 8 * 8, (4 * E // 3) // 8 * 8
+    mlp = {"kind": "moe", "expert": {"ff": f}, "router": {"experts": 8, "top": 2, "identity": 2, "groups": {"count": 2, "keep": 1}},
+           "shared": {"ff": fs}}
+    layers = [{"type": "attention", "mixer": att, "mlp": mlp} if i % 3 == 2 else {"type": "rglru", "mixer": rec, "mlp": mlp}
+              for i in range(g["n_layer"] - 3)]
+    return {"architecture": "Mogevik", "vocab": 50257, "width": E, "norm": {"eps": 1e-5}, "embedding": {"scale": 8.0},
+            "layers": layers, "loop": {"start": 0, "stop": 3, "times": 2}, "max_positions": n_positions,
+            # what decode_run and prefill_run read
+            "vocab_size": 50257, "n_positions": n_positions, "n_layer": g["n_layer"], "n_embd": E}
+
+
+def _mogevik_layer_params(c, L, experts_used):
+    E, m, f = c["width"], L["mixer"], L["mlp"]
+    if L["type"] == "rglru":
+        n = 3 * E * m["width"] + 2 * m["width"] ** 2 // m["blocks"] + m["conv"] * m["width"]
+    else:
+        n = E * (m["heads"] * (m["dim"] + 2 * m["vdim"]) + m["kv_heads"] * (m["dim"] + m["vdim"]))
+    return n + 3 * E * (experts_used * f["expert"]["ff"] + f["shared"]["ff"]) + (f["router"]["experts"] + f["router"]["identity"] + 1) * E
+
+
+def mogevik_step_bytes(c, el, batch, ctx_mean):
+    """What a decode step must read: every matrix of every run once (of the experts as many as ``batch`` tokens can
+    choose), the keys and values that the windows see, and the recurrences' states (read and written, 32-bit)."""
+    n, extra = c["vocab"] * c["width"], 0
+    for L in _salivik_runs(c):
+        r, m = L["mlp"]["router"], L["mixer"]
+        n += _mogevik_layer_params(c, L, min(r["experts"], r["top"] * batch))
+        if L["type"] == "rglru":
+            extra += batch * 2 * 4 * m["width"] * m["conv"]
+        else:
+            extra += batch * min(ctx_mean, m["mask"]["size"]) * m["kv_heads"] * (m["dim"] + m["vdim"]) * el
+    return n * el + extra
+
+
+def mogevik_step_flops(c, seq_lens_new):
+    """Matrix-product flops of a step (the parameters a token uses, twice; of its experts the share that has matrices) and
+    the attention's two products over the keys that each row sees."""
+    n = sum(seq_lens_new)
+    fl = 2 * len(seq_lens_new) * c["width"] * c["vocab"]
+    for L in _salivik_runs(c):
+        r, m = L["mlp"]["router"], L["mixer"]
+        fl += 2 * n * _mogevik_layer_params(c, L, r["top"] * r["experts"] / (r["experts"] + r["identity"]))
+        if L["type"] == "attention":
+            pairs = sum(sum(min(i + 1, m["mask"]["size"]) for i in range(t)) for t in seq_lens_new)
+            fl += 2 * pairs * m["heads"] * (m["dim"] + m["vdim"])
+    return fl
+
+
+def mogevik_compare(args):
+    """Decode and prefill of Mogevik beside Salivik (the closest of the engine's models: a linear recurrence, attention over
+    a window with a gate of the input on its results, routed experts beside a shared one, layers that run twice) at the
+    layer sizes of GPT-2 124M and 355M; one JSON line."""
+    out = {"metric": "decode tok/s at batch 8 of Mogevik at GPT-2 124M layer sizes (beside Salivik at the same sizes: see points)",
+           "unit": "tokens/s", "n_gpus": 1, "higher_is_better": True, "dtype": "bf16", "steps": args.steps, "warmup": args.warmup,
+           "data": "synthetic (random weights drawn on the GPU, uniform-random token ids)", "points": {}, "points_frac": {}}
+    measure_designs(args, out, {"salivik": (salivik_config, salivik_step_bytes, salivik_step_flops),
+                                "mogevik": (mogevik_config, mogevik_step_bytes, mogevik_step_flops)})
+    out["value"] = out["points"]["mogevik_124m_decode_b8"]
+    out["config"] = {"model": "mogevik beside salivik at gpt2-124m and gpt2-355m layer sizes", "global_batch": 8,
+                     "prompt_len": args.prompt_len,
+                     "mogevik": "two recurrent layers (a channel for each entry of the width in blocks of 64, four taps) and an "
+                                "attention layer (GPT-2's heads on a quarter as many key heads, window 512, slopes by distance, "
+                                "output gate) in turn; 8 gated experts of 2/3 width and 2 that hand the input on (2 a token, one "
+                                "of two groups) beside a shared one of 4/3 width; the first three layers run twice",
+                     "parallelism": "single-gpu"}
     print(json.dumps(out))
     return 0
 
@@ -579,6 +667,8 @@ def design_compare(args):
         return salivik_compare(args)
     if args.design == "luvatar":
         return luvatar_compare(args)
+    if args.design == "mogevik":
+        return mogevik_compare(args)
     return virudra_compare(args)
 
 
@@ -785,11 +875,12 @@ def main():
     ap.add_argument("--pool-tokens", type=int, default=None,
                     help="mixed workload: tokens of cache the pool holds (default: every request at full length; fewer force "
                          "requests out of the cache and back, which the line reports as preemptions)")
-    ap.add_argument("--design", default="gpt2", choices=["gpt2", "virudra", "pedatar", "pafolorn", "salivik", "luvatar"],
+    ap.add_argument("--design", default="gpt2", choices=["gpt2", "virudra", "pedatar", "pafolorn", "salivik", "luvatar", "mogevik"],
                     help="virudra: that design beside GPT-2 at equal sizes (decode at batch 1, 8, 64 and the prefill of 2,048 "
                          "tokens, at 124M and 355M layer sizes) instead of the default workload; pedatar: that design beside "
                          "Virudra, likewise; pafolorn: that design beside Pedatar, likewise; "
-                         "salivik: that design beside Pedatar, likewise; luvatar: that design beside Pafolorn, likewise")
+                         "salivik: that design beside Pedatar, likewise; luvatar: that design beside Pafolorn, likewise; "
+                         "mogevik: that design beside Salivik, likewise")
     ap.add_argument("--workload", default="decode", choices=["decode", "mixed"],
                     help="mixed: only the mixed workload, on --model (64 requests with prompts of 16 to 895 tokens arrive at "
                          "once, prompt portions of 512 tokens run beside the decoding of the others, 128 new tokens each)")

@@ -97,7 +97,7 @@ def bind_tensors(mc: ModelConfig, t: dict) -> dict:
             # the gate's rows ride behind q | k | v; they have no bias
             gate = w("g")
             d["mixer"] = {"qkv_weight": torch.cat([w("q"), w("k"), w("v"), gate], 0), "out_weight": w("o"),
-                          "qkv_bias": torch.cat([w("q.b"), w("k.b"), w("v.b"), torch.zeros(gate.shape[0], dtype=w("q.b").dtype)])}
+                          "qkv_bias": torch.cat([w("q.b"), w("k.b"), w("v.b"), w("q.b").new_zeros(gate.shape[0])])}
         if f is not None:
             q = p + "mlp."
             both = lambda e: torch.cat([t[e + "gate"], t[e + "up"]], 0)
