@@ -19,18 +19,18 @@ from ..config.specs import AttentionSpec, ExpertsFeedForwardSpec, ModelConfig, R
 from ..registry import Architecture, ModelSupport
 from ..weights.loader import TensorDecl
 
-# Random-weights distributions: matrices N(0, 0.05) (queries, keys and experts twice, routers four times that), norm gains
+# Random-weights distributions: matrices N(0, 0.1) (routers and the shared expert's gate twice that), norm gains
 # 1 + N(0, 0.1), biases N(0, 0.1), the recurrence's rates and square matrices N(0, 1) and N(0, 0.2).
-W_STD, GAIN_STD = 0.05, 0.1
+W_STD, GAIN_STD = 0.1, 0.1
 
 
 def read_config(d: dict) -> ModelConfig:
     return MogevikConfig.from_dict(d).to_model_config()
 
 
-def _gated(p: str, inner: int, E: int, std: float) -> List[TensorDecl]:
-    return [TensorDecl(p + "gate", (inner, E), "normal", std), TensorDecl(p + "up", (inner, E), "normal", std),
-            TensorDecl(p + "down", (E, inner), "normal", std)]
+def _gated(p: str, inner: int, E: int) -> List[TensorDecl]:
+    return [TensorDecl(p + "gate", (inner, E), "normal", W_STD), TensorDecl(p + "up", (inner, E), "normal", W_STD),
+            TensorDecl(p + "down", (E, inner), "normal", W_STD)]
 
 
 def _recurrence_decls(p: str, m: RealGatedRecurrenceSpec, E: int) -> List[TensorDecl]:
@@ -46,19 +46,19 @@ def _recurrence_decls(p: str, m: RealGatedRecurrenceSpec, E: int) -> List[Tensor
 def _attention_decls(p: str, m: AttentionSpec, E: int) -> List[TensorDecl]:
     H, G, D, Dv = m.n_heads, m.n_kv_heads, m.head_dim, m.value_dim
     out = []
-    for name, rows, std in (("q", H * D, 2 * W_STD), ("k", G * D, 2 * W_STD), ("v", G * Dv, W_STD)):
-        out += [TensorDecl(p + name, (rows, E), "normal", std), TensorDecl(p + name + ".b", (rows,), "normal", GAIN_STD)]
+    for name, rows in (("q", H * D), ("k", G * D), ("v", G * Dv)):
+        out += [TensorDecl(p + name, (rows, E), "normal", W_STD), TensorDecl(p + name + ".b", (rows,), "normal", GAIN_STD)]
     return out + [TensorDecl(p + "g", (H * Dv, E), "normal", W_STD), TensorDecl(p + "o", (E, H * Dv), "normal", W_STD)]
 
 
 def _experts_decls(p: str, f: ExpertsFeedForwardSpec, E: int) -> List[TensorDecl]:
     out: List[TensorDecl] = []
     for j in range(f.n_experts):
-        out += _gated(f"{p}e{j}.", f.inner, E, 2 * W_STD)
+        out += _gated(f"{p}e{j}.", f.inner, E)
     n = f.n_experts + f.identity
-    out += [TensorDecl(p + "router", (n, E), "normal", 4 * W_STD), TensorDecl(p + "correction", (n,), "normal", 0.1)]
+    out += [TensorDecl(p + "router", (n, E), "normal", 2 * W_STD), TensorDecl(p + "correction", (n,), "normal", 0.1)]
     if f.shared_inner:
-        out += _gated(p + "shared.", f.shared_inner, E, W_STD) + [TensorDecl(p + "shared.sg", (1, E), "normal", W_STD)]
+        out += _gated(p + "shared.", f.shared_inner, E) + [TensorDecl(p + "shared.sg", (1, E), "normal", 2 * W_STD)]
     return out
 
 

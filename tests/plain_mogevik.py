@@ -131,13 +131,17 @@ def expert(W, p, h, r=exact):
     return r(swish(h @ W[p + "gate"].T) * (h @ W[p + "up"].T)) @ W[p + "down"].T
 
 
+def softmax(z):
+    e = np.exp(z - z.max(axis=-1, keepdims=True))
+    return e / e.sum(axis=-1, keepdims=True)
+
+
 def choose(z, correction, top, groups=None):
     """Router logits z [T, n] -> (chosen [T, top], weights [T, top]).  The softmax over all of them plus the correction
     decides; with groups, only entries of the best ``keep`` of ``count`` runs of neighbours (a run counts as its largest
     entry) can be chosen.  The weights are the chosen softmax scores without the correction, over their sum."""
     T, n = z.shape
-    e = np.exp(z - z.max(axis=1, keepdims=True))
-    s = e / e.sum(axis=1, keepdims=True)
+    s = softmax(z)
     c = s + correction
     if groups:
         count, keep = groups["count"], groups["keep"]
@@ -147,16 +151,49 @@ def choose(z, correction, top, groups=None):
         np.put_along_axis(open_, best, True, axis=1)
         c = np.where(open_[:, :, None], runs, -np.inf).reshape(T, n)
     chosen = np.argsort(-c, axis=1, kind="stable")[:, :top]
+    return chosen, weights_of(s, chosen)
+
+
+def weights_of(s, chosen):
     w = np.take_along_axis(s, chosen, axis=1)
-    return chosen, w / (w.sum(axis=1, keepdims=True) + 1e-20)
+    return w / (w.sum(axis=1, keepdims=True) + 1e-20)
 
 
-def experts(W, p, mlp, h, r=exact, choices_out=None):
+def nearly_as_good(c, theirs, groups, slack):
+    """Whether the entries ``theirs`` are a choice from c [n] that an error of ``slack`` in the scores would explain."""
+    if len(set(theirs)) != len(theirs):
+        return False
+    open_ = np.ones(len(c), dtype=bool)
+    if groups:
+        count, keep = groups["count"], groups["keep"]
+        size = len(c) // count
+        top_of = c.reshape(count, size).max(axis=1)
+        used = {e // size for e in theirs}
+        order = np.argsort(-top_of, kind="stable")
+        if len(used) > keep or any(top_of[g] < top_of[order[keep - 1]] - slack for g in used):
+            return False
+        for g in order:                                # the groups that are left to be kept are the best of the rest
+            if len(used) < keep:
+                used.add(int(g))
+        open_ = np.isin(np.arange(len(c)) // size, sorted(used))
+    floor = np.sort(c[open_])[-len(theirs)]
+    return all(c[e] >= floor - slack for e in theirs)
+
+
+def experts(W, p, mlp, h, r=exact, routes=None, slack=0.0):
+    """``routes`` (position -> entries chosen elsewhere): followed where they are as good as the own choice within
+    ``slack`` of choice score, with the weights that go with them."""
     ro = mlp["router"]
     n = ro["experts"]
-    chosen, w = choose(h @ W[p + "router"].T, W[p + "correction"], ro["top"], ro.get("groups"))
-    if choices_out is not None:
-        choices_out.append(chosen)
+    z = h @ W[p + "router"].T
+    chosen, w = choose(z, W[p + "correction"], ro["top"], ro.get("groups"))
+    if routes is not None:
+        s = softmax(z)
+        for t in range(len(h)):
+            if t in routes and sorted(routes[t]) != sorted(chosen[t].tolist()) and \
+                    nearly_as_good(s[t] + W[p + "correction"], routes[t], ro.get("groups"), slack):
+                chosen[t] = routes[t]
+        w = weights_of(s, chosen)
     out = np.zeros_like(h)
     for e in range(n + (ro.get("identity") or 0)):
         t, k = np.nonzero(chosen == e)
@@ -181,12 +218,13 @@ def run_order(cfg):
     return order + [(i, None) for i in range(b, n)]
 
 
-def forward(cfg, W, ids, layers_out=None, r=exact, choices_out=None):
-    """Logits [T, V] of one whole sequence.  ``layers_out``: a list that receives the stream after every layer run."""
+def forward(cfg, W, ids, layers_out=None, r=exact, routes=None, slack=0.0):
+    """Logits [T, V] of one whole sequence.  ``layers_out``: a list that receives the stream after every layer run.
+    ``routes``: run -> position -> experts (see ``experts``)."""
     eps = cfg["norm"]["eps"]
     start = W["embed"][np.asarray(ids)] * cfg["embedding"]["scale"]
     x = start.copy()
-    for i, begins in run_order(cfg):
+    for run, (i, begins) in enumerate(run_order(cfg)):
         L, p = cfg["layers"][i], f"l{i}."
         if begins is not None:
             x = x + (start if begins else 0.0) + W["loop.step"][begins]
@@ -198,7 +236,7 @@ def forward(cfg, W, ids, layers_out=None, r=exact, choices_out=None):
         else:
             raise ValueError(L["type"])
         if L.get("mlp"):
-            y = y + experts(W, p + "mlp.", L["mlp"], h, r, choices_out)
+            y = y + experts(W, p + "mlp.", L["mlp"], h, r, None if routes is None else routes.get(run), slack)
         x = x + y
         if layers_out is not None:
             layers_out.append(x.copy())
