@@ -14,20 +14,20 @@
 //   da_rglru_decode   one-token sequences, from the projections to out in one launch: a workgroup takes 16 sequences and
 //                     a block of channels; filter (whose kept inputs move on), the block's two square matrices on the
 //                     matrix cores, gates, state, branch.
-//   da_rglru_portion  portions, in chunks of 64 tokens that run side by side.  A chunk of a block of channels: filter into
+//   da_rglru_portion  portions, in chunks of 32 tokens that run side by side.  A chunk of a block of channels: filter into
 //                     LDS, the square matrices on the matrix cores (16x16x32; a lane's four results of a tile are four
 //                     consecutive tokens of one channel), then the recurrence as a scan of pairs (product of the decays,
 //                     state from zero): four tokens in a lane's registers, four lanes by two exchanges, the chunk's tiles
-//                     one after the other.  A step whose portions all fit a chunk takes one launch; longer ones three:
-//                     every chunk's pair, the chunks' starting states one after the other, every chunk again from its
-//                     starting state (the second look at x and the matrices costs less than keeping two 32-bit numbers a
-//                     token and channel).
+//                     one after the other.  A step whose portions all fit a chunk takes one launch; longer ones two:
+//                     every chunk's pair, then every chunk again, with the pairs before it folded into its starting
+//                     state (the second look at x and the matrices costs less than keeping two 32-bit numbers a token and
+//                     channel).
 //
-// The order of a token's sums depends on its place in its portion only.
+// The order of a token's sums depends on its place in its portion and, for the fold, on its chunk's number only.
 #include "gemm_common.h"
 
 #define LRU_MAX_TAPS 16
-#define LRU_TOK 64            // tokens of a chunk
+#define LRU_TOK 32            // tokens of a chunk
 #define LRU_MAX_BLOCK 256
 #define LRU_LOG2E 1.4426950408889634f
 
@@ -125,6 +125,17 @@ __device__ __forceinline__ void lru_load8(const float* p, float* f) {
 __device__ __forceinline__ void lru_store8(float* p, const float* f) {
   *(float4*)p = make_float4(f[0], f[1], f[2], f[3]);
   *(float4*)(p + 4) = make_float4(f[4], f[5], f[6], f[7]);
+}
+
+// A pair (product of decays, state from zero) a lane; the four lanes of a channel (16 apart) hold pieces of time in order.
+// Afterwards a lane's pair is that of everything up to its own piece.
+__device__ __forceinline__ void lru_fold_lanes(int lane, int g, float& p, float& s) {
+#pragma unroll
+  for (int back = 16; back <= 32; back *= 2) {
+    const int from = lane - back >= 0 ? lane - back : lane;
+    const float bp = __shfl(p, from, DA_WAVE), bs = __shfl(s, from, DA_WAVE);
+    if (16 * g >= back) { s = p * bs + s; p = p * bp; }
+  }
 }
 
 // KS: pieces of 32 along a block's channels; a wavefront owns 16 channels, its two matrices' rows in registers.
@@ -226,13 +237,15 @@ rglru_decode_kernel(LruIn in, int seq0, int n) {
 
 #define LRU_WHOLE 0     // portions of one chunk: state from and to the slot
 #define LRU_PAIRS 1     // a chunk's pair (product of its decays, its state from zero) into `ends`
-#define LRU_AGAIN 2     // a chunk from its starting state, which `ends` holds by now
+#define LRU_AGAIN 2     // a chunk from its starting state
+#define LRU_FOLD 8      // pairs that a lane asks for at once
 
 // Workgroup (block of channels and 64 of them, chunk, portion); wavefront w owns 16 channels.  ends: [portion][chunk][2][C].
-// tails: the filter's kept inputs as they were before the step, [portion][K - 1][C] (LRU_AGAIN; else the slot's).
+// old: [portion][K][C], what the slots held before the step (state, then kept inputs; zeros without a slot): the first
+// chunks of LRU_PAIRS write it down, LRU_AGAIN reads it, and its last chunks write the slots.
 template <int KS, int KT, int MODE>
 __global__ void __launch_bounds__(4 * DA_WAVE)
-rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int max_chunks, const float* __restrict__ tails) {
+rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int max_chunks, float* __restrict__ old) {
   constexpr int PITCH = KS * 32 + 8, YP = 64 + 8;
   __shared__ __attribute__((aligned(16))) bf16_t us[LRU_TOK][PITCH];
   __shared__ __attribute__((aligned(16))) bf16_t ys[MODE == LRU_PAIRS ? 1 : LRU_TOK][YP];
@@ -249,12 +262,32 @@ rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int 
   uint4 wr[KS], wi[KS];
   if (cols) lru_load_gates<KS>(in, b, n0, lane, wr, wi);
   const float br = in.gate_b[(size_t)b * 2 * in.bs + ch], bi = in.gate_b[(size_t)b * 2 * in.bs + in.bs + ch], rate = in.rate[c];
-  float* const pair = ends + (((size_t)blockIdx.z * max_chunks + chunk) * 2) * in.C + c;
+  float* const row = in.state + (size_t)(slot >= 0 ? slot : 0) * in.state_ld;
+  float* const was = MODE == LRU_WHOLE ? nullptr : old + (size_t)blockIdx.z * in.K * in.C;
+  const float* tail = MODE == LRU_AGAIN ? was + in.C : (slot >= 0 ? row + in.C : nullptr);
   float start = 0.f;
-  if (MODE == LRU_WHOLE) start = slot >= 0 ? in.state[(size_t)slot * in.state_ld + c] : 0.f;
-  if (MODE == LRU_AGAIN) start = pair[in.C];
-  const float* tail = MODE == LRU_AGAIN ? tails + (size_t)blockIdx.z * (in.K - 1) * in.C
-                                        : (slot >= 0 ? in.state + (size_t)slot * in.state_ld + in.C : nullptr);
+  if (MODE == LRU_WHOLE) start = slot >= 0 ? row[c] : 0.f;
+  if (MODE == LRU_AGAIN) start = was[c];
+  // the pairs of the chunks before this one: a quarter of them, in a row, a group of 16 lanes; the first ones are asked
+  // for here (chunks that are not there read the first and count as nothing)
+  const float* const before = ends + (size_t)blockIdx.z * max_chunks * 2 * in.C + c;
+  const int per = (chunk + 3) / 4, k_first = g * per, k_end = k_first + per < chunk ? k_first + per : chunk;
+  float fp[LRU_FOLD], fs[LRU_FOLD];
+  auto ask = [&](int k0) {
+#pragma unroll
+    for (int q = 0; q < LRU_FOLD; ++q) {
+      const int k = k0 + q < k_end ? k0 + q : 0;
+      fp[q] = before[(size_t)k * 2 * in.C];
+      fs[q] = before[(size_t)k * 2 * in.C + in.C];
+    }
+  };
+  if (MODE == LRU_AGAIN && chunk > 0) ask(k_first);
+  if (MODE == LRU_PAIRS && chunk == 0) {
+    for (int e = t; e < 64 * in.K; e += 4 * DA_WAVE) {
+      const int k = e / 64, q = part * 64 + e % 64;
+      if (q < in.bs) was[(size_t)k * in.C + c0 + q] = slot >= 0 ? row[(size_t)k * in.C + c0 + q] : 0.f;
+    }
+  }
   if (MODE != LRU_PAIRS) {
     // the branch's entries of this workgroup's 64 channels, 16 bytes a thread
     for (int e = t; e < LRU_TOK * 8; e += 4 * DA_WAVE) {
@@ -296,18 +329,34 @@ rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int 
     *(uint4*)&us[tok][c8] = lru_pack8(acc);
   }
   __syncthreads();
-  if (MODE == LRU_WHOLE && parts == 1 && in.write && slot >= 0) {
-    // the kept inputs after the step (every read of the old ones lies before the barrier, and nobody else reads these
-    // channels'): a channel a thread, the ones that stay moved on in ascending order
-    float* tp = in.state + (size_t)slot * in.state_ld + in.C + c0;
-    for (int q = t; q < in.bs; q += 4 * DA_WAVE)
+  if ((MODE == LRU_WHOLE || (MODE == LRU_AGAIN && t0 + LRU_TOK >= len)) && in.write && slot >= 0) {
+    // the kept inputs after the step, a channel of this workgroup's a thread, the ones that stay moved on in ascending
+    // order (with the slot itself as their source every read of the old ones lies before the barrier, and nobody else
+    // reads these channels')
+    for (int q = part * 64 + t; q < in.bs && q < part * 64 + 64; q += 4 * DA_WAVE)
       for (int k = 0; k < in.K - 1; ++k) {
         const int r = len - (in.K - 1) + k;
-        tp[(size_t)k * in.C + q] = r >= 0 ? bf16_to_f32(in.yx[(size_t)(first + r) * in.ld + in.C + c0 + q])
-                                          : tp[(size_t)(in.K - 1 + r) * in.C + q];
+        row[(size_t)(k + 1) * in.C + c0 + q] = r >= 0 ? bf16_to_f32(in.yx[(size_t)(first + r) * in.ld + in.C + c0 + q])
+                                                      : tail[(size_t)(in.K - 1 + r) * in.C + c0 + q];
       }
   }
   if (cols) {
+    if (MODE == LRU_AGAIN && chunk > 0) {
+      float ip = 1.f, is = 0.f;
+      for (int k0 = k_first;;) {
+#pragma unroll
+        for (int q = 0; q < LRU_FOLD; ++q)
+          if (k0 + q < k_end) {
+            is = fp[q] * is + fs[q];
+            ip = ip * fp[q];
+          }
+        k0 += LRU_FOLD;
+        if (k0 - k_first >= per) break;                             // (the same for the wavefront)
+        ask(k0);
+      }
+      lru_fold_lanes(lane, g, ip, is);
+      start = __shfl(ip, 48 + fr, DA_WAVE) * start + __shfl(is, 48 + fr, DA_WAVE);
+    }
     float run_p = 1.f, run_s = start;                               // everything before the tile: decays' product, state
 #pragma unroll
     for (int i = 0; i < LRU_TOK / 16; ++i) {
@@ -329,16 +378,9 @@ rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int 
         p[r] = r ? p[r ? r - 1 : 0] * a : a;
         st[r] = r ? a * st[r ? r - 1 : 0] + add : add;
       }
-      // the lanes before this one that hold earlier tokens of the channel: 16, then 32 lanes back
+      // with the lanes before this one that hold earlier tokens of the channel
       float ip = p[3], is = st[3];
-      {
-        const float bp = __shfl(ip, lane - 16 >= 0 ? lane - 16 : lane, DA_WAVE), bs_ = __shfl(is, lane - 16 >= 0 ? lane - 16 : lane, DA_WAVE);
-        if (g >= 1) { is = ip * bs_ + is; ip = ip * bp; }
-      }
-      {
-        const float bp = __shfl(ip, lane - 32 >= 0 ? lane - 32 : lane, DA_WAVE), bs_ = __shfl(is, lane - 32 >= 0 ? lane - 32 : lane, DA_WAVE);
-        if (g >= 2) { is = ip * bs_ + is; ip = ip * bp; }
-      }
+      lru_fold_lanes(lane, g, ip, is);
       float ep = __shfl(ip, lane - 16 >= 0 ? lane - 16 : lane, DA_WAVE), es = __shfl(is, lane - 16 >= 0 ? lane - 16 : lane, DA_WAVE);
       if (g == 0) { ep = 1.f; es = 0.f; }
       const float in_s = ep * run_s + es;                           // the state in front of this lane's first token
@@ -355,8 +397,13 @@ rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int 
       run_p = run_p * lp;
     }
     if (g == 0 && n0 + fr < in.bs) {
-      if (MODE == LRU_PAIRS) { pair[0] = run_p; pair[in.C] = run_s; }
-      if (MODE == LRU_WHOLE && in.write && slot >= 0) in.state[(size_t)slot * in.state_ld + c] = run_s;
+      if (MODE == LRU_PAIRS) {
+        float* pair = ends + (((size_t)blockIdx.z * max_chunks + chunk) * 2) * in.C + c;
+        pair[0] = run_p;
+        pair[in.C] = run_s;
+      } else if (t0 + LRU_TOK >= len && in.write && slot >= 0) {
+        row[c] = run_s;
+      }
     }
   }
   if (MODE != LRU_PAIRS) {
@@ -364,45 +411,6 @@ rglru_chunk_kernel(LruIn in, int seq0, int parts, float* __restrict__ ends, int 
     for (int e = t; e < nt * 8; e += 4 * DA_WAVE) {
       const int tok = e / 8, cc = part * 64 + (e % 8) * 8;
       if (cc < in.bs) *(uint4*)(in.out + (size_t)(first + t0 + tok) * in.out_ld + c0 + cc) = *(const uint4*)&ys[tok][(e % 8) * 8];
-    }
-  }
-}
-
-// The chunks' starting states, one after the other, a channel of a portion a thread: the place of a chunk's own state
-// takes its starting state, the state after the last chunk goes to the slot.  The filter's kept inputs move on here too;
-// the old ones are kept in `tails` for the chunks' second pass.
-__global__ void rglru_carry_kernel(LruIn in, int seq0, int S, float* __restrict__ ends, int max_chunks, float* __restrict__ tails) {
-  const long e = (long)blockIdx.x * blockDim.x + threadIdx.x;
-  if (e >= (long)S * in.C) return;
-  const int j = (int)(e / in.C), c = (int)(e % in.C), s = seq0 + j;
-  const int first = in.q_start[s], len = in.q_start[s + 1] - first, slot = in.slots[s];
-  const int n_chunks = (len + LRU_TOK - 1) / LRU_TOK;
-  float* row = in.state + (size_t)(slot >= 0 ? slot : 0) * in.state_ld;
-  float st = slot >= 0 ? row[c] : 0.f;
-  float* base = ends + (size_t)j * max_chunks * 2 * in.C + c;
-  for (int k0 = 0; k0 < n_chunks; k0 += 8) {            // eight chunks' numbers asked for at once, then walked in order
-    float p[8], own[8];
-#pragma unroll
-    for (int q = 0; q < 8; ++q) {
-      const int k = k0 + q < n_chunks ? k0 + q : n_chunks - 1;
-      p[q] = base[(size_t)k * 2 * in.C];
-      own[q] = base[(size_t)k * 2 * in.C + in.C];
-    }
-#pragma unroll
-    for (int q = 0; q < 8; ++q)
-      if (k0 + q < n_chunks) {
-        base[(size_t)(k0 + q) * 2 * in.C + in.C] = st;
-        st = p[q] * st + own[q];
-      }
-  }
-  for (int k = 0; k < in.K - 1; ++k)
-    tails[((size_t)j * (in.K - 1) + k) * in.C + c] = slot >= 0 ? row[(size_t)(k + 1) * in.C + c] : 0.f;
-  if (in.write && slot >= 0) {
-    row[c] = st;
-    for (int k = 0; k < in.K - 1; ++k) {
-      const int r = len - (in.K - 1) + k;
-      row[(size_t)(k + 1) * in.C + c] = r >= 0 ? bf16_to_f32(in.yx[(size_t)(first + r) * in.ld + in.C + c])
-                                               : tails[((size_t)j * (in.K - 1) + in.K - 1 + r) * in.C + c];
     }
   }
 }
@@ -450,7 +458,7 @@ extern "C" int da_rglru_decode(const void* yx, int ld, const float* conv_w, cons
 extern "C" int da_rglru_chunk_tokens() { return LRU_TOK; }
 
 // Sequences seq0 .. seq0 + S - 1 of the step, the longest of which brings max_len tokens.  scratch (when max_len is more
-// than a chunk): S * (chunks * 2 + K - 1) * C floats.
+// than a chunk, or a block has more than 64 channels): S * (chunks * 2 + K) * C floats.
 extern "C" int da_rglru_portion(const void* yx, int ld, const float* conv_w, const float* conv_b, const void* gate_w,
                                 const float* gate_b, const float* rate, int act, float* state, long state_ld,
                                 const int* state_slots, const int* q_start, void* out, int out_ld, int seq0, int S, int C, int bs,
@@ -471,14 +479,13 @@ extern "C" int da_rglru_portion(const void* yx, int ld, const float* conv_w, con
     DA_CHECK_LAUNCH("rglru_portion");
     return 0;
   }
-  const long need = (long)S * (2L * chunks + K - 1) * C;
+  const long need = (long)S * (2L * chunks + K) * C;
   DA_REQUIRE(scratch && scratch_floats >= need, "rglru_portion: the scratch holds %ld numbers, %ld are needed", scratch_floats, need);
-  float* tails = scratch + (long)S * chunks * 2 * C;
+  float* old = scratch + (long)S * chunks * 2 * C;
 #define LRU_GO(KS, KT)                                                                                                          \
   do {                                                                                                                          \
-    hipLaunchKernelGGL((rglru_chunk_kernel<KS, KT, LRU_PAIRS>), grid, block, 0, st, in, seq0, parts, scratch, chunks, nullptr); \
-    hipLaunchKernelGGL(rglru_carry_kernel, dim3(da_ceil_div((long)S * C, 64)), dim3(64), 0, st, in, seq0, S, scratch, chunks, tails); \
-    hipLaunchKernelGGL((rglru_chunk_kernel<KS, KT, LRU_AGAIN>), grid, block, 0, st, in, seq0, parts, scratch, chunks, tails);   \
+    hipLaunchKernelGGL((rglru_chunk_kernel<KS, KT, LRU_PAIRS>), grid, block, 0, st, in, seq0, parts, scratch, chunks, old);     \
+    hipLaunchKernelGGL((rglru_chunk_kernel<KS, KT, LRU_AGAIN>), grid, block, 0, st, in, seq0, parts, scratch, chunks, old);     \
   } while (0)
   LRU_PICK(LRU_GO);
 #undef LRU_GO

@@ -1730,7 +1730,7 @@ def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tenso
     """The recurrence of a step in bfloat16 serving, from the rows ``yx`` [N, y: C | x: C] to out = S * act(y): the filter
     of x (``conv_w`` float32 [taps, C], the last row meets the token itself; ``conv_b`` float32 [C]), the blocks' two square
     matrices (``gate_w`` [blocks, 2 b, b], ``gate_b`` float32 [blocks, 2 b]: r's rows, then i's), and ``rglru_walk``'s
-    recurrence.  One-token sequences and portions go to a launch (or, for portions longer than a chunk, three) each.
+    recurrence.  One-token sequences and portions go to a launch (or, for portions longer than a chunk, two) each.
     ``state`` [slots, taps * C]: S, then the filter's last inputs; both move on with ``write``."""
     _dev(yx, conv_w, conv_b, gate_w, gate_b, rate, state, out)
     _rows_2d(yx, "yx"); _rows_2d(out, "out")
@@ -1758,7 +1758,7 @@ def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tenso
         chunks = -(-longest // int(_lib().da_rglru_chunk_tokens()))
         scratch = None
         if chunks > 1 or bs > 64:
-            scratch = ctx.buf("rglru_scratch", (S - nd) * (2 * chunks + K - 1), C, torch.float32)
+            scratch = ctx.buf("rglru_scratch", (S - nd) * (2 * chunks + K), C, torch.float32)
         with _timed("rglru_portion", (N - nd) * C * 3 * 2 + (S - nd) * C * 2 * K * 4 + weights, (N - nd) * C * (4 * bs + 2 * K + 20), "bf16"):
             _check(_lib().da_rglru_portion(*args(), nd, S - nd, C, bs, K, int(bool(write)), longest, _ptr(scratch),
                                            0 if scratch is None else scratch.numel(), _stream()))
