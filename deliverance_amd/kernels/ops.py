@@ -7,6 +7,7 @@ back to a library or to the CPU: a missing kernel library is an error.
 from __future__ import annotations
 
 import ctypes
+from dataclasses import dataclass
 from typing import Optional
 
 import torch
@@ -149,6 +150,11 @@ _ARGTYPES = {
     "da_selective_scan": [_VP, _I, _I, _VP, _I, _VP, _I, _I, _I, _VP, _I, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP,
                           _VP, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_moe_combine": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _I, _VP, _I, _I, _VP, _I, _VP, _I, _VP],
+    "da_moe_choose_route_takes": [_I, _I, _I, _I, _I],
+    "da_moe_choose_route": [_VP, _I, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
+    "da_moe_combine_norm_takes": [_I],
+    "da_moe_combine_norm": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _VP, _I, _VP, _I, _VP, _I, _VP, _VP, _VP, _I, _VP, _I, _F, _F,
+                            _I, _VP, _I, _VP],
     "da_moe_choose": [_VP, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_add_rows": [_VP, _VP, _VP, _I, _I, _VP],
     "da_rglru_walk": [_VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _VP],
@@ -538,6 +544,40 @@ def moe_combine(out: torch.Tensor, slot_of_pair: torch.Tensor, weights: Optional
                                      0 if h is None else h.stride(0), _ptr(shared), 0 if shared is None else shared.stride(0),
                                      _ptr(shared_logit), 0 if shared is None else shared_logit.stride(0), _stream()))
     return y
+
+
+def moe_combine_norm(out: torch.Tensor, slot_of_pair: torch.Tensor, weights: Optional[torch.Tensor], uniform: float, top: int,
+                     y: torch.Tensor, accumulate: bool, h: Optional[torch.Tensor], shared: Optional[torch.Tensor],
+                     shared_logit: Optional[torch.Tensor], add: Optional[torch.Tensor], vec: Optional[torch.Tensor],
+                     norm, h_next: torch.Tensor) -> torch.Tensor:
+    """``moe_combine`` into the stream y, then (optional) y += add + vec, then h_next = the norm of y's rows.  ``norm``:
+    (centre, gain, bias or None, gain offset, eps), see csrc/moe.hip."""
+    centre, gain, bias, offset, eps = norm
+    _dev(out, slot_of_pair, weights, y, h, shared, shared_logit, add, vec, gain, bias, h_next)
+    _rows_2d(out, "out")
+    N, width = y.shape
+    _need(y.dtype == out.dtype == torch.float32 and y.is_contiguous() and y.dim() == 2 and out.shape[1] == width
+          and slot_of_pair.dtype == torch.int32 and slot_of_pair.numel() >= N * top, "moe_combine_norm: float32 [N, width], a slot a pair")
+    _need(weights is None or (weights.dtype == torch.float32 and weights.is_contiguous() and weights.numel() >= N * top),
+          "moe_combine_norm: a weight a pair")
+    _need(h is None or (h.dim() == 2 and h.stride(1) == 1 and h.dtype == h_next.dtype and h.shape[0] >= N and h.shape[1] == width),
+          "moe_combine_norm: the input must be [N, width] of h_next's dtype")
+    _need((shared is None) == (shared_logit is None) and (shared is None or (
+        shared.dtype == shared_logit.dtype == torch.float32 and shared.dim() == 2 and shared.stride(1) == 1 and shared.shape[0] >= N
+        and shared.shape[1] == width and shared_logit.dim() == 2 and shared_logit.shape[0] >= N)), "moe_combine_norm: the shared result")
+    for t_, n_, nm in ((add, N * width, "add"), (vec, width, "vec")):
+        _need(t_ is None or (t_.dtype == torch.float32 and t_.is_contiguous() and t_.numel() >= n_), f"moe_combine_norm: {nm} must be contiguous float32")
+    _need(gain.is_contiguous() and gain.numel() == width and (bias is None or (bias.is_contiguous() and bias.numel() == width)),
+          "moe_combine_norm: the norm's parameters differ from the width")
+    _need(h_next.is_contiguous() and tuple(h_next.shape) == (N, width), "moe_combine_norm: h_next must be contiguous [N, width]")
+    nb = (top + 2) * N * width * 4 + _nbytes(shared, add, h_next)
+    with _timed("moe_combine_norm", nb, (top + 8) * N * width, "fp32"):
+        _check(_lib().da_moe_combine_norm(
+            _ptr(out), out.stride(0), _ptr(slot_of_pair), _ptr(weights), float(uniform), top, _ptr(y), N, width, int(accumulate),
+            _ptr(h), 0 if h is None else h.stride(0), _ptr(shared), 0 if shared is None else shared.stride(0), _ptr(shared_logit),
+            0 if shared is None else shared_logit.stride(0), _ptr(add), _ptr(vec), _ptr(gain), _dt(gain), _ptr(bias),
+            0 if bias is None else _dt(bias), float(offset), float(eps), int(bool(centre)), _ptr(h_next), _dt(h_next), _stream()))
+    return h_next
 
 
 # ------------------------------------------------------------------------------- products
@@ -1268,6 +1308,31 @@ def moe_choose(z: torch.Tensor, outputs: int, correction: torch.Tensor, top: int
                                     _ptr(weights), _stream()))
 
 
+def moe_choose_route(choice: "ExpertChoice", top: int, extra: int, n_experts: int, tile: int, ids: torch.Tensor, weights: torch.Tensor,
+                     slot_of_pair: torch.Tensor, row_of_slot: torch.Tensor, tile_expert: torch.Tensor, n_tokens: int) -> None:
+    """``moe_choose`` and ``moe_route`` of a small step in one launch.  ids and weights are [N, top + extra]: the choice (ids
+    from ``n_experts`` on are moved up by ``extra``), then the ``extra`` experts n_experts .. that every token uses with the
+    weight logistic(z[n, outputs])."""
+    z, E = choice.z, choice.outputs
+    _dev(z, choice.correction, ids, weights, slot_of_pair, row_of_slot, tile_expert)
+    _rows_2d(z, "z")
+    N, each = n_tokens, top + extra
+    tiles, rows = moe_slot_space(N, each, n_experts + extra, tile)
+    _need(z.dtype == torch.float32 and z.shape[0] >= N and z.shape[1] >= E + (1 if extra else 0), "moe_choose_route: router logits must be float32 [N, >= outputs]")
+    _need(choice.correction.dtype == torch.float32 and choice.correction.is_contiguous() and choice.correction.numel() == E,
+          "moe_choose_route: the correction must be float32 with one entry an output")
+    _need(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= N * each and weights.dtype == torch.float32
+          and weights.is_contiguous() and weights.numel() >= N * each, "moe_choose_route: ids int32 and weights float32, [N, top + extra]")
+    for t_ in (slot_of_pair, row_of_slot, tile_expert):
+        _need(t_.dtype == torch.int32 and t_.is_contiguous(), "moe_choose_route: int32 contiguous operands")
+    _need(slot_of_pair.numel() >= N * each and row_of_slot.numel() >= rows and tile_expert.numel() >= tiles,
+          "moe_choose_route: the outputs are smaller than the slot space")
+    with _timed("moe_choose_route", N * E * 4 + N * each * 12 + 4 * (rows + tiles), N * E * (top + 6), "fp32"):
+        _check(_lib().da_moe_choose_route(_ptr(z), z.stride(0), _ptr(choice.correction), N, E, top, int(choice.groups),
+                                          int(choice.groups_kept), extra, n_experts, tile, _ptr(ids), _ptr(weights), _ptr(slot_of_pair),
+                                          _ptr(row_of_slot), _ptr(tile_expert), rows, tiles, _stream()))
+
+
 def _moe_mfma_ok(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor) -> bool:
     return (_MODE == "tuned" and h.dtype == torch.bfloat16 and gate_up.dtype == torch.bfloat16 and h.shape[1] % 8 == 0
             and h.stride(0) % 8 == 0 and down.shape[2] % 8 == 0 and h.data_ptr() % 16 == 0
@@ -1288,36 +1353,70 @@ def moe_top_logistic(z: torch.Tensor, top: int, renorm: bool, ids: torch.Tensor,
         _check(_lib().da_moe_top_logistic(_ptr(z), z.stride(0), N, E, top, int(renorm), _ptr(ids), _ptr(weights), _stream()))
 
 
+@dataclass(frozen=True)
+class ExpertChoice:
+    """A choice still to be made: what ``moe_choose`` takes (``z`` may hold a shared gate behind the outputs)."""
+    z: torch.Tensor
+    outputs: int
+    correction: torch.Tensor
+    groups: int
+    groups_kept: int
+
+
+SHARED_AS_EXPERTS_MAX_ROWS = 64      # steps in which a shared feed-forward rides along as further experts
+
+
+def shared_rides_along(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, choice: ExpertChoice, n_experts: int, top: int,
+                       extra: int) -> bool:
+    """Whether a shared feed-forward of this step runs as ``extra`` further experts of the grouped products (``gate_up`` and
+    ``down`` are the stacks with them): few rows, so that weights are streamed once either way and three launches fall away."""
+    N = h.shape[0]
+    return (extra > 0 and N <= SHARED_AS_EXPERTS_MAX_ROWS and N * (top + extra) < 64 * (n_experts + extra) and _moe_mfma_ok(h, gate_up, down)
+            and bool(_lib().da_moe_choose_route_takes(N, choice.outputs, top, extra, n_experts)))
+
+
 def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up: torch.Tensor, down: torch.Tensor,
                     n_experts: int, top: int, weight: float, act: str, x: torch.Tensor, accumulate: bool,
                     ids: Optional[torch.Tensor] = None, pair_weights: Optional[torch.Tensor] = None,
                     gated: bool = True, weight_input: bool = False, limit: float = 0.0, identity: bool = False,
-                    shared_out: Optional[torch.Tensor] = None, shared_logit: Optional[torch.Tensor] = None) -> torch.Tensor:
+                    shared_out: Optional[torch.Tensor] = None, shared_logit: Optional[torch.Tensor] = None,
+                    choice: Optional[ExpertChoice] = None, extra: int = 0, ahead=None) -> Optional[torch.Tensor]:
     """x (+)= sum_k weight_k * expert_k(h) (or, with ``weight_input``, sum_k expert_k(weight_k * h)): route, two
     grouped products, combine.  The experts of a row come from ``table[token, k]`` or from ``ids[n, k]``; the
-    weights are ``pair_weights[n, k]`` or the one ``weight``.  ``gated``: the first matrix of an expert is gate | up
+    weights are ``pair_weights[n, k]`` or the one weight ``weight``.  ``gated``: the first matrix of an expert is gate | up
     ([2 inner, width]) and its middle is act(gate h) * (up h); else it is [inner, width] and the middle is act(up h).
-    ``identity``: ids from ``n_experts`` on name experts whose output is h itself.  ``shared_out`` with ``shared_logit``: see
-    ``moe_combine``.
+    ``choice``: ids and pair_weights are still to be chosen and are filled here (small steps: together with the pairs'
+    layout).  ``identity``: ids behind the experts' name experts whose output is h itself.  ``extra``: the stacks hold so many
+    experts more, which every token uses with the logistic weight behind the choice's outputs (``shared_rides_along``; ids
+    and pair_weights are then [N, top + extra]).  ``shared_out`` with ``shared_logit``: see ``moe_combine``.  ``ahead``: what
+    happens to the stream x next (``parts.base.Ahead``); returns the next block's normed input then (None: it is still to be
+    made, and nothing of ``ahead`` has been done).
     bfloat16 steps run the grouped products on the matrix cores; 32-bit and the reference mode use the plain ones."""
     N, width = h.shape
     inner = down.shape[2]
     first_rows = (2 if gated else 1) * inner
+    n_experts, each, routed, chosen = n_experts + extra, top + extra, n_experts, top
     mfma = _moe_mfma_ok(h, gate_up, down)
     # Many rows an expert (prompt portions): the rows are gathered expert by expert and go through the block
     # tiles of the dense products, a matrix per group of 128 rows.  Few (decoding): tiles of 32 rows that
     # stream each expert's weights once.  The choice reads the step's shape only.
-    block = mfma and N * top >= 64 * n_experts and inner % 8 == 0
+    block = mfma and N * each >= 64 * n_experts and inner % 8 == 0
     tile = MOE_TILE_ROWS_BLOCK if block else (MOE_TILE_ROWS_MFMA if mfma else MOE_TILE_ROWS)
+    top = each
     tiles, rows = moe_slot_space(N, top, n_experts, tile)
     ints = ctx.buf("moe_route", N * top + rows + tiles, 1, torch.int32).view(-1)
     slot_of_pair, row_of_slot, tile_expert = ints[:N * top], ints[N * top:N * top + rows], ints[N * top + rows:]
     _need(not weight_input or pair_weights is not None, "experts: weights on the input need a weight a pair")
     # a pair's weight where its slot is: the first product scales its rows with it
     slot_scale = ctx.buf("moe_slot_scale", rows, 1, torch.float32).view(-1) if weight_input else None
-    if ids is None:
+    if choice is not None and not weight_input and bool(_lib().da_moe_choose_route_takes(N, choice.outputs, chosen, extra, routed)):
+        moe_choose_route(choice, chosen, extra, routed, tile, ids, pair_weights, slot_of_pair, row_of_slot, tile_expert, N)
+    elif ids is None:
         moe_route(ctx.tokens, table, None, N, top, n_experts, tile, slot_of_pair, row_of_slot, tile_expert)
     else:
+        if choice is not None:
+            _need(extra == 0, "experts: a shared feed-forward rides along in small steps only")
+            moe_choose(choice.z, choice.outputs, choice.correction, top, choice.groups, choice.groups_kept, ids, pair_weights)
         moe_route(None, None, ids, N, top, n_experts, tile, slot_of_pair, row_of_slot, tile_expert,
                   pair_weights if weight_input else None, slot_scale)
     mid = ctx.buf("moe_mid", rows, inner, h.dtype)
@@ -1376,11 +1475,17 @@ def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up
                                             _ptr(slot_scale), _ptr(mid), mid.stride(0), tiles, width, inner, ACTIVATIONS[act],
                                             _stream()))
         moe_down_ref(mid, row_of_slot, tile_expert, down, pair_out, tiles)
+    _need(not (weight_input and identity), "experts: an expert that hands its input on takes its weight on the output")
     if weight_input:               # the weights already sit in the rows
-        _need(not identity, "experts: an expert that hands its input on takes its weight on the output")
-        return moe_combine(pair_out, slot_of_pair, None, 1.0, top, x, accumulate, None, shared_out, shared_logit)
-    return moe_combine(pair_out, slot_of_pair, pair_weights, weight, top, x, accumulate, h if identity else None, shared_out,
-                       shared_logit)
+        pair_weights, weight = None, 1.0
+    norm = None if ahead is None or _MODE != "tuned" else ahead.params()
+    if norm is not None and x.is_contiguous() and bool(_lib().da_moe_combine_norm_takes(width)):
+        h_next = ahead.rows(ctx, h)
+        moe_combine_norm(pair_out, slot_of_pair, pair_weights, weight, top, x, accumulate, h if identity else None, shared_out,
+                         shared_logit, ahead.add, ahead.vec, norm, h_next)
+        return h_next
+    moe_combine(pair_out, slot_of_pair, pair_weights, weight, top, x, accumulate, h if identity else None, shared_out, shared_logit)
+    return None
 
 
 # ------------------------------------------------------------------------------- rotation, latent attention

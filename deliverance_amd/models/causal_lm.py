@@ -16,14 +16,9 @@ import torch
 from ..config.specs import ModelConfig
 from ..kernels import ops
 from ..parts.norms import STREAM_ITSELF
-from ..parts import Block, StepContext, build_norm, build_position, to_matrix, to_vector
+from ..parts import Ahead, Block, StepContext, build_norm, build_position, to_matrix, to_vector
 from ..registry import Architecture, ModelSupport, read_config_json
 from ..weights.loader import load_declared
-
-
-def _changes_stream(call) -> bool:
-    """Whether something happens to the stream right before this run-order entry."""
-    return bool(getattr(call, "mix_input", False) or getattr(call, "add_input", False) or getattr(call, "add_step", None) is not None)
 
 
 class CausalLM:
@@ -53,13 +48,13 @@ class CausalLM:
         elif any(getattr(c, "mix_input", False) for c in config.schedule):
             raise ValueError("the run order mixes the stream with the embedding output, but the model has no matrix for it")
         # vectors [n, width] of which run-order entries add one to the stream (32-bit)
-        self.step_vectors, self.adds_input = None, any(getattr(c, "add_input", False) for c in config.schedule)
+        self.step_vectors, self.adds_input = None, any(c.add_input for c in config.schedule)
         n_steps = int(getattr(config, "step_vectors", 0))
         if n_steps:
             self.step_vectors = params["step_vectors"]["weight"].to(device=device, dtype=torch.float32).contiguous()
             if tuple(self.step_vectors.shape) != (n_steps, config.width):
                 raise ValueError(f"the step vectors are {list(self.step_vectors.shape)}, expected {[n_steps, config.width]}")
-        if any(c.add_step is not None and not (0 <= c.add_step < n_steps) for c in config.schedule if hasattr(c, "add_step")):
+        if any(c.add_step is not None and not (0 <= c.add_step < n_steps) for c in config.schedule):
             raise ValueError(f"the run order names a step vector that is not among the model's {n_steps}")
         head = params["head"]["weight"]
         if head is emb["tokens"] and self.token_table.dtype == dtype:
@@ -90,6 +85,9 @@ class CausalLM:
         if self.input_mix is not None or self.step_vectors is not None or self.adds_input or self.config.logit_softcap > 0.0:
             names.append("elementwise")
         return sorted(set(names))
+
+    def _step_vector(self, call) -> Optional[torch.Tensor]:
+        return None if call.add_step is None else self.step_vectors[call.add_step]
 
     # ---- what the cache must provide -----------------------------------------------------
     def cache_needs(self) -> Dict[int, object]:
@@ -146,14 +144,20 @@ class CausalLM:
             first = ops.copy_rows(x, ctx.buf("embedded", N, self.config.width, torch.float32))
         h = None                                        # a block's input that the block before has made
         for call, after in zip(self.config.schedule, (*self.config.schedule[1:], None)):
-            if getattr(call, "mix_input", False):       # x <- W [x; embedding output]
+            if call.mix_input:                          # x <- W [x; embedding output]
                 ops.concat_rows(x, both, 0)
                 ops.linear(both, self.input_mix, None, x)
-            again, vec = getattr(call, "add_input", False), getattr(call, "add_step", None)
-            if again or vec is not None:                # x <- x + embedding output + step vector
-                ops.add_rows(x, first if again else None, None if vec is None else self.step_vectors[vec])
-            ahead = after is not None and not _changes_stream(after) and self.blocks[after.layer].takes_stream_ahead()
-            h = self.blocks[call.layer].forward(ctx, x, call, h_ready=h, next_pre=STREAM_ITSELF if ahead else None)
+            if h is None and (call.add_input or call.add_step is not None):       # x <- x + embedding output + step vector
+                ops.add_rows(x, first if call.add_input else None, self._step_vector(call))
+            block, ahead = self.blocks[call.layer], None
+            if after is not None and not after.mix_input and not debug:
+                nxt = self.blocks[after.layer]
+                if block.hands_ahead() and nxt.pre_mixer_norm is not None:
+                    # the block's last kernel also does what is next: the additions, and the norm in front of the next block
+                    ahead = Ahead(nxt.pre_mixer_norm, first if after.add_input else None, self._step_vector(after))
+                elif nxt.takes_stream_ahead() and not after.add_input and after.add_step is None:
+                    ahead = STREAM_ITSELF
+            h = block.forward(ctx, x, call, h_ready=h, next_pre=ahead)
             if debug:
                 ctx.emit(call.layer, "layer_output", x)
         logits = ctx.buf("logits", n_want, self.config.vocab_size, torch.float32)

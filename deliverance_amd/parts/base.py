@@ -19,7 +19,9 @@ Interfaces (shapes: N tokens of the step, E model width):
   ``ctx.positions``, ``ctx.q_start``, ``ctx.state_slots``); ``ops.state_gather`` hands every row
   its sequence's state and ``ops.state_scatter`` keeps the state that each portion's last row
   leaves.  One that reads these only (never the ``*_host`` lists) may set ``graph_safe``.
-* ``FeedForward.forward(ctx, h, x) -> None``: reads h, adds its result to x in place.
+* ``FeedForward.forward(ctx, h, x) -> None``: reads h, adds its result to x in place.  One that declares
+  ``takes_ahead`` also takes ``ahead`` (an ``Ahead`` or None) when x is the stream itself, and returns the next block's
+  input when it has made it.
 * ``PositionEncoding``: ``embed_table()`` returns a [P, E] table added to token embeddings
   (or None); ``apply_qk(ctx, qkv, ...)`` may rotate queries and keys in place (default: none).
 
@@ -155,6 +157,29 @@ class Arena:
         return t[:rows]
 
 
+@dataclass(frozen=True)
+class Ahead:
+    """What happens to the stream behind a block, for a block whose last kernel can do it in passing: ``add`` [N, width] and
+    ``vec`` [width] (32-bit, or None) join the stream, and ``norm`` of its rows is the next block's input."""
+    norm: "Norm"
+    add: Optional[torch.Tensor] = None
+    vec: Optional[torch.Tensor] = None
+
+    def params(self):
+        """(centre, gain, bias or None, gain offset, eps), or None for a norm that must run as a kernel of its own."""
+        ln = self.norm.fusable_params()
+        if ln is not None:
+            return True, ln[0], ln[1], 0.0, ln[2]
+        rms = getattr(self.norm, "rms_params", lambda: None)()
+        return None if rms is None else (False, rms[0], None, rms[1], rms[2])
+
+    @staticmethod
+    def rows(ctx: "StepContext", h: torch.Tensor) -> torch.Tensor:
+        """A buffer for the next block's input that is not this block's own (``h``)."""
+        out = ctx.buf("norm_ahead_a", h.shape[0], h.shape[1], ctx.dtype)
+        return out if out.data_ptr() != h.data_ptr() else ctx.buf("norm_ahead_b", h.shape[0], h.shape[1], ctx.dtype)
+
+
 class Norm:
     # The kernel units (kernels/build.py) that the norm's steps call; a model's are compiled together before its first
     # step.  (A unit that is not named is compiled when it is first called.)
@@ -190,6 +215,7 @@ class Mixer:
 
 class FeedForward:
     graph_safe = False
+    takes_ahead = False
 
     def kernel_units(self, dtype: torch.dtype) -> Tuple[str, ...]:
         return ()

@@ -10,7 +10,7 @@ from __future__ import annotations
 import torch
 
 from ..kernels import ops
-from .base import StepContext, build_feed_forward, build_mixer, build_norm, to_vector
+from .base import Ahead, StepContext, build_feed_forward, build_mixer, build_norm, to_vector
 from .norms import STREAM_ITSELF
 
 
@@ -102,26 +102,31 @@ class Block:
         convert it in passing (``forward(next_pre=STREAM_ITSELF)`` there, ``h_ready`` here)."""
         return self.pre_mixer_norm is None
 
-    def _forward_parallel(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None):
+    def hands_ahead(self) -> bool:
+        """Whether the block's last kernel may do what follows it (an ``Ahead`` for ``forward(next_pre=)``)."""
+        return self.parallel and self.feed_forward.takes_ahead
+
+    def _forward_parallel(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None, ahead=None):
         """x += mixer(h) + ff(h), h = norm(x): the norm's output is a buffer of its own, so the mixer may add into the
-        stream before the feed-forward reads."""
+        stream before the feed-forward reads.  Returns the next block's input if ``ahead`` was done in passing."""
         h = h_ready if h_ready is not None else Block._normed(ctx, x, self.pre_mixer_norm)
         self.mixer.forward(ctx, h, x, call)
         if ctx.debug_hook is not None:
             ctx.emit(call.layer, "post_attention_residual", x)
-        self.feed_forward.forward(ctx, h, x)
+        h_next = self.feed_forward.forward(ctx, h, x, ahead=ahead) if ahead is not None else self.feed_forward.forward(ctx, h, x)
         if ctx.debug_hook is not None:
             chosen = getattr(self.feed_forward, "last_choice", None)
             if chosen is not None:
                 ctx.emit(call.layer, "expert_choice", chosen)
             ctx.emit(call.layer, "post_ff_residual", x)
+        return h_next
 
     def forward(self, ctx: StepContext, x: torch.Tensor, call, h_ready=None, next_pre=None):
         """Runs the block.  ``h_ready``: the mixer's input, when the block before has made it.  ``next_pre``: what the
-        block behind wants of the new stream (``STREAM_ITSELF`` or None); returns it when the block's last norm could make
+        block behind wants of the new stream (``STREAM_ITSELF``, an ``Ahead`` if ``hands_ahead``, or None); returns it when the block's last norm could make
         it in the same pass, else None."""
         if self.parallel:
-            return self._forward_parallel(ctx, x, call, h_ready)
+            return self._forward_parallel(ctx, x, call, h_ready, next_pre if isinstance(next_pre, Ahead) else None)
         if ctx.debug_hook is not None or self.post_block_norm is not None:
             next_pre = None
         fused = getattr(self.mixer, "forward_normed", None)

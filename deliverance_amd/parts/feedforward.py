@@ -90,10 +90,12 @@ class ExpertsFeedForward(FeedForward):
     products run over that layout, and the pairs' results are added up per token; a weight on the input scales
     the pair's row in the first product.  A shared expert, if any, runs as a dense feed-forward for every token; with a gate
     a token (``shared_token_gate``, one more row of the router's product) its result goes to a buffer of its own and joins
-    where the pairs are added up.
+    where the pairs are added up, or, in small steps and if its columns are a multiple of an expert's, it runs as so many
+    further experts that every token uses.
     Nothing is read back to the host, so a step can be recorded."""
     graph_safe = True
     can_store = True
+    takes_ahead = True
 
     def __init__(self, spec, params, dtype, device):
         self.width, self.inner, self.activation = spec.width, spec.inner, spec.activation
@@ -163,7 +165,21 @@ class ExpertsFeedForward(FeedForward):
                 raise ValueError(f"the router's bias has {self.router_bias.numel()} entries for {self.n_experts} experts")
         self.weight = 1.0 / self.top
         self.last_choice = None
-        self.shared = None
+        self.shared, self.extra = None, 0
+        shared_inner = int(getattr(spec, "shared_inner", 0))
+        if self.token_gate and self.gated and getattr(spec, "shared_gated", False) and shared_inner % self.inner == 0 \
+                and (spec.shared_activation or self.activation) == self.activation \
+                and float(getattr(spec, "shared_limit", 0.0) or 0.0) == self.limit and dtype == torch.bfloat16:
+            # A gated feed-forward of m times an expert's columns is the sum of m experts: in small steps they run among
+            # the others.  (Its weights are kept twice: dense for large steps, and behind the experts.)
+            self.extra = shared_inner // self.inner
+            gu, dn = params["shared_gate_up_weight"], params["shared_down_weight"]
+            pieces = [(torch.cat([gu[j:j + self.inner], gu[shared_inner + j:shared_inner + j + self.inner]], 0), dn[:, j:j + self.inner])
+                      for j in range(0, shared_inner, self.inner)]
+            stack = lambda own, more: torch.cat([own, torch.stack([to_matrix(m, dtype, device) for m in more])], 0).contiguous()
+            self.gate_up_all = stack(self.gate_up_weight, [p[0] for p in pieces])
+            self.down_all = stack(self.down_weight, [p[1] for p in pieces])
+            self.gate_up_weight, self.down_weight = self.gate_up_all[:self.n_experts], self.down_all[:self.n_experts]
         if getattr(spec, "shared_inner", 0) and getattr(spec, "shared_gated", False):
             from ..config.specs import GatedFeedForwardSpec
             self.shared = GatedFeedForward(
@@ -180,41 +196,46 @@ class ExpertsFeedForward(FeedForward):
     def kernel_units(self, dtype):
         return ("moe", "elementwise") + (() if self.shared is None else self.shared.kernel_units(dtype))
 
-    def forward(self, ctx: StepContext, h: torch.Tensor, x: torch.Tensor) -> None:
-        ids = weights = None
+    def forward(self, ctx: StepContext, h: torch.Tensor, x: torch.Tensor, ahead=None):
+        N, z, ids, weights, choice, shared_out, extra = h.shape[0], None, None, None, None, None, 0
+        gate_up, down = self.gate_up_weight, self.down_weight
         if self.router_weight is not None:
-            N = h.shape[0]
             z = ctx.buf("moe_logits", N, self.router_weight.shape[0], torch.float32)      # 32-bit sums of the products
             ops.linear(h, self.router_weight, None, z)
-            ids = ctx.buf("moe_ids", N, self.top, torch.int32)
-            weights = ctx.buf("moe_weights", N, self.top, torch.float32)
             if self.router == "softmax_all":
-                ops.moe_choose(z, self.outputs, self.correction, self.top, self.groups, self.groups_kept, ids, weights)
-            elif self.router == "softmax_top":
+                choice = ops.ExpertChoice(z, self.outputs, self.correction, self.groups, self.groups_kept)
+                if self.extra and ops.shared_rides_along(h, self.gate_up_all, self.down_all, choice, self.n_experts, self.top, self.extra):
+                    extra, gate_up, down = self.extra, self.gate_up_all, self.down_all
+            ids = ctx.buf("moe_ids", N, self.top + extra, torch.int32)
+            weights = ctx.buf("moe_weights", N, self.top + extra, torch.float32)
+            if self.router == "softmax_top":
                 ops.moe_top(z, self.router_bias, self.top, "softmax", False, ids, weights)
-            else:
+            elif self.router == "logistic_top":
                 ops.moe_top(z, self.router_bias, self.top, "logistic", self.renormalize, ids, weights)
-        self.last_choice = ids if ctx.debug_hook is not None else None      # handed to the layer debug hook
-        shared_out = None
-        if self.token_gate:
-            shared_out = ctx.buf("moe_shared_out", h.shape[0], self.width, torch.float32)
-            keep, ctx.part_accumulate = ctx.part_accumulate, False
-            try:
-                self.shared.forward(ctx, h, shared_out)
-            finally:
-                ctx.part_accumulate = keep
-        ops.experts_forward(ctx, h, self.table, self.gate_up_weight, self.down_weight, self.n_experts, self.top,
-                            self.weight, self.activation, x, accumulate=ctx.part_accumulate, ids=ids,
-                            pair_weights=weights, gated=self.gated, weight_input=self.weight_on == "input",
-                            limit=self.limit, identity=self.identity > 0, shared_out=shared_out,
-                            shared_logit=z[:, self.outputs:] if self.token_gate else None)
-        if self.shared is not None and not self.token_gate:
-            keep = ctx.part_accumulate
-            ctx.part_accumulate = True          # the shared expert joins the experts' sum, stored or added above
-            try:
-                self.shared.forward(ctx, h, x)
-            finally:
-                ctx.part_accumulate = keep
+        if self.token_gate and not extra:
+            shared_out = ctx.buf("moe_shared_out", N, self.width, torch.float32)
+            self._run_shared(ctx, h, shared_out, False)
+        plain_shared = self.shared is not None and not self.token_gate
+        h_next = ops.experts_forward(
+            ctx, h, self.table, gate_up, down, self.n_experts, self.top, self.weight, self.activation, x,
+            accumulate=ctx.part_accumulate, ids=ids, pair_weights=weights, gated=self.gated, weight_input=self.weight_on == "input",
+            limit=self.limit, identity=self.identity > 0, shared_out=shared_out,
+            shared_logit=None if shared_out is None else z[:, self.outputs:], choice=choice, extra=extra,
+            ahead=None if plain_shared else ahead)
+        self.last_choice = None
+        if ctx.debug_hook is not None and ids is not None:      # handed to the layer debug hook, as the router names them
+            of = ids[:, :self.top]
+            self.last_choice = torch.where(of >= self.n_experts + extra, of - extra, of) if extra else ids
+        if plain_shared:
+            self._run_shared(ctx, h, x, True)      # the shared expert joins the experts' sum, stored or added above
+        return h_next
+
+    def _run_shared(self, ctx: StepContext, h: torch.Tensor, into: torch.Tensor, accumulate: bool) -> None:
+        keep, ctx.part_accumulate = ctx.part_accumulate, accumulate
+        try:
+            self.shared.forward(ctx, h, into)
+        finally:
+            ctx.part_accumulate = keep
 
 
 register_feed_forward("gated", GatedFeedForward)

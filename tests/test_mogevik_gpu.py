@@ -481,6 +481,75 @@ def test_the_choice_of_experts(experts, top, groups):
         assert np.abs(host(w) - want_w).max() <= 2e-6
 
 
+@pytest.mark.parametrize("rows,experts,ident,top,groups,extra", [quick(5, 6, 2, 3, (4, 2), 2), (1, 1, 0, 1, None, 1), (17, 9, 3, 4, (3, 2), 0), (64, 8, 2, 2, (2, 1), 2),
+                                                                 (33, 100, 28, 6, (16, 5), 4), (100, 3, 5, 2, None, 3)])
+def test_the_choice_and_the_layout_in_one_launch(rows, experts, ident, top, groups, extra):
+    """The same ids and weights as the choice alone, ids of experts that hand their input on moved up, the further experts'
+    pairs behind them with a logistic weight; every pair of an expert with matrices in a slot of its expert's tiles."""
+    from deliverance_amd.kernels import ops
+    rng = np.random.default_rng(rows)
+    E, each, tile = experts + ident, top + extra, 32
+    z = dev(rng.normal(size=(rows, E + 1)) * 2, torch.float32)
+    corr = dev(rng.normal(size=E) * 0.3, torch.float32)
+    g = groups or (0, 0)
+    i1, w1 = torch.zeros(rows, top, dtype=torch.int32, device=DEV), torch.zeros(rows, top, dtype=torch.float32, device=DEV)
+    ops.moe_choose(z, E, corr, top, *g, i1, w1)
+    tiles, space = ops.moe_slot_space(rows, each, experts + extra, tile)
+    i2, w2 = torch.full((rows, each), -7, dtype=torch.int32, device=DEV), torch.zeros(rows, each, dtype=torch.float32, device=DEV)
+    slot, row_of, tile_of = (torch.full((n,), -9, dtype=torch.int32, device=DEV) for n in (rows * each, space, tiles))
+    ops.moe_choose_route(ops.ExpertChoice(z, E, corr, *g), top, extra, experts, tile, i2, w2, slot, row_of, tile_of, rows)
+    i1, i2, slot, row_of, tile_of = (t.cpu().numpy() for t in (i1, i2, slot, row_of, tile_of))
+    assert np.array_equal(i2[:, :top], np.where(i1 < experts, i1, i1 + extra)) and torch.equal(w2[:, :top].contiguous(), w1)
+    assert np.array_equal(i2[:, top:], np.tile(np.arange(experts, experts + extra), (rows, 1)))
+    if extra:
+        assert np.abs(host(w2)[:, top:] - P.logistic(host(z)[:, E:])).max() <= 1e-6
+    slot, used = slot.reshape(rows, each), set()
+    for n in range(rows):
+        for k in range(each):
+            if i2[n, k] >= experts + extra:
+                assert slot[n, k] == -1
+            else:
+                assert row_of[slot[n, k]] == n and tile_of[slot[n, k] // tile] == i2[n, k] and slot[n, k] not in used
+                used.add(slot[n, k])
+    assert all(row_of[i] == -1 for i in range(space) if i not in used)
+
+
+@pytest.mark.parametrize("dtype", ["float32", quick("bfloat16")])
+@pytest.mark.parametrize("rows,width,centre", [quick(5, 52, True), (3, 320, True), (700, 768, True), (2, 1600, True), (9, 4096, False), quick(4, 64, False)])
+def test_the_pairs_sum_the_streams_additions_and_the_next_norm_in_one_pass(rows, width, centre, dtype):
+    from deliverance_amd.kernels import ops
+    helpers.skip_in_simulation_if(rows > 100)
+    rng = np.random.default_rng(width)
+    top, slots = 3, 40
+    out, y0 = rng.normal(size=(slots, width)).astype(np.float32), rng.normal(size=(rows, width)).astype(np.float32)
+    slot = rng.integers(-1, slots, size=(rows, top))
+    w = rng.random(size=(rows, top)).astype(np.float32)
+    h, shared, gate = bf16(rng.normal(size=(rows, width))), rng.normal(size=(rows, width)).astype(np.float32), rng.normal(size=(rows, 5)).astype(np.float32)
+    add, vec = rng.normal(size=(rows, width)).astype(np.float32), rng.normal(size=width).astype(np.float32)
+    gain, bias = bf16(1 + 0.2 * rng.normal(size=width)), bf16(rng.normal(size=width))
+    f = lambda a: dev(a, torch.float32)
+    for full in (True, False):
+        y = f(y0)
+        nxt = torch.zeros(rows, width, dtype=DTYPES[dtype], device=DEV)
+        ops.moe_combine_norm(f(out), dev(slot), f(w) if full else None, 0.5, top, y, full, dev(h, DTYPES[dtype]) if full else None,
+                             f(shared) if full else None, f(gate)[:, 3:] if full else None, f(add) if full else None, f(vec) if full else None,
+                             (centre, dev(gain, torch.bfloat16), dev(bias, torch.bfloat16) if full else None, 0.25, 1e-3), nxt)
+        want = y0.astype(np.float64) if full else np.zeros((rows, width))
+        for n in range(rows):
+            for k in range(top):
+                wk = w[n, k] if full else 0.5
+                if slot[n, k] >= 0:
+                    want[n] += wk * out[slot[n, k]]
+                elif full:
+                    want[n] += wk * h[n]
+        if full:
+            want += P.logistic(gate[:, 3:4].astype(np.float64)) * shared + add + vec
+        assert np.abs(host(y) - want).max() <= 1e-5
+        d = want - (want.mean(1, keepdims=True) if centre else 0.0)
+        normed = d / np.sqrt((d * d).mean(1, keepdims=True) + 1e-3) * (0.25 + gain) + (bias if full else 0.0)
+        assert np.abs(host(nxt) - normed).max() <= (2e-5 if dtype == "float32" else 2.0 ** -8) * np.abs(normed).max()
+
+
 EXPERTS = [quick(9, moe(7, 3, 24, identity=2, groups=(3, 2), shared=48)), (150, moe(7, 3, 24, identity=2, groups=(3, 2), shared=48)),
            quick(20, moe(4, 2, 32, shared=40)), (600, moe(4, 2, 32, shared=40)), (6, moe(1, 1, 40)), (33, moe(2, 2, 16, identity=4, groups=(1, 1), shared=16)),
            (70, moe(3, 4, 20, identity=1, groups=(2, 2), shared=12)), (1, moe(12, 5, 8, identity=3, groups=(5, 3), shared=24)),
@@ -674,6 +743,18 @@ def test_mixed_batches_over_a_small_pool(mmodels, name, dtype):
             one = helpers.replay(alone, helpers.trace_whole(rid, ids))[rid]
             scale = float(np.sqrt((one.astype(np.float64) ** 2).mean()))
             assert np.abs(one.astype(np.float64) - got[rid]).max() <= 3e-5 * scale
+
+
+@pytest.mark.parametrize("name", ["D", quick("E"), "F"])
+def test_a_blocks_last_kernel_does_what_is_next(mmodels, name):
+    """With the layer debug hook every step of a block is a launch of its own; without it a block's last kernel also adds
+    what joins the stream before the next block and makes its norm.  The logits are the same but for rounding."""
+    m = mmodels[name]
+    ids = m.prompt(50, salt=70)
+    steps = helpers.trace_portions("r", ids, (30, 1, 1, 5, 1))
+    one = helpers.replay(helpers.trace_session(m.folder, "float32", 128, state_slots=1), steps)["r"]
+    two, _ = replay_routed(helpers.trace_session(m.folder, "float32", 128, state_slots=1), steps, m.cfg)
+    assert np.abs(one - two["r"]).max() <= 2e-5 * np.abs(one).max()
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
