@@ -22,34 +22,56 @@
 #define MOE_MAX_EXPERTS 1024
 
 struct MoeRouteLds {
-  int counts[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], cursor[MOE_MAX_EXPERTS];
+  int counts[MOE_MAX_EXPERTS], start[MOE_MAX_EXPERTS], cursor[MOE_MAX_EXPERTS], total;
 };
 
-// One workgroup lays the pairs out.  `expert_of(i)`: pair i's expert, or -1.
+// One workgroup lays the pairs out.  `expert_of(i)`: pair i's expert, or -1.  Every place of row_of_slot and tile_expert is
+// written once, so that no barrier has to wait for memory: a pair's slot by the pair, the places behind an expert's last
+// pair and the tiles by whoever finds their expert among the starts.
 template <class ExpertOf>
 __device__ __forceinline__ void moe_lay_out(MoeRouteLds& l, ExpertOf expert_of, int P, int top, int n_experts, int tile,
                                             int* slot_of_pair, int* row_of_slot, int* tile_expert, int P_cap, int T_cap,
                                             const float* pair_weights, float* slot_weight) {
-  const int t = threadIdx.x, nt = blockDim.x;
+  const int t = threadIdx.x, nt = blockDim.x, lane = t % DA_WAVE;
   for (int e = t; e < n_experts; e += nt) l.counts[e] = l.cursor[e] = 0;
-  for (int i = t; i < P_cap; i += nt) row_of_slot[i] = -1;
-  for (int i = t; i < T_cap; i += nt) tile_expert[i] = -1;
-  __syncthreads();
+  lds_barrier();
   for (int i = t; i < P; i += nt) {
     const int e = expert_of(i);
     if (e >= 0) atomicAdd(&l.counts[e], 1);
   }
-  __syncthreads();
-  if (t == 0) {
+  lds_barrier();
+  if (t < DA_WAVE) {                                   // the first wavefront: starts, 64 experts at a time
     int run = 0;
-    for (int e = 0; e < n_experts; ++e) {
-      l.start[e] = run;
-      const int tiles = (l.counts[e] + tile - 1) / tile;
-      for (int k = 0; k < tiles; ++k) tile_expert[run / tile + k] = e;
-      run += tiles * tile;
+    for (int e0 = 0; e0 < n_experts; e0 += DA_WAVE) {
+      const int e = e0 + lane;
+      const int own = e < n_experts ? (l.counts[e] + tile - 1) / tile * tile : 0;
+      int upto = own;                                  // this expert's slots and those of the ones before it
+#pragma unroll
+      for (int back = 1; back < DA_WAVE; back *= 2) {
+        const int v = __shfl(upto, lane >= back ? lane - back : lane, DA_WAVE);
+        if (lane >= back) upto += v;
+      }
+      if (e < n_experts) l.start[e] = run + upto - own;
+      run += __builtin_amdgcn_readlane(upto, DA_WAVE - 1);
     }
+    if (t == 0) l.total = run;
   }
-  __syncthreads();
+  lds_barrier();
+  auto owner = [&](int i) -> int {                     // the last expert that starts at or before slot i
+    int lo = 0, hi = n_experts - 1;
+    while (lo < hi) {
+      const int mid = (lo + hi + 1) / 2;
+      if (l.start[mid] <= i) lo = mid;
+      else hi = mid - 1;
+    }
+    return lo;
+  };
+  const int total = l.total;
+  for (int i = t; i < P_cap; i += nt) {
+    const int e = i < total ? owner(i) : 0;
+    if (i >= total || i - l.start[e] >= l.counts[e]) row_of_slot[i] = -1;
+  }
+  for (int i = t; i < T_cap; i += nt) tile_expert[i] = i * tile < total ? owner(i * tile) : -1;
   for (int i = t; i < P; i += nt) {
     const int e = expert_of(i);
     int slot = -1;
@@ -313,6 +335,7 @@ __device__ __forceinline__ float moe_choose_token(const float* __restrict__ row,
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
   };
+  const float corr0 = correction[lane < E ? lane : 0];       // (asked for ahead of the sums)
   float m = -INFINITY;
   for (int e = lane; e < E; e += DA_WAVE) m = fmaxf(m, row[e]);
   m = wave_max(m);
@@ -326,7 +349,7 @@ __device__ __forceinline__ float moe_choose_token(const float* __restrict__ row,
   for (int e = lane; e < E; e += DA_WAVE) {
     const float v = sc[e] / sum;
     sc[e] = v;
-    c[e] = v + correction[e];
+    c[e] = v + (e < DA_WAVE ? corr0 : correction[e]);
   }
   wave_fence();
   if (groups > 0) {
@@ -364,104 +387,200 @@ __device__ __forceinline__ float moe_choose_token(const float* __restrict__ row,
   return chosen;
 }
 
+// The same for at most 64 outputs: an output a lane, everything in registers.
+template <class Give>
+__device__ __forceinline__ float moe_choose_token64(const float* __restrict__ row, const float* __restrict__ correction, int E, int top,
+                                                    int groups, int keep, int lane, Give give) {
+  const bool in = lane < E;
+  const float corr = correction[in ? lane : 0];
+  const float z = in ? row[lane] : -INFINITY;
+  const float m = wave_max(z);                         // (every lane takes part in what goes across lanes)
+  const float ex = in ? expf(z - m) : 0.f;
+  const float s = ex / wave_sum(ex);
+  float c = in ? s + corr : -INFINITY;
+  if (groups > 0) {
+    const int size = E / groups, mine = (in ? lane : 0) / size;
+    float best = -INFINITY;                            // of this lane's run
+    for (int e = 0; e < size; ++e) best = fmaxf(best, __shfl(c, mine * size + e, DA_WAVE));
+    int ahead = 0;                                     // runs that come before it
+    for (int k = 0; k < groups; ++k) {
+      const float other = __shfl(best, k * size, DA_WAVE);
+      ahead += other > best || (other == best && k < mine);
+    }
+    if (ahead >= keep) c = -INFINITY;
+  }
+  float chosen = 0.f;
+  auto better = [](float a, int ai, float b, int bi) { return a > b || (a == b && ai < bi); };
+  for (int k = 0; k < top; ++k) {
+    float bv = c;
+    int be = in ? lane : E - 1;
+    wave_best(bv, be, better);
+    const float sb = __builtin_bit_cast(float, __builtin_amdgcn_readlane(__builtin_bit_cast(int, s), be));
+    chosen += sb;
+    if (lane == 0) give(k, be, sb);
+    if (lane == be) c = -INFINITY;                     // taken
+  }
+  return chosen;
+}
+
 // (EC: outputs that LDS has room for.)
 #define MC_WAVES 4
 template <int EC>
 __global__ void __launch_bounds__(MC_WAVES * DA_WAVE)
 moe_choose_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ correction, int N, int E, int top, int groups,
-                  int keep, int* __restrict__ ids, float* __restrict__ weights) {
-  __shared__ float mc_lds[MC_WAVES][3][EC];
+                  int keep, int extra, int n_experts, int* __restrict__ ids, float* __restrict__ weights) {
+  __shared__ float mc_lds[EC > 64 ? MC_WAVES : 1][3][EC > 64 ? EC : 1];
   const int lane = threadIdx.x % DA_WAVE, wave = threadIdx.x / DA_WAVE;
   const int n = blockIdx.x * MC_WAVES + wave;
   if (n >= N) return;                                  // (wavefronts do not wait for one another)
-  int* const id = ids + (size_t)n * top;
-  float* const w = weights + (size_t)n * top;
-  const float sum = moe_choose_token(z + (size_t)n * ldz, correction, E, top, groups, keep, mc_lds[wave][0], mc_lds[wave][1], mc_lds[wave][2], lane,
-                                     [&](int k, int e, float s) { id[k] = e; w[k] = s; });
+  const float* row = z + (size_t)n * ldz;
+  const float gate = extra ? row[E] : 0.f;
+  int* const id = ids + (size_t)n * (top + extra);
+  float* const w = weights + (size_t)n * (top + extra);
+  float sum;
+  auto give = [&](int k, int e, float s) {
+    id[k] = e < n_experts ? e : e + extra;
+    w[k] = s;
+  };
+  if (EC <= 64) sum = moe_choose_token64(row, correction, E, top, groups, keep, lane, give);
+  else sum = moe_choose_token(row, correction, E, top, groups, keep, mc_lds[EC > 64 ? wave : 0][0], mc_lds[EC > 64 ? wave : 0][1],
+                              mc_lds[EC > 64 ? wave : 0][2], lane, give);
   if (lane == 0)
     for (int k = 0; k < top; ++k) w[k] /= sum + 1e-20f;
+  for (int k = lane; k < extra; k += DA_WAVE) {
+    id[top + k] = n_experts + k;
+    w[top + k] = 1.f / (1.f + expf(-gate));
+  }
 }
 
-// Small steps: the choice and the pairs' layout in one launch.  A shared feed-forward may ride along as `extra` experts
-// behind the others, which every token uses with the weight logistic(z[n, E]): pairs top .. top + extra - 1 of a token.
-// Outputs from n_experts on (experts that hand their input on) become ids from n_experts + extra on, which have no slot.
+// ids[n] and weights[n]: `top` choices (outputs from n_experts on, experts that hand their input on, become ids from n_experts
+// + extra on), then the `extra` further experts n_experts .., which every token uses with the weight logistic(z[n, E]).
+extern "C" int da_moe_choose(const float* z, int ldz, const float* correction, int N, int E, int top, int groups, int keep,
+                             int extra, int n_experts, int* ids, float* weights, void* stream) {
+  DA_REQUIRE(N >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && extra >= 0 && n_experts > 0 && n_experts <= E &&
+             ldz >= E + (extra > 0) && correction, "moe_choose: bad sizes");
+  DA_REQUIRE(groups == 0 || (groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= E / groups * keep),
+             "moe_choose: top %d of %d outputs in %d groups of which %d are kept", top, E, groups, keep);
+  if (N == 0) return 0;
+#define MC_GO(EC)                                                                                                            \
+  hipLaunchKernelGGL((moe_choose_kernel<EC>), dim3(da_ceil_div(N, MC_WAVES)), dim3(MC_WAVES * DA_WAVE), 0, (hipStream_t)stream, \
+                     z, ldz, correction, N, E, top, groups, keep, extra, n_experts, ids, weights)
+  if (E <= 64) MC_GO(64);
+  else if (E <= 256) MC_GO(256);
+  else MC_GO(MOE_MAX_EXPERTS);
+#undef MC_GO
+  DA_CHECK_LAUNCH("moe_choose");
+  return 0;
+}
+
+// The products of all tokens' inputs with one row of a router, by one wavefront: a lane holds every 64th run of 8 entries,
+// the row and MR_TOKENS inputs are asked for at once, and a sum is added up across the lanes in a fixed order.
+#define MR_TOKENS 8
+template <class Give>
+__device__ __forceinline__ void moe_router_row(const bf16_t* __restrict__ h, int ldh, int N, const bf16_t* __restrict__ row, int K,
+                                               int lane, Give give) {
+  for (int n0 = 0; n0 < N; n0 += MR_TOKENS) {
+    float acc[MR_TOKENS];
+#pragma unroll
+    for (int j = 0; j < MR_TOKENS; ++j) acc[j] = 0.f;
+    for (int k = lane * 8; k < K; k += 8 * DA_WAVE) {
+      uint4 hv[MR_TOKENS];
+      const uint4 wv = load16(row + k);
+#pragma unroll
+      for (int j = 0; j < MR_TOKENS; ++j) hv[j] = load16(h + (size_t)(n0 + j < N ? n0 + j : N - 1) * ldh + k);
+      const uint32_t b[4] = {wv.x, wv.y, wv.z, wv.w};
+#pragma unroll
+      for (int j = 0; j < MR_TOKENS; ++j) {
+        const uint32_t a[4] = {hv[j].x, hv[j].y, hv[j].z, hv[j].w};
+#pragma unroll
+        for (int e = 0; e < 4; ++e) {
+          acc[j] = fmaf(__uint_as_float(a[e] << 16), __uint_as_float(b[e] << 16), acc[j]);
+          acc[j] = fmaf(__uint_as_float(a[e] & 0xffff0000u), __uint_as_float(b[e] & 0xffff0000u), acc[j]);
+        }
+      }
+    }
+#pragma unroll
+    for (int j = 0; j < MR_TOKENS; ++j) {
+      const float v = wave_sum(acc[j]);
+      if (lane == 0 && n0 + j < N) give(n0 + j, v);
+    }
+  }
+}
+
+// The smallest steps: the router's product (h, router [E (+ 1)][K] in bfloat16, sums in 32-bit; or z holds its results), the
+// choice, and the pairs' layout in one launch.  ids and weights as da_moe_choose has them.
 #define MCR_WAVES 16
-#define MCR_MAX_OUTPUTS 128
+#define MCR_MAX_OUTPUTS 64
+#define MCR_MAX_TOKENS 16
 #define MCR_MAX_PAIRS 1024
+#define MCR_MAX_ROUTER_STEPS 8        // round trips to memory of a wavefront
 __global__ void __launch_bounds__(MCR_WAVES * DA_WAVE)
-moe_choose_route_kernel(const float* __restrict__ z, int ldz, const float* __restrict__ correction, int N, int E, int top, int groups,
+moe_choose_route_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __restrict__ router, int K,
+                        const float* __restrict__ z, int ldz, const float* __restrict__ correction, int N, int E, int top, int groups,
                         int keep, int extra, int n_experts, int tile, int* __restrict__ ids, float* __restrict__ weights,
                         int* __restrict__ slot_of_pair, int* __restrict__ row_of_slot, int* __restrict__ tile_expert, int P_cap,
                         int T_cap) {
-  __shared__ float mc_lds[MCR_WAVES][3][MCR_MAX_OUTPUTS];
+  __shared__ float logits[MCR_MAX_TOKENS][MCR_MAX_OUTPUTS + 1];
   __shared__ MoeRouteLds l;
   __shared__ int pair[MCR_MAX_PAIRS];
+  __shared__ float score[MCR_MAX_PAIRS];
   const int lane = threadIdx.x % DA_WAVE, wave = threadIdx.x / DA_WAVE, each = top + extra;
-  for (int n = wave; n < N; n += MCR_WAVES) {
-    int* const id = ids + (size_t)n * each;
-    float* const w = weights + (size_t)n * each;
+  if (h) {                                             // the logits are made here
+    for (int r = wave; r < E + (extra > 0); r += MCR_WAVES)
+      moe_router_row(h, ldh, N, router + (size_t)r * K, K, lane, [&](int n, float v) { logits[n][r] = v; });
+    lds_barrier();
+  }
+  const int n = wave;                                  // a token a wavefront
+  if (n < N) {
     int* const pr = pair + n * each;
-    const float* row = z + (size_t)n * ldz;
+    float* const sc = score + n * each;
+    const float* row = h ? logits[n] : z + (size_t)n * ldz;
     const float gate = extra ? row[E] : 0.f;
-    const float sum = moe_choose_token(row, correction, E, top, groups, keep, mc_lds[wave][0], mc_lds[wave][1], mc_lds[wave][2], lane,
-                                       [&](int k, int e, float s) {
-                                         const int x = e < n_experts ? e : e + extra;
-                                         id[k] = x;
-                                         pr[k] = x;
-                                       });
+    const float sum = moe_choose_token64(row, correction, E, top, groups, keep, lane, [&](int k, int e, float s) {
+      pr[k] = e < n_experts ? e : e + extra;
+      sc[k] = s;
+    });
     __builtin_amdgcn_fence(__ATOMIC_RELEASE, "workgroup", "local");
     __builtin_amdgcn_wave_barrier();
     __builtin_amdgcn_fence(__ATOMIC_ACQUIRE, "workgroup", "local");
     for (int k = lane; k < each; k += DA_WAVE) {
-      if (k < top) {
-        const int x = pr[k];
-        w[k] = mc_lds[wave][1][x < n_experts ? x : x - extra] / (sum + 1e-20f);
-      } else {
-        pr[k] = id[k] = n_experts + (k - top);
-        w[k] = 1.f / (1.f + expf(-gate));
-      }
+      const int e = k < top ? pr[k] : n_experts + (k - top);
+      if (k >= top) pr[k] = e;
+      ids[(size_t)n * each + k] = e;
+      weights[(size_t)n * each + k] = k < top ? sc[k] / (sum + 1e-20f) : 1.f / (1.f + expf(-gate));
     }
   }
-  __syncthreads();
+  lds_barrier();
   moe_lay_out(l, [&](int i) -> int { const int e = pair[i]; return e < n_experts + extra ? e : -1; }, N * each, each, n_experts + extra, tile,
               slot_of_pair, row_of_slot, tile_expert, P_cap, T_cap, nullptr, nullptr);
 }
 
 extern "C" int da_moe_choose_route_takes(int N, int E, int top, int extra, int n_experts) {
-  return E <= MCR_MAX_OUTPUTS && (long)N * (top + extra) <= MCR_MAX_PAIRS && n_experts + extra <= MOE_MAX_EXPERTS;
+  return N <= MCR_MAX_TOKENS && E <= MCR_MAX_OUTPUTS && (long)N * (top + extra) <= MCR_MAX_PAIRS && n_experts + extra <= MOE_MAX_EXPERTS;
 }
 
-extern "C" int da_moe_choose_route(const float* z, int ldz, const float* correction, int N, int E, int top, int groups, int keep,
+// 1 when it pays to make the logits there too
+extern "C" int da_moe_choose_route_takes_router(int N, int rows, int K) {
+  return N > 0 && N <= MCR_MAX_TOKENS && rows <= MCR_MAX_OUTPUTS + 1 && K % 8 == 0 &&
+         (long)da_ceil_div(rows, MCR_WAVES) * da_ceil_div(N, MR_TOKENS) * da_ceil_div(K, 8 * DA_WAVE) <= MCR_MAX_ROUTER_STEPS;
+}
+
+extern "C" int da_moe_choose_route(const void* h, int ldh, const void* router, int K, const float* z, int ldz, const float* correction, int N, int E, int top, int groups, int keep,
                                    int extra, int n_experts, int tile, int* ids, float* weights, int* slot_of_pair, int* row_of_slot,
                                    int* tile_expert, int P_cap, int T_cap, void* stream) {
   DA_REQUIRE(N >= 0 && E > 0 && top > 0 && top <= E && extra >= 0 && n_experts > 0 && n_experts <= E && tile > 0 &&
-             ldz >= E + (extra > 0) && correction, "moe_choose_route: bad sizes");
+             correction && (h || (z && ldz >= E + (extra > 0))), "moe_choose_route: bad sizes");
+  DA_REQUIRE(!h || (router && N <= MCR_MAX_TOKENS && K > 0 && K % 8 == 0 && ldh >= K && ldh % 8 == 0 && ((uintptr_t)h | (uintptr_t)router) % 16 == 0),
+             "moe_choose_route: the router's operands (rows of multiples of 8 entries, 16-byte aligned)");
   DA_REQUIRE(da_moe_choose_route_takes(N, E, top, extra, n_experts), "moe_choose_route: %d tokens with %d of %d outputs are not taken", N, top + extra, E);
   DA_REQUIRE(groups == 0 || (groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= E / groups * keep),
              "moe_choose_route: top %d of %d outputs in %d groups of which %d are kept", top, E, groups, keep);
   DA_REQUIRE(T_cap >= da_ceil_div((long)N * (top + extra), tile) + n_experts + extra && P_cap >= T_cap * tile,
              "moe_choose_route: the slot space (%d rows, %d tiles) is too small", P_cap, T_cap);
   if (N == 0) return 0;
-  hipLaunchKernelGGL(moe_choose_route_kernel, dim3(1), dim3(MCR_WAVES * DA_WAVE), 0, (hipStream_t)stream, z, ldz, correction, N, E, top,
-                     groups, keep, extra, n_experts, tile, ids, weights, slot_of_pair, row_of_slot, tile_expert, P_cap, T_cap);
+  hipLaunchKernelGGL(moe_choose_route_kernel, dim3(1), dim3(MCR_WAVES * DA_WAVE), 0, (hipStream_t)stream, (const bf16_t*)h, ldh,
+                     (const bf16_t*)router, K, z, ldz, correction, N, E, top, groups, keep, extra, n_experts, tile, ids, weights, slot_of_pair, row_of_slot, tile_expert, P_cap, T_cap);
   DA_CHECK_LAUNCH("moe_choose_route");
-  return 0;
-}
-
-extern "C" int da_moe_choose(const float* z, int ldz, const float* correction, int N, int E, int top, int groups, int keep,
-                             int* ids, float* weights, void* stream) {
-  DA_REQUIRE(N >= 0 && E > 0 && E <= MOE_MAX_EXPERTS && top > 0 && top <= E && ldz >= E && correction, "moe_choose: bad sizes");
-  DA_REQUIRE(groups == 0 || (groups > 0 && E % groups == 0 && keep > 0 && keep <= groups && top <= E / groups * keep),
-             "moe_choose: top %d of %d outputs in %d groups of which %d are kept", top, E, groups, keep);
-  if (N == 0) return 0;
-#define MC_GO(EC)                                                                                                            \
-  hipLaunchKernelGGL((moe_choose_kernel<EC>), dim3(da_ceil_div(N, MC_WAVES)), dim3(MC_WAVES * DA_WAVE), 0, (hipStream_t)stream, \
-                     z, ldz, correction, N, E, top, groups, keep, ids, weights)
-  if (E <= 64) MC_GO(64);
-  else if (E <= 256) MC_GO(256);
-  else MC_GO(MOE_MAX_EXPERTS);
-#undef MC_GO
-  DA_CHECK_LAUNCH("moe_choose");
   return 0;
 }
 
@@ -525,6 +644,7 @@ extern "C" int da_moe_combine(const float* out, int ldo, const int* slot_of_pair
 // `add` [N][width], `vec` [width], when the stream is changed before the next block), and the next block's norm of the new
 // row leaves in h_next.  centre: (x - mean) / sqrt(var + eps) * gain (+ bias); else x / sqrt(mean x^2 + eps) * (offset +
 // gain).  A wavefront owns a row, VPL float4 a lane (width a multiple of 4, at most 256 * VPL); all in 32-bit.
+template <int VPL> struct McnPairs { static const int value = VPL <= 4 ? 4 : (VPL <= 8 ? 2 : 1); };
 struct CombineNorm {
   const float* out; int ldo;
   const int* slot_of_pair;
@@ -560,9 +680,22 @@ moe_combine_norm_kernel(CombineNorm p) {
   const int n = blockIdx.x * (blockDim.x / DA_WAVE) + threadIdx.x / DA_WAVE;
   if (n >= p.N) return;
   const int E = p.width;
-  float4 x[VPL], g[VPL], b[VPL];
-  float4 s[VPL];
-  int at[VPL];
+  constexpr int PAIRS = McnPairs<VPL>::value;
+  // Everything whose place is known is asked for at once: the stream's row, the norm's parameters, the first pairs' slots
+  // and weights, the input that is handed on, the shared result; then PAIRS pairs' rows at a time (a pair without a
+  // slot reads row 0 and counts as nothing: looked at afterwards, a load under a condition would be waited for on the spot).
+  float4 x[VPL], g[VPL], b[VPL], s[VPL], hv[VPL], sv[VPL];
+  int at[VPL], slot[PAIRS];
+  float w[PAIRS];
+  auto ask = [&](int k0) {
+#pragma unroll
+    for (int k = 0; k < PAIRS; ++k) {
+      const size_t i = (size_t)n * p.top + (k0 + k < p.top ? k0 + k : 0);
+      slot[k] = p.slot_of_pair[i];
+      w[k] = p.weights ? p.weights[i] : p.uniform;
+    }
+  };
+  ask(0);
 #pragma unroll
   for (int i = 0; i < VPL; ++i) {
     const int c = (lane + i * DA_WAVE) * 4;
@@ -571,22 +704,33 @@ moe_combine_norm_kernel(CombineNorm p) {
     x[i] = mcn_load4(p.y + (size_t)n * E + at[i]);
     g[i] = mcn_param4(p.gain, p.gain_dtype, at[i]);
     b[i] = p.bias ? mcn_param4(p.bias, p.bias_dtype, at[i]) : make_float4(0.f, 0.f, 0.f, 0.f);
+    if (p.h) hv[i] = mcn_load4((const T*)p.h + (size_t)n * p.ldh + at[i]);
+    if (p.shared) sv[i] = mcn_load4(p.shared + (size_t)n * p.lds + at[i]);
   }
-  for (int k = 0; k < p.top; ++k) {
-    const int slot = p.slot_of_pair[(size_t)n * p.top + k];
-    const float w = p.weights ? p.weights[(size_t)n * p.top + k] : p.uniform;
-    if (slot >= 0) {
+  const float gate = p.shared ? p.gate[(size_t)n * p.ldg] : 0.f;
+  float handed_on = 0.f;
+  for (int k0 = 0; k0 < p.top; k0 += PAIRS) {
+    if (k0) ask(k0);
+    float4 v[PAIRS][VPL];
 #pragma unroll
-      for (int i = 0; i < VPL; ++i) s[i] = mcn_fma(w, mcn_load4(p.out + (size_t)slot * p.ldo + at[i]), s[i]);
-    } else if (p.h) {
+    for (int k = 0; k < PAIRS; ++k)
 #pragma unroll
-      for (int i = 0; i < VPL; ++i) s[i] = mcn_fma(w, mcn_load4((const T*)p.h + (size_t)n * p.ldh + at[i]), s[i]);
+      for (int i = 0; i < VPL; ++i) v[k][i] = mcn_load4(p.out + (size_t)(slot[k] >= 0 ? slot[k] : 0) * p.ldo + at[i]);
+#pragma unroll
+    for (int k = 0; k < PAIRS; ++k) {
+      if (k0 + k >= p.top) continue;
+      if (slot[k] >= 0) {
+#pragma unroll
+        for (int i = 0; i < VPL; ++i) s[i] = mcn_fma(w[k], v[k][i], s[i]);
+      } else {
+        handed_on += w[k];
+      }
     }
   }
-  if (p.shared) {
-    const float w = 1.f / (1.f + expf(-p.gate[(size_t)n * p.ldg]));
 #pragma unroll
-    for (int i = 0; i < VPL; ++i) s[i] = mcn_fma(w, mcn_load4(p.shared + (size_t)n * p.lds + at[i]), s[i]);
+  for (int i = 0; i < VPL; ++i) {
+    if (p.h) s[i] = mcn_fma(handed_on, hv[i], s[i]);
+    if (p.shared) s[i] = mcn_fma(1.f / (1.f + expf(-gate)), sv[i], s[i]);
   }
   float sum = 0.f;
 #pragma unroll
@@ -672,19 +816,28 @@ moe_mfma_kernel(const bf16_t* __restrict__ a, int lda, const int* __restrict__ r
   constexpr bool GATED = MODE == MOE_GATED, GATHER = MODE != MOE_DOWN;
   constexpr int G = GATED ? 2 : 1;
   __shared__ float sums[NW][G][8][DA_WAVE];                 // [wavefront][product][register of the tile][lane]
-  const int e = tile_expert[blockIdx.y];
-  if (e < 0) return;
   const int t = threadIdx.x, lane = t % DA_WAVE, wave = t / DA_WAVE;
   const int fr = lane % 16, fk = (lane / 16) * 8;
   const int m0 = blockIdx.y * MM_ROWS, n0 = blockIdx.x * MM_COLS;
+  // every load of the routing at once: the expert, the rows of a, the rows that this thread will store
+  constexpr int PER = (8 + NW - 1) / NW;
+  const int e = tile_expert[blockIdx.y];
+  int srow[2], used[PER];
+#pragma unroll
+  for (int i = 0; i < 2; ++i) srow[i] = row_of_slot[m0 + i * 16 + fr];
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int x = (wave + j * NW) % 8;
+    used[j] = row_of_slot[m0 + x / 4 * 16 + 4 * (lane / 16) + x % 4];
+  }
+  if (e < 0) return;
   // the rows of a: gathered by slot for the first product (a padding slot reads row 0 and is never stored),
   // the slot's own row for the second; an expert's slots are filled from the front
-  const bool two = row_of_slot[m0 + 16] >= 0;               // (the same for the workgroup)
+  const bool two = __builtin_amdgcn_readfirstlane(srow[1]) >= 0;      // (lane 0's: slot m0 + 16; the same for the workgroup)
   const bf16_t* ap[2];
 #pragma unroll
   for (int i = 0; i < 2; ++i) {
-    const int srow = row_of_slot[m0 + i * 16 + fr];
-    const int r = GATHER ? (srow >= 0 ? srow : 0) : m0 + i * 16 + fr;
+    const int r = GATHER ? (srow[i] >= 0 ? srow[i] : 0) : m0 + i * 16 + fr;
     ap[i] = a + (size_t)r * lda + fk;
   }
   const int wcol = n0 + fr < F ? n0 + fr : 0;
@@ -727,11 +880,13 @@ moe_mfma_kernel(const bf16_t* __restrict__ a, int lda, const int* __restrict__ r
     for (int i = 0; i < 2; ++i)
 #pragma unroll
       for (int r = 0; r < 4; ++r) sums[wave][g][i * 4 + r][lane] = acc[i][g][r];
-  __syncthreads();
+  lds_barrier();
   // acc[i][.][r] of a lane is row 16 i + 4 (lane / 16) + r of the tile, column n0 + lane % 16
-  for (int x = wave; x < 8; x += NW) {
+#pragma unroll
+  for (int j = 0; j < PER; ++j) {
+    const int x = wave + j * NW;
     const int row = x / 4 * 16 + 4 * (lane / 16) + x % 4;
-    if (row_of_slot[m0 + row] < 0 || n0 + fr >= F) continue;
+    if (x >= 8 || used[j] < 0 || n0 + fr >= F) continue;
     float v[G];
 #pragma unroll
     for (int g = 0; g < G; ++g) {

@@ -151,11 +151,12 @@ _ARGTYPES = {
                           _VP, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_moe_combine": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _I, _VP, _I, _I, _VP, _I, _VP, _I, _VP],
     "da_moe_choose_route_takes": [_I, _I, _I, _I, _I],
-    "da_moe_choose_route": [_VP, _I, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
+    "da_moe_choose_route_takes_router": [_I, _I, _I],
+    "da_moe_choose_route": [_VP, _I, _VP, _I, _VP, _I, _VP, _I, _I, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP, _VP, _VP, _I, _I, _VP],
     "da_moe_combine_norm_takes": [_I],
     "da_moe_combine_norm": [_VP, _I, _VP, _VP, _F, _I, _VP, _I, _I, _I, _VP, _I, _VP, _I, _VP, _I, _VP, _VP, _VP, _I, _VP, _I, _F, _F,
                             _I, _VP, _I, _VP],
-    "da_moe_choose": [_VP, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP, _VP],
+    "da_moe_choose": [_VP, _I, _VP, _I, _I, _I, _I, _I, _I, _I, _VP, _VP, _VP],
     "da_add_rows": [_VP, _VP, _VP, _I, _I, _VP],
     "da_rglru_walk": [_VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _VP],
     "da_rglru_serve_takes": [_I],
@@ -436,6 +437,7 @@ def softcap(logits: torch.Tensor, cap: float) -> torch.Tensor:
 
 
 # ------------------------------------------------------------------------------- experts
+MOE_MAX_EXPERTS = 1024   # (csrc/moe.hip)
 MOE_TILE_ROWS = 64       # rows of a tile of the plain grouped products
 MOE_TILE_ROWS_MFMA = 32  # ... of the matrix-core grouped products for few rows an expert (csrc/moe.hip)
 MOE_TILE_ROWS_BLOCK = 128  # ... of the block-tile product with a matrix per group of rows (csrc/gemm_mfma.hip)
@@ -1291,32 +1293,42 @@ def moe_top(z: torch.Tensor, bias: Optional[torch.Tensor], top: int, mode: str, 
 
 
 def moe_choose(z: torch.Tensor, outputs: int, correction: torch.Tensor, top: int, groups: int, groups_kept: int, ids: torch.Tensor,
-               weights: torch.Tensor) -> None:
+               weights: torch.Tensor, extra: int = 0, n_experts: int = 0) -> None:
     """From 32-bit router logits (the first ``outputs`` columns of z): s = their softmax, the ``top`` largest entries of
     s + correction (the lower index wins a tie; inside the ``groups_kept`` best of ``groups`` equal groups of neighbours,
-    if there are groups) as ids[n, k] in descending order, and weights[n, k] = s over the chosen ones' sum (+ 1e-20)."""
+    if there are groups) as ids[n, k] in descending order, and weights[n, k] = s over the chosen ones' sum (+ 1e-20).
+    ``extra``: ids and weights are [N, top + extra]; ids from ``n_experts`` on are moved up by it, and behind the choice come
+    the experts n_experts .. that every token uses with the weight logistic(z[n, outputs])."""
     _dev(z, correction, ids, weights)
     _rows_2d(z, "z")
     N = z.shape[0]
-    _need(z.dtype == torch.float32 and z.shape[1] >= outputs, "moe_choose: router logits must be float32 [N, >= outputs]")
+    each = top + extra
+    _need(z.dtype == torch.float32 and z.shape[1] >= outputs + (1 if extra else 0), "moe_choose: router logits must be float32 [N, >= outputs]")
     _need(correction.dtype == torch.float32 and correction.is_contiguous() and correction.numel() == outputs,
           "moe_choose: the correction must be float32 with one entry an output")
-    _need(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= N * top and weights.dtype == torch.float32
-          and weights.is_contiguous() and weights.numel() >= N * top, "moe_choose: ids int32 and weights float32, [N, top]")
+    _need(ids.dtype == torch.int32 and ids.is_contiguous() and ids.numel() >= N * each and weights.dtype == torch.float32
+          and weights.is_contiguous() and weights.numel() >= N * each, "moe_choose: ids int32 and weights float32, [N, top]")
     with _timed("moe_choose", N * outputs * 4 + N * top * 8, N * outputs * (top + 6), "fp32"):
-        _check(_lib().da_moe_choose(_ptr(z), z.stride(0), _ptr(correction), N, outputs, top, int(groups), int(groups_kept), _ptr(ids),
-                                    _ptr(weights), _stream()))
+        _check(_lib().da_moe_choose(_ptr(z), z.stride(0), _ptr(correction), N, outputs, top, int(groups), int(groups_kept), extra,
+                                    n_experts if extra else outputs, _ptr(ids), _ptr(weights), _stream()))
 
 
 def moe_choose_route(choice: "ExpertChoice", top: int, extra: int, n_experts: int, tile: int, ids: torch.Tensor, weights: torch.Tensor,
-                     slot_of_pair: torch.Tensor, row_of_slot: torch.Tensor, tile_expert: torch.Tensor, n_tokens: int) -> None:
-    """``moe_choose`` and ``moe_route`` of a small step in one launch.  ids and weights are [N, top + extra]: the choice (ids
+                     slot_of_pair: torch.Tensor, row_of_slot: torch.Tensor, tile_expert: torch.Tensor, n_tokens: int,
+                     h: Optional[torch.Tensor] = None) -> None:
+    """``moe_choose`` and ``moe_route`` of a small step in one launch; with ``h`` [N, width] also the product with
+    ``choice.router`` (bfloat16, 32-bit sums; ``choice.z`` is then not used).  ids and weights are [N, top + extra]: the choice (ids
     from ``n_experts`` on are moved up by ``extra``), then the ``extra`` experts n_experts .. that every token uses with the
     weight logistic(z[n, outputs])."""
     z, E = choice.z, choice.outputs
-    _dev(z, choice.correction, ids, weights, slot_of_pair, row_of_slot, tile_expert)
+    _dev(z, choice.correction, ids, weights, slot_of_pair, row_of_slot, tile_expert, h)
     _rows_2d(z, "z")
     N, each = n_tokens, top + extra
+    if h is not None:
+        _rows_2d(h, "h")
+        _need(h.dtype == choice.router.dtype == torch.bfloat16 and h.shape[0] >= N and choice.router.is_contiguous()
+              and choice.router.shape[0] >= E + (1 if extra else 0) and choice.router.shape[1] == h.shape[1],
+              "moe_choose_route: h [N, width] and the router [outputs (+ 1), width] in bfloat16")
     tiles, rows = moe_slot_space(N, each, n_experts + extra, tile)
     _need(z.dtype == torch.float32 and z.shape[0] >= N and z.shape[1] >= E + (1 if extra else 0), "moe_choose_route: router logits must be float32 [N, >= outputs]")
     _need(choice.correction.dtype == torch.float32 and choice.correction.is_contiguous() and choice.correction.numel() == E,
@@ -1327,8 +1339,9 @@ def moe_choose_route(choice: "ExpertChoice", top: int, extra: int, n_experts: in
         _need(t_.dtype == torch.int32 and t_.is_contiguous(), "moe_choose_route: int32 contiguous operands")
     _need(slot_of_pair.numel() >= N * each and row_of_slot.numel() >= rows and tile_expert.numel() >= tiles,
           "moe_choose_route: the outputs are smaller than the slot space")
-    with _timed("moe_choose_route", N * E * 4 + N * each * 12 + 4 * (rows + tiles), N * E * (top + 6), "fp32"):
-        _check(_lib().da_moe_choose_route(_ptr(z), z.stride(0), _ptr(choice.correction), N, E, top, int(choice.groups),
+    with _timed("moe_choose_route", (N * E * 4 if h is None else _nbytes(choice.router) + N * h.shape[1] * 2) + N * each * 12 + 4 * (rows + tiles), N * E * (top + 6), "fp32"):
+        _check(_lib().da_moe_choose_route(_ptr(h), 0 if h is None else h.stride(0), None if h is None else _ptr(choice.router),
+                                          0 if h is None else h.shape[1], None if h is not None else _ptr(z), z.stride(0), _ptr(choice.correction), N, E, top, int(choice.groups),
                                           int(choice.groups_kept), extra, n_experts, tile, _ptr(ids), _ptr(weights), _ptr(slot_of_pair),
                                           _ptr(row_of_slot), _ptr(tile_expert), rows, tiles, _stream()))
 
@@ -1355,24 +1368,25 @@ def moe_top_logistic(z: torch.Tensor, top: int, renorm: bool, ids: torch.Tensor,
 
 @dataclass(frozen=True)
 class ExpertChoice:
-    """A choice still to be made: what ``moe_choose`` takes (``z`` may hold a shared gate behind the outputs)."""
+    """A choice still to be made: what ``moe_choose`` takes (``z`` may hold a shared gate behind the outputs).  ``router``
+    [outputs (+ 1), width]: z has not been filled; it is made where the choice is, or by a product in front of it."""
     z: torch.Tensor
     outputs: int
     correction: torch.Tensor
     groups: int
     groups_kept: int
+    router: Optional[torch.Tensor] = None
 
 
 SHARED_AS_EXPERTS_MAX_ROWS = 64      # steps in which a shared feed-forward rides along as further experts
 
 
-def shared_rides_along(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, choice: ExpertChoice, n_experts: int, top: int,
-                       extra: int) -> bool:
+def shared_rides_along(h: torch.Tensor, gate_up: torch.Tensor, down: torch.Tensor, n_experts: int, top: int, extra: int) -> bool:
     """Whether a shared feed-forward of this step runs as ``extra`` further experts of the grouped products (``gate_up`` and
     ``down`` are the stacks with them): few rows, so that weights are streamed once either way and three launches fall away."""
     N = h.shape[0]
     return (extra > 0 and N <= SHARED_AS_EXPERTS_MAX_ROWS and N * (top + extra) < 64 * (n_experts + extra) and _moe_mfma_ok(h, gate_up, down)
-            and bool(_lib().da_moe_choose_route_takes(N, choice.outputs, top, extra, n_experts)))
+            and n_experts + extra <= MOE_MAX_EXPERTS)
 
 
 def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up: torch.Tensor, down: torch.Tensor,
@@ -1410,13 +1424,20 @@ def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up
     # a pair's weight where its slot is: the first product scales its rows with it
     slot_scale = ctx.buf("moe_slot_scale", rows, 1, torch.float32).view(-1) if weight_input else None
     if choice is not None and not weight_input and bool(_lib().da_moe_choose_route_takes(N, choice.outputs, chosen, extra, routed)):
-        moe_choose_route(choice, chosen, extra, routed, tile, ids, pair_weights, slot_of_pair, row_of_slot, tile_expert, N)
+        inside = (choice.router is not None and mfma and choice.router.dtype == torch.bfloat16
+                  and bool(_lib().da_moe_choose_route_takes_router(N, choice.outputs + (1 if extra else 0), width)))
+        if choice.router is not None and not inside:
+            linear(h, choice.router, None, choice.z)
+        moe_choose_route(choice, chosen, extra, routed, tile, ids, pair_weights, slot_of_pair, row_of_slot, tile_expert, N,
+                         h if inside else None)
     elif ids is None:
         moe_route(ctx.tokens, table, None, N, top, n_experts, tile, slot_of_pair, row_of_slot, tile_expert)
     else:
         if choice is not None:
-            _need(extra == 0, "experts: a shared feed-forward rides along in small steps only")
-            moe_choose(choice.z, choice.outputs, choice.correction, top, choice.groups, choice.groups_kept, ids, pair_weights)
+            if choice.router is not None:
+                linear(h, choice.router, None, choice.z)
+            moe_choose(choice.z, choice.outputs, choice.correction, chosen, choice.groups, choice.groups_kept, ids, pair_weights,
+                       extra, routed)
         moe_route(None, None, ids, N, top, n_experts, tile, slot_of_pair, row_of_slot, tile_expert,
                   pair_weights if weight_input else None, slot_scale)
     mid = ctx.buf("moe_mid", rows, inner, h.dtype)

@@ -3,6 +3,8 @@ Reference: core/src/main/java/io/teknek/deliverance/generator/MLPBlock.java:250-
 two-bias, no-gate form GPT-2 uses, :93-114); residual add TransformerBlock.java:188."""
 from __future__ import annotations
 
+import dataclasses
+
 import torch
 
 from ..kernels import ops
@@ -201,18 +203,22 @@ class ExpertsFeedForward(FeedForward):
         gate_up, down = self.gate_up_weight, self.down_weight
         if self.router_weight is not None:
             z = ctx.buf("moe_logits", N, self.router_weight.shape[0], torch.float32)      # 32-bit sums of the products
-            ops.linear(h, self.router_weight, None, z)
             if self.router == "softmax_all":
-                choice = ops.ExpertChoice(z, self.outputs, self.correction, self.groups, self.groups_kept)
-                if self.extra and ops.shared_rides_along(h, self.gate_up_all, self.down_all, choice, self.n_experts, self.top, self.extra):
+                # (z is filled where the choice is made; not yet where a gate behind the outputs is read from it)
+                choice = ops.ExpertChoice(z, self.outputs, self.correction, self.groups, self.groups_kept, self.router_weight)
+                if self.extra and ops.shared_rides_along(h, self.gate_up_all, self.down_all, self.n_experts, self.top, self.extra):
                     extra, gate_up, down = self.extra, self.gate_up_all, self.down_all
             ids = ctx.buf("moe_ids", N, self.top + extra, torch.int32)
             weights = ctx.buf("moe_weights", N, self.top + extra, torch.float32)
+            if self.router != "softmax_all":
+                ops.linear(h, self.router_weight, None, z)
             if self.router == "softmax_top":
                 ops.moe_top(z, self.router_bias, self.top, "softmax", False, ids, weights)
             elif self.router == "logistic_top":
                 ops.moe_top(z, self.router_bias, self.top, "logistic", self.renormalize, ids, weights)
         if self.token_gate and not extra:
+            ops.linear(h, self.router_weight, None, z)
+            choice = dataclasses.replace(choice, router=None)
             shared_out = ctx.buf("moe_shared_out", N, self.width, torch.float32)
             self._run_shared(ctx, h, shared_out, False)
         plain_shared = self.shared is not None and not self.token_gate

@@ -131,6 +131,7 @@ static inline float __shfl_xor(float v, int mask, int) {
 static inline int __shfl_xor(int v, int mask, int) {
   return (int)simt::lane_exchange((uint32_t)v, simt::lane_id() ^ mask, 0u);
 }
+static inline int __shfl(int v, int src, int) { return (int)simt::lane_exchange((uint32_t)v, src, 0u); }
 static inline float __shfl(float v, int src, int) {
   return __uint_as_float(simt::lane_exchange(__float_as_uint(v), src, 0u));
 }

@@ -481,8 +481,8 @@ def test_the_choice_of_experts(experts, top, groups):
         assert np.abs(host(w) - want_w).max() <= 2e-6
 
 
-@pytest.mark.parametrize("rows,experts,ident,top,groups,extra", [quick(5, 6, 2, 3, (4, 2), 2), (1, 1, 0, 1, None, 1), (17, 9, 3, 4, (3, 2), 0), (64, 8, 2, 2, (2, 1), 2),
-                                                                 (33, 100, 28, 6, (16, 5), 4), (100, 3, 5, 2, None, 3)])
+@pytest.mark.parametrize("rows,experts,ident,top,groups,extra", [quick(5, 6, 2, 3, (4, 2), 2), (1, 1, 0, 1, None, 1), (13, 9, 3, 4, (3, 2), 0), (16, 8, 2, 2, (2, 1), 2),
+                                                                 (11, 50, 14, 6, (16, 5), 4), (2, 3, 5, 2, None, 3)])
 def test_the_choice_and_the_layout_in_one_launch(rows, experts, ident, top, groups, extra):
     """The same ids and weights as the choice alone, ids of experts that hand their input on moved up, the further experts'
     pairs behind them with a logistic weight; every pair of an expert with matrices in a slot of its expert's tiles."""
@@ -512,6 +512,20 @@ def test_the_choice_and_the_layout_in_one_launch(rows, experts, ident, top, grou
                 assert row_of[slot[n, k]] == n and tile_of[slot[n, k] // tile] == i2[n, k] and slot[n, k] not in used
                 used.add(slot[n, k])
     assert all(row_of[i] == -1 for i in range(space) if i not in used)
+    # the choice alone, with the further experts behind it
+    i5, w5 = torch.zeros(rows, each, dtype=torch.int32, device=DEV), torch.zeros_like(w2)
+    ops.moe_choose(z, E, corr, top, *g, i5, w5, extra, experts)
+    assert np.array_equal(i5.cpu().numpy(), i2) and float((w5 - w2).abs().max()) <= 1e-6
+    # ... and with the router's product inside (a step of few tokens)
+    h, router = bf16(rng.normal(size=(rows, 1104))), bf16(rng.normal(size=(E + 1, 1104)) * 0.1)
+    zz = dev((h @ router.T).astype(np.float32), torch.float32)
+    i3, w3, i4, w4 = torch.zeros(rows, each, dtype=torch.int32, device=DEV), torch.zeros_like(w2), torch.zeros(rows, each, dtype=torch.int32, device=DEV), torch.zeros_like(w2)
+    lay = [torch.full((n,), -9, dtype=torch.int32, device=DEV) for n in (rows * each, space, tiles)]
+    ops.moe_choose_route(ops.ExpertChoice(zz, E, corr, *g), top, extra, experts, tile, i3, w3, *lay, rows)
+    ops.moe_choose_route(ops.ExpertChoice(torch.full_like(zz, float("nan")), E, corr, *g, dev(router, torch.bfloat16)), top, extra, experts, tile,
+                         i4, w4, *lay, rows, dev(h, torch.bfloat16))
+    same = (i3 == i4).all(1)                            # (two scores may lie within rounding of one another)
+    assert int((~same).sum()) <= 1 and (not bool(same.any()) or float((w3 - w4)[same].abs().max()) <= 1e-5)
 
 
 @pytest.mark.parametrize("dtype", ["float32", quick("bfloat16")])
