@@ -32,6 +32,9 @@ struct KvScatter {
   const int* slot_map;  // per row: page * page_size + row in page, or -1
   int q_cols, kv_cols;  // k occupies columns [q_cols, q_cols + kv_cols), v the next kv_cols
   int Hkv, D, page;
+  // The products for few rows also take values of a size of their own (a page then holds Hkv * page * D keys, then Hkv *
+  // Dv * page values) and columns behind q | k | v that are not kept; 0: Dv is D, and v is the last of the columns.
+  int Dv = 0;
 };
 
 // column n (>= q_cols) of a row whose place in the cache is row `row` of page `pg`
@@ -44,7 +47,15 @@ __device__ __forceinline__ void kv_scatter_bits(const KvScatter& kv, int pg, int
 }
 
 __device__ __forceinline__ void kv_scatter_store(const KvScatter& kv, int slot, int n, float v) {
-  kv_scatter_bits(kv, slot / kv.page, slot % kv.page, n, f32_to_bf16(v));
+  const int pg = slot / kv.page, row = slot % kv.page;
+  if (kv.Dv == 0) {
+    kv_scatter_bits(kv, pg, row, n, f32_to_bf16(v));
+    return;
+  }
+  bf16_t* base = (bf16_t*)kv.cache + (long long)pg * kv.Hkv * kv.page * (kv.D + kv.Dv);
+  const int c = n - kv.q_cols, cv = c - kv.kv_cols;
+  if (cv < 0) base[((long long)(c / kv.D) * kv.page + row) * kv.D + c % kv.D] = f32_to_bf16(v);
+  else if (cv < kv.Hkv * kv.Dv) base[(long long)kv.Hkv * kv.page * kv.D + (long long)cv * kv.page + row] = f32_to_bf16(v);
 }
 
 __device__ __forceinline__ uint4 load16(const bf16_t* p) { return *(const uint4*)p; }

@@ -741,10 +741,13 @@ static int launch_skinny4(int nw, hipStream_t s, const bf16_t* A, int lda, const
   return 0;
 }
 
-extern "C" int da_gemm_bf16(const void* a, int lda, const void* w, int ldw, const void* bias, int bias_dtype,
-                            int act, int accumulate, void* out, int out_dtype, int ldo, int M, int N, int K,
-                            void* kv_cache, const int* slot_map, int q_cols, int kv_cols, int Hkv, int D, int page,
-                            void* stream) {
+// 1 when a product of so many rows and columns goes to the kernels for few rows
+extern "C" int da_gemm_few_rows(int M, int N) {
+  return M <= 32 || (M <= 64 && N <= 8192);           // (a vocabulary with more than 32 rows: block tiles reuse the rows of a)
+}
+
+static int gemm_bf16_checks(const void* a, int lda, const void* w, int ldw, int act, int accumulate, int out_dtype, int ldo, int M,
+                            int N, int K) {
   DA_REQUIRE(M >= 0 && N > 0 && K > 0, "gemm_bf16: bad sizes M=%d N=%d K=%d", M, N, K);
   DA_REQUIRE(K % 8 == 0 && lda % 8 == 0 && ldw % 8 == 0,
              "gemm_bf16: K, lda and ldw must be multiples of 8 (K=%d lda=%d ldw=%d)", K, lda, ldw);
@@ -752,13 +755,45 @@ extern "C" int da_gemm_bf16(const void* a, int lda, const void* w, int ldw, cons
   DA_REQUIRE(lda >= K && ldw >= K && ldo >= N, "gemm_bf16: leading sizes too small");
   DA_REQUIRE(!accumulate || out_dtype == DA_F32, "gemm_bf16: accumulation needs a 32-bit output");
   DA_REQUIRE(act >= DA_ACT_NONE && act <= DA_ACT_LAST, "gemm_bf16: unknown activation %d", act);
+  return 0;
+}
+
+static int gemm_bf16_launch(const void* a, int lda, const void* w, int ldw, const Epilogue& ep, const KvScatter& kv, int M, int N,
+                            int K, void* stream);
+
+extern "C" int da_gemm_bf16(const void* a, int lda, const void* w, int ldw, const void* bias, int bias_dtype,
+                            int act, int accumulate, void* out, int out_dtype, int ldo, int M, int N, int K,
+                            void* kv_cache, const int* slot_map, int q_cols, int kv_cols, int Hkv, int D, int page,
+                            void* stream) {
+  if (gemm_bf16_checks(a, lda, w, ldw, act, accumulate, out_dtype, ldo, M, N, K)) return 1;
   if (kv_cache) {
     DA_REQUIRE(out_dtype == DA_BF16 && !accumulate && q_cols >= 0 && kv_cols == Hkv * D && q_cols + 2 * kv_cols == N &&
                page > 0 && (page & (page - 1)) == 0, "gemm_bf16: the q|k|v columns (%d + 2*%d) must add up to N=%d, the page size a power of two", q_cols, kv_cols, N);
   }
   if (M == 0) return 0;
-  Epilogue ep{bias, bias_dtype, act, accumulate, out, out_dtype, ldo};
-  KvScatter kv{kv_cache, slot_map, q_cols, kv_cols, Hkv, D, page};
+  const Epilogue ep{bias, bias_dtype, act, accumulate, out, out_dtype, ldo};
+  const KvScatter kv{kv_cache, slot_map, q_cols, kv_cols, Hkv, D, page};
+  return gemm_bf16_launch(a, lda, w, ldw, ep, kv, M, N, K, stream);
+}
+
+// The same for few rows (da_gemm_few_rows) of a q | k | v | rest product whose values have a size of their own and whose
+// columns behind v are not kept (see KvScatter).
+extern "C" int da_gemm_bf16_kv_split(const void* a, int lda, const void* w, int ldw, const void* bias, int bias_dtype, void* out,
+                                     int ldo, int M, int N, int K, void* kv_cache, const int* slot_map, int q_cols, int Hkv, int D,
+                                     int Dv, int page, void* stream) {
+  if (gemm_bf16_checks(a, lda, w, ldw, DA_ACT_NONE, 0, DA_BF16, ldo, M, N, K)) return 1;
+  DA_REQUIRE(da_gemm_few_rows(M, N), "gemm_bf16_kv_split: %d rows of %d columns are more than the kernels for few rows take", M, N);
+  DA_REQUIRE(kv_cache && slot_map && q_cols >= 0 && Hkv > 0 && D > 0 && Dv > 0 && page > 0 && q_cols + Hkv * (D + Dv) <= N,
+             "gemm_bf16_kv_split: the k and v columns leave the row");
+  if (M == 0) return 0;
+  const Epilogue ep{bias, bias_dtype, DA_ACT_NONE, 0, out, DA_BF16, ldo};
+  const KvScatter kv{kv_cache, slot_map, q_cols, Hkv * D, Hkv, D, page, Dv};
+  return gemm_bf16_launch(a, lda, w, ldw, ep, kv, M, N, K, stream);
+}
+
+static int gemm_bf16_launch(const void* a, int lda, const void* w, int ldw, const Epilogue& ep, const KvScatter& kv, int M, int N,
+                            int K, void* stream) {
+  const int act = ep.act, accumulate = ep.accumulate, out_dtype = ep.out_dtype;
   hipStream_t s = (hipStream_t)stream;
   const bf16_t* A = (const bf16_t*)a;
   const bf16_t* W = (const bf16_t*)w;
@@ -767,7 +802,7 @@ extern "C" int da_gemm_bf16(const void* a, int lda, const void* w, int ldw, cons
     const int nw = K >= 2048 ? 16 : (K >= 1024 ? 8 : 4);   // by K alone, so a row's sums keep their order
     if (N <= 1024 ? launch_skinny4<1>(nw, s, A, lda, W, ldw, ep, kv, M, N, K)
                   : launch_skinny4<2>(nw, s, A, lda, W, ldw, ep, kv, M, N, K)) return 1;
-  } else if (M <= 32 || (M <= 64 && N <= 8192)) {     // (a vocabulary with more than 32 rows: block tiles reuse the rows of a)
+  } else if (da_gemm_few_rows(M, N)) {
     // The number of wavefronts that split K depends on K and N alone, so a row's sums keep their order:
     // 4 where the workgroups are many (a vocabulary: several then share a compute unit), else 8, or 12 for a long K.
     const int nw = da_ceil_div(N, 16) > 1024 ? 4 : (K >= 2048 ? 12 : 8);

@@ -389,10 +389,9 @@ __device__ __forceinline__ float moe_choose_token(const float* __restrict__ row,
 
 // The same for at most 64 outputs: an output a lane, everything in registers.
 template <class Give>
-__device__ __forceinline__ float moe_choose_token64(const float* __restrict__ row, const float* __restrict__ correction, int E, int top,
-                                                    int groups, int keep, int lane, Give give) {
-  const bool in = lane < E;
-  const float corr = correction[in ? lane : 0];
+__device__ __forceinline__ float moe_choose_token64(const float* __restrict__ row, float corr, int E, int top, int groups, int keep,
+                                                    int lane, Give give) {
+  const bool in = lane < E;                            // corr: this lane's output's
   const float z = in ? row[lane] : -INFINITY;
   const float m = wave_max(z);                         // (every lane takes part in what goes across lanes)
   const float ex = in ? expf(z - m) : 0.f;
@@ -442,7 +441,7 @@ moe_choose_kernel(const float* __restrict__ z, int ldz, const float* __restrict_
     id[k] = e < n_experts ? e : e + extra;
     w[k] = s;
   };
-  if (EC <= 64) sum = moe_choose_token64(row, correction, E, top, groups, keep, lane, give);
+  if (EC <= 64) sum = moe_choose_token64(row, correction[lane < E ? lane : 0], E, top, groups, keep, lane, give);
   else sum = moe_choose_token(row, correction, E, top, groups, keep, mc_lds[EC > 64 ? wave : 0][0], mc_lds[EC > 64 ? wave : 0][1],
                               mc_lds[EC > 64 ? wave : 0][2], lane, give);
   if (lane == 0)
@@ -525,6 +524,7 @@ moe_choose_route_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __r
   __shared__ int pair[MCR_MAX_PAIRS];
   __shared__ float score[MCR_MAX_PAIRS];
   const int lane = threadIdx.x % DA_WAVE, wave = threadIdx.x / DA_WAVE, each = top + extra;
+  const float corr = correction[lane < E ? lane : 0];  // (asked for first)
   if (h) {                                             // the logits are made here
     for (int r = wave; r < E + (extra > 0); r += MCR_WAVES)
       moe_router_row(h, ldh, N, router + (size_t)r * K, K, lane, [&](int n, float v) { logits[n][r] = v; });
@@ -536,7 +536,7 @@ moe_choose_route_kernel(const bf16_t* __restrict__ h, int ldh, const bf16_t* __r
     float* const sc = score + n * each;
     const float* row = h ? logits[n] : z + (size_t)n * ldz;
     const float gate = extra ? row[E] : 0.f;
-    const float sum = moe_choose_token64(row, correction, E, top, groups, keep, lane, [&](int k, int e, float s) {
+    const float sum = moe_choose_token64(row, corr, E, top, groups, keep, lane, [&](int k, int e, float s) {
       pr[k] = e < n_experts ? e : e + extra;
       sc[k] = s;
     });

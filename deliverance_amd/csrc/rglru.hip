@@ -152,11 +152,11 @@ __device__ __forceinline__ void lru_load_gates(const LruIn& in, int b, int n0, i
   }
 }
 
-// Decode: rows q_start[seq0 + j], j = 0 .. n - 1.  blockDim = 2 KS wavefronts, so that every 16 channels have one.
+// Decode: sequence j of the first n has row j (one-token sequences lead a step).  blockDim = 2 KS wavefronts, so that every 16 channels have one.
 // KT: taps rounded up; taps that do not exist have no weight and read the token itself.
 template <int KS, int KT>
 __global__ void __launch_bounds__(2 * KS * DA_WAVE)
-rglru_decode_kernel(LruIn in, int seq0, int n) {
+rglru_decode_kernel(LruIn in, int n) {
   constexpr int PITCH = KS * 32 + 8;
   __shared__ __attribute__((aligned(16))) bf16_t us[16][PITCH];
   const int b = blockIdx.x, j0 = blockIdx.y * 16;
@@ -169,24 +169,24 @@ rglru_decode_kernel(LruIn in, int seq0, int n) {
   if (cols) lru_load_gates<KS>(in, b, n0, lane, wr, wi);
   // this lane's four sequences: state, branch, what the gates need
   float s_old[4], yv[4];
-  int slot[4], row[4];
+  int slot[4];
 #pragma unroll
   for (int r = 0; r < 4; ++r) {
     const int j = j0 + 4 * g + r, jj = j < n ? j : n - 1;
-    row[r] = in.q_start[seq0 + jj];
-    slot[r] = in.slots[seq0 + jj];
-    s_old[r] = in.state[(size_t)(slot[r] >= 0 ? slot[r] : 0) * in.state_ld + c];
-    yv[r] = bf16_to_f32(in.yx[(size_t)row[r] * in.ld + c]);
+    slot[r] = in.slots[jj];
+    yv[r] = bf16_to_f32(in.yx[(size_t)jj * in.ld + c]);
   }
+#pragma unroll
+  for (int r = 0; r < 4; ++r) s_old[r] = in.state[(size_t)(slot[r] >= 0 ? slot[r] : 0) * in.state_ld + c];
   const float br = in.gate_b[(size_t)b * 2 * in.bs + ch], bi = in.gate_b[(size_t)b * 2 * in.bs + in.bs + ch], rate = in.rate[c];
   // the filter: 8 channels of a sequence a thread, which also moves the kept inputs on
   for (int e = t; e < 16 * KS * 4; e += 2 * KS * DA_WAVE) {
     const int j = e / (KS * 4), c8 = (e % (KS * 4)) * 8;
     float acc[8] = {0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f, 0.f};
     if (c8 < in.bs && j0 + j < n) {
-      const int sl = in.slots[seq0 + j0 + j];
+      const int sl = in.slots[j0 + j];
       float xv[8], tail[KT - 1][8], w[KT][8];
-      lru_unpack8(load16(in.yx + (size_t)in.q_start[seq0 + j0 + j] * in.ld + in.C + c0 + c8), xv);
+      lru_unpack8(load16(in.yx + (size_t)(j0 + j) * in.ld + in.C + c0 + c8), xv);
       float* tp = in.state + (size_t)(sl >= 0 ? sl : 0) * in.state_ld + in.C + c0 + c8;
 #pragma unroll
       for (int k = 0; k < KT - 1; ++k) lru_load8(k < in.K - 1 ? tp + (size_t)k * in.C : tp - in.C, tail[k]);   // (or the row's S)
@@ -231,7 +231,7 @@ rglru_decode_kernel(LruIn in, int seq0, int n) {
     lru_step(ar[r] + br, ai[r] + bi, rate, bf16_to_f32(us[j][ch]), a, add);
     const float st = a * (slot[r] >= 0 ? s_old[r] : 0.f) + add;
     if (in.write && slot[r] >= 0) in.state[(size_t)slot[r] * in.state_ld + c] = st;
-    in.out[(size_t)row[r] * in.out_ld + c] = f32_to_bf16(st * apply_act_bf16(yv[r], in.act));
+    in.out[(size_t)(j0 + j) * in.out_ld + c] = f32_to_bf16(st * apply_act_bf16(yv[r], in.act));
   }
 }
 
@@ -437,18 +437,18 @@ static int lru_checks(const LruIn& in, const char* name) {
     else { if (in.K <= 4) GO(8, 4); else GO(8, 16); }                  \
   } while (0)
 
-// Sequences seq0 .. seq0 + n - 1 of the step, which bring one token each.
+// The step's first n sequences, which bring one token each: sequence j has row j.
 extern "C" int da_rglru_decode(const void* yx, int ld, const float* conv_w, const float* conv_b, const void* gate_w,
                                const float* gate_b, const float* rate, int act, float* state, long state_ld,
-                               const int* state_slots, const int* q_start, void* out, int out_ld, int seq0, int n, int C, int bs,
-                               int K, int write, void* stream) {
-  const LruIn in{(const bf16_t*)yx, ld, conv_w, conv_b, (const bf16_t*)gate_w, gate_b, rate, state, state_ld, state_slots, q_start,
+                               const int* state_slots, void* out, int out_ld, int n, int C, int bs, int K,
+                               int write, void* stream) {
+  const LruIn in{(const bf16_t*)yx, ld, conv_w, conv_b, (const bf16_t*)gate_w, gate_b, rate, state, state_ld, state_slots, nullptr,
                  (bf16_t*)out, out_ld, C, bs, K, act, write};
   if (lru_checks(in, "rglru_decode")) return 1;
-  DA_REQUIRE(seq0 >= 0 && n >= 0, "rglru_decode: bad sizes");
+  DA_REQUIRE(n >= 0, "rglru_decode: bad sizes");
   if (n == 0) return 0;
   const dim3 grid(C / bs, da_ceil_div(n, 16));
-#define LRU_GO(KS, KT) hipLaunchKernelGGL((rglru_decode_kernel<KS, KT>), grid, dim3(2 * KS * DA_WAVE), 0, (hipStream_t)stream, in, seq0, n)
+#define LRU_GO(KS, KT) hipLaunchKernelGGL((rglru_decode_kernel<KS, KT>), grid, dim3(2 * KS * DA_WAVE), 0, (hipStream_t)stream, in, n)
   LRU_PICK(LRU_GO);
 #undef LRU_GO
   DA_CHECK_LAUNCH("rglru_decode");

@@ -80,6 +80,8 @@ _ARGTYPES = {
     "da_layernorm": [_VP, _VP, _VP, _I, _VP, _I, _F, _VP, _I, _I, _I, _VP],
     "da_gemm_ref": [_VP, _I, _VP, _I, _I, _VP, _I, _I, _I, _VP, _I, _I, _I, _I, _I, _VP],
     "da_gemm_bf16": [_VP, _I, _VP, _I, _VP, _I, _I, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP, _I, _I, _I, _I, _I, _VP],
+    "da_gemm_few_rows": [_I, _I],
+    "da_gemm_bf16_kv_split": [_VP, _I, _VP, _I, _VP, _I, _VP, _I, _I, _I, _I, _VP, _VP, _I, _I, _I, _I, _I, _VP],
     "da_gemm_bf16_wide": [_VP, _I, _VP, _I, _VP, _I, _I, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP],
     "da_gemm_wide_choice": [_I, _I, _I],
     "da_gemm_bf16_ln": [_VP, _VP, _VP, _I, _VP, _I, _F, _VP, _I, _VP, _I, _I, _VP, _I, _I, _I, _I, _I, _VP, _VP,
@@ -161,7 +163,7 @@ _ARGTYPES = {
     "da_rglru_walk": [_VP, _I, _I, _VP, _I, _I, _VP, _VP, _I, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _VP],
     "da_rglru_serve_takes": [_I],
     "da_rglru_chunk_tokens": [],
-    "da_rglru_decode": [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _VP],
+    "da_rglru_decode": [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP, _I, _I, _I, _I, _I, _I, _VP],
     "da_rglru_portion": [_VP, _I, _VP, _VP, _VP, _VP, _VP, _I, _VP, ctypes.c_long, _VP, _VP, _VP, _I, _I, _I, _I, _I, _I, _I, _I,
                          _VP, ctypes.c_long, _VP],
 }
@@ -963,6 +965,33 @@ def linear(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: 
     return out
 
 
+def linear_kv_split(a: torch.Tensor, w: torch.Tensor, bias: Optional[torch.Tensor], out: torch.Tensor, cache_slot: torch.Tensor,
+                    slot_map: torch.Tensor, q_cols: int, n_kv_heads: int, head_dim: int, v_head_dim: int, page: int) -> torch.Tensor:
+    """out = a @ w.T + bias with columns q | k | v | rest, and keys (``head_dim`` a head) and values (``v_head_dim`` a head) in
+    their cache rows ``slot_map`` (see ``kv_write_split``): in the product's epilogue for few rows on the matrix cores, by the
+    write kernel otherwise."""
+    M, K = a.shape
+    N = w.shape[0]
+    if not (_MODE == "tuned" and out.dtype == torch.bfloat16 and _mfma_ok(a, w) and bool(_lib().da_gemm_few_rows(M, N))):
+        linear(a, w, bias, out)
+        if v_head_dim == head_dim and cache_slot.dim() == 5:
+            kv_write(out, q_cols, q_cols + n_kv_heads * head_dim, cache_slot, slot_map, n_kv_heads, head_dim)
+        else:
+            kv_write_split(out, q_cols, q_cols + n_kv_heads * head_dim, cache_slot, slot_map, n_kv_heads, head_dim, v_head_dim, page)
+        return out
+    _dev(a, w, bias, out, cache_slot, slot_map)
+    _rows_2d(a, "a"); _rows_2d(w, "w"); _rows_2d(out, "out")
+    _need(w.shape[1] == K and out.shape[0] == M and out.shape[1] == N and (bias is None or bias.numel() == N), "linear_kv_split: shapes differ")
+    _need(cache_slot.is_contiguous() and cache_slot.dtype == torch.bfloat16
+          and cache_page_elems(cache_slot) == n_kv_heads * page * (head_dim + v_head_dim) and slot_map.dtype == torch.int32
+          and slot_map.numel() >= M, "linear_kv_split: a page of the cache slot holds Hkv * page * (D + Dv) bfloat16 entries; slot_map int32 [rows]")
+    with _timed("product_skinny", _product_bytes(a, w, bias, out, False), 2 * M * N * K):
+        _check(_lib().da_gemm_bf16_kv_split(_ptr(a), a.stride(0), _ptr(w), w.stride(0), _ptr(bias), _dt(bias) if bias is not None else 0,
+                                            _ptr(out), out.stride(0), M, N, K, _ptr(cache_slot), _ptr(slot_map), q_cols, n_kv_heads,
+                                            head_dim, v_head_dim, page, _stream()))
+    return out
+
+
 def _attn_common(q, cache_slot, block_table, n_heads, out, name):
     _dev(q, cache_slot, block_table, out)
     _rows_2d(q, "q"); _rows_2d(out, "out")
@@ -1418,11 +1447,11 @@ def experts_forward(ctx, h: torch.Tensor, table: Optional[torch.Tensor], gate_up
     tile = MOE_TILE_ROWS_BLOCK if block else (MOE_TILE_ROWS_MFMA if mfma else MOE_TILE_ROWS)
     top = each
     tiles, rows = moe_slot_space(N, top, n_experts, tile)
-    ints = ctx.buf("moe_route", N * top + rows + tiles, 1, torch.int32).view(-1)
-    slot_of_pair, row_of_slot, tile_expert = ints[:N * top], ints[N * top:N * top + rows], ints[N * top + rows:]
+    slot_of_pair, row_of_slot, tile_expert = (ctx.flat("moe_slot_of_pair", N * top, torch.int32), ctx.flat("moe_row_of_slot", rows, torch.int32),
+                                              ctx.flat("moe_tile_expert", tiles, torch.int32))
     _need(not weight_input or pair_weights is not None, "experts: weights on the input need a weight a pair")
     # a pair's weight where its slot is: the first product scales its rows with it
-    slot_scale = ctx.buf("moe_slot_scale", rows, 1, torch.float32).view(-1) if weight_input else None
+    slot_scale = ctx.flat("moe_slot_scale", rows, torch.float32) if weight_input else None
     if choice is not None and not weight_input and bool(_lib().da_moe_choose_route_takes(N, choice.outputs, chosen, extra, routed)):
         inside = (choice.router is not None and mfma and choice.router.dtype == torch.bfloat16
                   and bool(_lib().da_moe_choose_route_takes_router(N, choice.outputs + (1 if extra else 0), width)))
@@ -1856,7 +1885,7 @@ def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tenso
     """The recurrence of a step in bfloat16 serving, from the rows ``yx`` [N, y: C | x: C] to out = S * act(y): the filter
     of x (``conv_w`` float32 [taps, C], the last row meets the token itself; ``conv_b`` float32 [C]), the blocks' two square
     matrices (``gate_w`` [blocks, 2 b, b], ``gate_b`` float32 [blocks, 2 b]: r's rows, then i's), and ``rglru_walk``'s
-    recurrence.  One-token sequences and portions go to a launch (or, for portions longer than a chunk, two) each.
+    recurrence.  One-token sequences (they lead the step, a row each) and portions go to a launch (or, for portions longer than a chunk, two) each.
     ``state`` [slots, taps * C]: S, then the filter's last inputs; both move on with ``write``."""
     _dev(yx, conv_w, conv_b, gate_w, gate_b, rate, state, out)
     _rows_2d(yx, "yx"); _rows_2d(out, "out")
@@ -1872,13 +1901,13 @@ def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tenso
 
     def args():
         return (_ptr(yx), yx.stride(0), _ptr(conv_w), _ptr(conv_b), _ptr(gate_w), _ptr(gate_b), _ptr(rate), ACTIVATIONS[act],
-                _ptr(state), ld, _ptr(ctx.state_slots), _ptr(ctx.q_start), _ptr(out), out.stride(0))
+                _ptr(state), ld, _ptr(ctx.state_slots))
 
     nd, S = ctx.n_decode, ctx.n_seqs
     weights = _nbytes(gate_w, gate_b, conv_w, conv_b, rate)
     if nd:
         with _timed("rglru_decode", nd * C * (3 * 2 + 2 * K * 4) + weights, nd * C * (4 * bs + 2 * K + 20), "bf16"):
-            _check(_lib().da_rglru_decode(*args(), 0, nd, C, bs, K, int(bool(write)), _stream()))
+            _check(_lib().da_rglru_decode(*args(), _ptr(out), out.stride(0), nd, C, bs, K, int(bool(write)), _stream()))
     if S > nd:
         longest = int(ctx.max_query_len)
         chunks = -(-longest // int(_lib().da_rglru_chunk_tokens()))
@@ -1886,7 +1915,7 @@ def rglru_serve(ctx, yx: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tenso
         if chunks > 1 or bs > 64:
             scratch = ctx.buf("rglru_scratch", (S - nd) * (2 * chunks + K), C, torch.float32)
         with _timed("rglru_portion", (N - nd) * C * 3 * 2 + (S - nd) * C * 2 * K * 4 + weights, (N - nd) * C * (4 * bs + 2 * K + 20), "bf16"):
-            _check(_lib().da_rglru_portion(*args(), nd, S - nd, C, bs, K, int(bool(write)), longest, _ptr(scratch),
+            _check(_lib().da_rglru_portion(*args(), _ptr(ctx.q_start), _ptr(out), out.stride(0), nd, S - nd, C, bs, K, int(bool(write)), longest, _ptr(scratch),
                                            0 if scratch is None else scratch.numel(), _stream()))
     return out
 

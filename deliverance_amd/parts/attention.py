@@ -237,6 +237,10 @@ class CausalSelfAttention(Mixer):
             ops.linear(h, self.qkv_weight, self.qkv_bias, raw)
             self._attend(ctx, self._prepare(ctx, raw, slot, group, call), x, slot, group, call, gate_off=self.q_cols)
             return
+        elif self.position is None and call.write:
+            # nothing turns, but values of their own size or a gate behind them: keys and values are kept as they come
+            ops.linear_kv_split(h, self.qkv_weight, self.qkv_bias, qkv, slot, ctx.slot_maps[group], self.q_cols, self.n_kv_heads,
+                                self.head_dim, self.v_head_dim, ctx.cache.page_size)
         else:
             ops.linear(h, self.qkv_weight, self.qkv_bias, qkv)
             self._turn_and_keep(ctx, qkv, slot, group, call)

@@ -131,6 +131,10 @@ class StepContext:
         """A scratch matrix [rows, cols] that lives until the step ends."""
         return self._arena.get(name, rows, cols, dtype)
 
+    def flat(self, name: str, n: int, dtype: torch.dtype) -> torch.Tensor:
+        """A scratch vector of n entries, likewise."""
+        return self._arena.flat(name, n, dtype)
+
     def group_of(self, cache_slot: int) -> int:
         return self.cache.group_of_slot[cache_slot]
 
@@ -141,20 +145,39 @@ class StepContext:
 
 
 class Arena:
-    """Named scratch buffers reused from step to step (no allocation in steady state)."""
+    """Named scratch buffers reused from step to step (no allocation in steady state).  The view that was handed out last
+    is kept: a step of the same rows gets it back without making another."""
 
     def __init__(self, device):
         self.device = device
         self._bufs: Dict[tuple, torch.Tensor] = {}
+        self._views: Dict[tuple, torch.Tensor] = {}
+        self._flats: Dict[tuple, list] = {}
 
     def get(self, name, rows, cols, dtype):
         key = (name, cols, dtype)
+        v = self._views.get(key)
+        if v is not None and v.shape[0] == rows:
+            return v
         t = self._bufs.get(key)
         if t is None or t.shape[0] < rows:
             cap = max(rows, 16) if t is None else max(rows, 2 * t.shape[0])
             t = torch.empty((cap, cols), dtype=dtype, device=self.device)
             self._bufs[key] = t
-        return t[:rows]
+        v = self._views[key] = t[:rows]
+        return v
+
+    def flat(self, name, n, dtype):
+        """A vector of n entries, likewise."""
+        key = (name, dtype)
+        entry = self._flats.get(key)
+        if entry is None or entry[0].shape[0] < n:
+            cap = max(n, 256) if entry is None else max(n, 2 * entry[0].shape[0])
+            t = torch.empty((cap,), dtype=dtype, device=self.device)
+            entry = self._flats[key] = [t, t[:n]]
+        elif entry[1].shape[0] != n:
+            entry[1] = entry[0][:n]
+        return entry[1]
 
 
 @dataclass(frozen=True)

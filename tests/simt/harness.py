@@ -257,6 +257,9 @@ def make_arena(sim: Sim):
                 self._bufs[key] = t
             return t
 
+        def flat(self, name, n, dtype):
+            return self.get(name, n, 1, dtype).view(-1)
+
     return SimArena()
 
 
