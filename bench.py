@@ -869,7 +869,7 @@ def main():
     ap.add_argument("--no-extra", action="store_true", help="skip the GPT-2 1.5B points and the 355M mixed workload")
     ap.add_argument("--profile-stages", action="store_true", help="also print a per-kernel table with roofline fractions (stderr)")
     ap.add_argument("--page-size", type=int, default=16, choices=[16, 32, 64], help="tokens a cache page")
-    ap.add_argument("--prefill-shape", default="2x1024", help="prompts x tokens of the prefill step (the contract's: 2x1024)")
+    ap.add_argument("--prefill-shape", default="2x1024", help="prompts x tokens of the prefill step (default: 2x1024)")
     ap.add_argument("--step-tokens", type=int, default=512 + 64,
                     help="mixed workload: the most tokens a step holds, decoded tokens and a prompt portion together (default: a portion of 512 beside 64 decoded tokens)")
     ap.add_argument("--pool-tokens", type=int, default=None,

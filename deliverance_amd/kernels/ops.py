@@ -1875,6 +1875,14 @@ def rglru_walk(ctx, u: torch.Tensor, raw: torch.Tensor, block: int, rate: torch.
     return out
 
 
+RGLRU_MAX_BLOCK = 256        # channels of a block that the forms for serving take (csrc/rglru.hip)
+
+
+def rglru_block_fits(block: int) -> bool:
+    """What those forms ask of a block's channels (without loading a kernel library)."""
+    return block % 8 == 0 and block <= RGLRU_MAX_BLOCK
+
+
 def rglru_serve_takes(yx: torch.Tensor, block: int) -> bool:
     """Whether the forms for bfloat16 serving take blocks of so many channels (and the kernel mode allows them)."""
     return _MODE == "tuned" and yx.dtype == torch.bfloat16 and bool(_lib().da_rglru_serve_takes(int(block)))

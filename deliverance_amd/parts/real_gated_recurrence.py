@@ -57,7 +57,7 @@ class RealGatedRecurrence(Mixer):
         self.conv_off = C                            # where the filter's inputs start in a state row
 
     def kernel_units(self, dtype):
-        return ("rglru", "ssm")
+        return ("rglru",) if dtype == torch.bfloat16 and ops.rglru_block_fits(self.block) else ("rglru", "ssm")
 
     def cache_need(self):
         return StateNeed(self.channels * self.taps)

@@ -125,3 +125,18 @@ def test_trace_run_without_a_gpu_says_so(tmp_path):
     p = subprocess.run([sys.executable, os.path.join(ROOT, "bin", "trace_run"), "--model", str(tmp_path), "--dtype", "float32",
                         "--out", str(tmp_path / "o"), "--max-tokens", "64"], input="", capture_output=True, text=True, timeout=300)
     assert p.returncode != 0 and "no GPU is visible" in p.stderr and "Traceback" not in p.stderr
+
+
+def test_random_then_inspect_a_design_that_runs_layers_again(tmp_path):
+    """... and on a Mogevik configuration: a layer of the loop has one set of tensors and a slot for every pass."""
+    from mogevik_models import CONFIG_D
+    cfg = tmp_path / "config.json"
+    cfg.write_text(json.dumps(CONFIG_D))
+    out = tmp_path / "model"
+    p = run("random", "--config", str(cfg), "--seed", "9", "--out", str(out))
+    assert p.returncode == 0, p.stderr
+    p = run("inspect", str(out))
+    assert p.returncode == 0, p.stderr
+    assert f"architecture Mogevik: 4 layers, width {CONFIG_D['width']}, vocabulary {CONFIG_D['vocab']}" in p.stdout
+    assert "8 layer calls, 8 cache slots" in p.stdout
+    assert "loop.step" in p.stdout and "l0.mix.ra.b" in p.stdout and "l1.mix.v.b" in p.stdout and "l0.mlp.shared.sg" in p.stdout

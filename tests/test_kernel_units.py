@@ -58,6 +58,7 @@ def test_models_name_units_that_exist(tmp_path):
     from deliverance_amd.models.causal_lm import load_model
     from deliverance_amd.random_model import random_model
     from luvatar_models import CONFIG_A
+    from mogevik_models import CONFIG_D, CONFIG_E
     from pafolorn_models import CONFIG_F
     from pedatar_models import CONFIG_P
     from salivik_models import CONFIG_S
@@ -65,7 +66,7 @@ def test_models_name_units_that_exist(tmp_path):
     names = set(build.units())
     of = {}
     for key, cfg in (("gpt2", helpers.CONFIG_A), ("virudra", CONFIG_X), ("pedatar", CONFIG_P), ("pafolorn", CONFIG_F),
-                     ("salivik", CONFIG_S), ("luvatar", CONFIG_A)):
+                     ("salivik", CONFIG_S), ("luvatar", CONFIG_A), ("mogevik", CONFIG_D), ("mogevik_plain", CONFIG_E)):
         folder = str(tmp_path / key)
         random_model(folder, cfg, 1)
         for dtype in (torch.bfloat16, torch.float32):
@@ -74,3 +75,9 @@ def test_models_name_units_that_exist(tmp_path):
     lu = of["luvatar", torch.bfloat16]
     assert {"gla", "attn_window", "attn_prepare"} <= lu and not lu & {"moe", "ssm", "retention", "attn_latent", "attn_prefill", "gemm_ref"}
     assert "gla" not in of["gpt2", torch.bfloat16] and "gemm_mfma" not in of["luvatar", torch.float32]
+    mo = of["mogevik", torch.bfloat16]
+    assert {"rglru", "moe", "attn_window", "elementwise"} <= mo and not mo & {"ssm", "gla", "attn_prepare", "norm_rms", "gemm_ref", "attn_latent"}
+    assert {"rglru", "ssm"} <= of["mogevik_plain", torch.bfloat16] and {"rglru", "ssm", "attn_rel"} <= of["mogevik", torch.float32]
+    from deliverance_amd.kernels import ops
+    if build.is_built():
+        assert all(bool(ops._lib().da_rglru_serve_takes(n)) == ops.rglru_block_fits(n) for n in range(1, 300))

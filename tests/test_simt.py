@@ -59,6 +59,11 @@ RUNS = {
                ["tests/test_luvatar_gpu.py", "-n", "3", "-m", QUICK, "-k",
                 "not float32 and not (portions and (sizes0 or A)) and not token_by_token and not (mixed_batches and (A or C)) "
                 "and not (edge and True and not 56)"],
+    # a seventh design's kernels and parts (a recurrence with one number a channel, attention with slopes by distance, the
+    # choice of experts inside groups) and its models through the step function
+    "mogevik": ["tests/test_mogevik_gpu.py", "-n", "4"] if FULL else
+               ["tests/test_mogevik_gpu.py", "-n", "3", "-m", QUICK, "-k",
+                "not float32 and not (portions and (sizes0 or D)) and not token_by_token and not mixed_batches and not (edge and 16-48)"],
     "replay": ["tests/test_replay_gpu.py", "-n", "4"] if FULL else
               ["tests/test_replay_gpu.py", "-n", "2", "-k", "(mixed and (A or B) and not 32) or want_subset or errors_leave or first_tokens"],
     # inner sizes of 32 in an engine step: qkv and fc of seed 11 (and, in the full run, proj of seed 5)
